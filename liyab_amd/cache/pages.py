@@ -18,7 +18,7 @@ lives in `CacheStorage`.
 from __future__ import annotations
 
 import ctypes
-from dataclasses import dataclass
+from dataclasses import dataclass, replace
 from typing import Dict, Hashable, List, Sequence, Tuple
 
 import numpy as np
@@ -52,6 +52,7 @@ class KVSpec:
     head_dim: int
     window: int = 0  # 0: every position is kept; W > 0: only the last W are read
     rows: Tuple[Tuple[str, int, int], ...] = ()
+    keep_first: int = 0  # with a window: the first `keep_first` positions are read too, however far back
 
     @property
     def planes(self) -> Tuple[Tuple[str, int, int], ...]:
@@ -60,7 +61,15 @@ class KVSpec:
     @property
     def key(self) -> tuple:
         """Layers with equal keys share a group: the same pages, one block table a request."""
-        return (self.planes, self.window)
+        return (self.planes, self.window, self.keep_first if self.window > 0 else 0)
+
+    def covering(self, other: "KVSpec") -> "KVSpec":
+        """What a layer's pages must hold when another layer reads them too: every position either one reads."""
+        if self.planes != other.planes:
+            raise InvalidArgument(f"a layer that reads another's cache needs its rows: {other.planes} of {self.planes}")
+        if self.window <= 0 or other.window <= 0:
+            return replace(self, window=0, keep_first=0)
+        return replace(self, window=max(self.window, other.window), keep_first=max(self.keep_first, other.keep_first))
 
 
 @dataclass(frozen=True)
@@ -165,7 +174,8 @@ class CacheManager:
             raise InvalidArgument(f"{len(group_specs)} cache groups; at most {host.MAX_GROUPS} are taken")
         self._lib = host.lib()
         windows = _ints([spec.window for spec, _ in group_specs])
-        self._h = self._lib.liyab_cm_create(len(group_specs), _ip(windows), _ip(_ints(counts)), page_size, max_requests,
+        kept = _ints([spec.keep_first for spec, _ in group_specs])
+        self._h = self._lib.liyab_cm_create(len(group_specs), _ip(windows), _ip(kept), _ip(_ints(counts)), page_size, max_requests,
                                             max_positions)
         if not self._h:
             raise InvalidArgument(self._lib.liyab_host_last_error().decode())
@@ -265,7 +275,8 @@ class CacheManager:
     def commit(self, rid: Hashable, new_length: int) -> None:
         """The request now holds `new_length` positions. Windowed groups give
         back the pages no later query can see: a query at position p >= length
-        reads [p - W + 1, p], so pages wholly below length - W + 1 go."""
+        reads [p - W + 1, p], so pages wholly below length - W + 1 go, but for the pages of a
+        group's first positions where it keeps them (`keep_first`)."""
         host.check(self._lib.liyab_cm_commit(self._h, self._slots[rid], new_length))
 
     def commit_slots(self, slots: np.ndarray, new_lengths: np.ndarray) -> None:

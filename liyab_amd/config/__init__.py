@@ -29,3 +29,4 @@ from .bokulix import BokulixConfig  # noqa: F401  (registers itself)
 from .mofulix import MofulixConfig  # noqa: F401  (registers itself)
 from .dopilorn import DopilornConfig  # noqa: F401  (registers itself)
 from .larulorn import LarulornConfig  # noqa: F401  (registers itself)
+from .lolulorn import LolulornConfig  # noqa: F401  (registers itself)

@@ -134,7 +134,8 @@ class RoutedFFNSpec:
     neighbours, a group's score is its largest, and only experts of the `keep` best groups can be chosen; the
     weights are the chosen scores divided by their sum. `shared_inner` > 0: one more expert of the same form
     and that inner width runs for every token with weight one (tensors shared_up, shared_down, and shared_gate
-    if gated)."""
+    if gated). `scores` "logistic": s = sigmoid(z); the choice goes by s + correction (tensor `correction`, optional), with `groups` a
+    group's score is the sum of its two largest such values, and the weights are the chosen s as they are."""
 
     kind: str  # "routed_ffn"
     width: int
@@ -146,6 +147,7 @@ class RoutedFFNSpec:
     gated: bool = True
     groups: Optional[tuple] = None  # (count, keep)
     shared_inner: int = 0
+    scores: str = "softmax"  # | "logistic"
 
 
 @dataclass(frozen=True)
@@ -176,7 +178,7 @@ class RotarySpec:
     `halves`: the pairs are (i, i + dims / 2) instead. `ramp` (factor, fast, slow, original): the other way of stretching, by the
     entry's number: with at(t) = dims ln(original / (2 pi t)) / (2 ln base), lo = max(floor(at(fast)), 0), hi = min(ceil(at(slow)),
     dims - 1) and r_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1), f_i becomes f_i / factor * r_i + f_i (1 - r_i), and cosine and
-    sine are multiplied by `ramp_magnitude` * ln(factor) + 1."""
+    sine are multiplied by `ramp_magnitude` * ln(factor) + 1. `linear`: every f_i divided by it."""
 
     dims: int
     base: float
@@ -184,6 +186,7 @@ class RotarySpec:
     halves: bool = False
     ramp: Optional[tuple] = None  # (factor, fast, slow, original)
     ramp_magnitude: float = 0.1
+    linear: float = 1.0
 
 
 @dataclass(frozen=True)
@@ -198,7 +201,9 @@ class ScoredAttentionSpec:
     the three projections (`biased`), a learned logit a head that joins the softmax's denominator with no key and no value
     (`sink`), values shared between layers (`value_mix`: "first" = this layer's values, as projected, are kept for the later
     layers of the same step; "later" = v <- (1 - lam) v + lam v_first with the learned scalar `vmix`, and the mixed values are
-    what is cached)."""
+    what is cached). `qk_norm_rows`: a root-mean-square norm of a token's whole queries (and whole keys) before they are heads, a
+    weight an entry (tensors q_norm, k_norm). With a `window`, positions below `keep_first` stay visible. `kv_shared`: the keys and
+    values are another layer's, as its cache holds them (the run order's `cache_of`, writes_cache False); the layer has queries only."""
 
     kind: str  # "scored_attention"
     width: int
@@ -221,6 +226,9 @@ class ScoredAttentionSpec:
     biased: bool = False
     sink: bool = False
     value_mix: str = ""  # "" | "first" | "later"
+    qk_norm_rows: bool = False
+    keep_first: int = 0
+    kv_shared: bool = False
 
 
 @dataclass(frozen=True)
@@ -324,6 +332,56 @@ class DeltaRuleSpec:
 
 
 @dataclass(frozen=True)
+class GatedDeltaSpec:
+    """A delta rule whose state decays by one number a head and token, behind a short convolution: q, k, v = silu(conv(W h)) a channel
+    over time (`taps` inputs, no bias; the last inputs are part of a request's state); q and k of a head to length one (key_eps under
+    the root), q times q_scale; beta = sigmoid(Wb h), g = exp(-exp(A_log) softplus(Wa h + dt_bias)) a head; S <- g S, S <- S + k (beta (v
+    - S^T k))^T, o = S^T q; each head's o brought to unit root mean square, times a weight shared by the heads and silu(Wg h), then
+    the output projection. Heads share q and k in `n_kv_head` groups."""
+
+    kind: str  # "gated_delta"
+    width: int
+    n_head: int
+    n_kv_head: int
+    head_dim: int
+    value_dim: int
+    taps: int
+    eps: float
+    q_scale: float
+    key_eps: float = 1e-6
+    tensors: dict = field(default_factory=dict)  # q, k, v, q_conv, k_conv, v_conv, b, a, A_log, dt_bias, g, norm, out
+
+
+@dataclass(frozen=True)
+class GatedLinearAttentionSpec:
+    """A mixer that carries a matrix of state a head under a decay a key channel: q = Wq h q_scale, k, v = W h; w = sigmoid(W2 (W1 h) +
+    b)^(1 / tau) (`decay_rank` wide in between); S <- diag(w) S + k v^T, o = S^T q; each head's o brought to unit root mean square, times
+    a weight shared by the heads and silu(Wg h), then the output projection."""
+
+    kind: str  # "gated_linear_attention"
+    width: int
+    n_head: int
+    head_dim: int
+    value_dim: int
+    decay_rank: int
+    tau: float
+    eps: float
+    q_scale: float
+    tensors: dict = field(default_factory=dict)  # q, k, v, g, w1, w2, w2_bias, norm, out
+
+
+@dataclass(frozen=True)
+class GatedFFNSpec:
+    """A gated feed-forward, down(act(gate h) * (up h)), act "silu" or "gelu_tanh"."""
+
+    kind: str  # "gated_ffn"
+    width: int
+    inner: int
+    activation: str
+    tensors: dict = field(default_factory=dict)  # gate, up, down
+
+
+@dataclass(frozen=True)
 class DifferentialAttentionSpec:
     """Attention in two maps a head that share their values: queries and keys hold [map 1 | map 2] a head, each map an
     ordinary softmax attention under the window, and a head's result is o = a1 - lam * a2 with lam = exp(lq1 . lk1) -
@@ -378,7 +436,7 @@ class LayerSpec:
     arrangement "pre_norm": x += mixer(norm_mixer(x)); x += ffn(norm_ffn(x)).
     arrangement "parallel": h = norm_mixer(x); x += mixer(h) + ffn(h): one norm, both sublayers read its output.
     arrangement "post_norm_gated": x += norm_mixer(gate_mixer * mixer(conv(x))); x += norm_ffn(gate_ffn *
-    ffn(x)): the sublayers read the stream itself, the norms stand on their results; `input_conv`
+    ffn(x)): the sublayers read the stream itself, the norms (root-mean-square or layer norms) stand on their results; `input_conv`
     (what the mixer reads is first convolved over time) and the gates are optional.
     arrangement "parallel_pair": x += mixer(c1(norm_mixer(x))) + ffn(c2(norm_ffn(x))): two norms of the same x, each
     followed by a convolution over time of its own (`input_conv`, `ffn_conv`: h <- h + conv(h); optional).

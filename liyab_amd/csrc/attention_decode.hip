@@ -84,7 +84,8 @@ __device__ __forceinline__ void add_sink(float& m, float& l, float (&acc)[N], fl
 
 // SCORED: the score scale * q . k is worked on before the softmax: a soft cap, cap * tanh(score / cap) (softcap > 0), then
 // a bias by distance, bias_table[min(position - key, max_dist), head] (bias_table given); `sinks` (one logit a head) join the
-// softmax's denominator where the row's sums are final. Without SCORED these arguments are not read, and the kernel is the one it was.
+// softmax's denominator where the row's sums are final; with a window, the first `keep_first` positions may stay visible: the
+// walk goes over places first - kept .. position, of which those ahead of `first` are positions 0 .. kept - 1. Without SCORED these arguments are not read, and the kernel is the one it was.
 template <typename T, int LPK, int AD_WAVES, int AD_U, bool SCORED = false>
 __global__ void __launch_bounds__(64 * AD_WAVES)
 attention_decode_kernel(T* __restrict__ out, int64_t out_stride, const T* __restrict__ q, int64_t q_stride,
@@ -93,7 +94,8 @@ attention_decode_kernel(T* __restrict__ out, int64_t out_stride, const T* __rest
                         const int* __restrict__ tok_seq, const int* __restrict__ tok_pos, float scale, int window,
                         int n_head, int n_kv_head, int hd, int page_size, int page_shift, int rows_are_requests,
                         int n_splits, int chunk, float* __restrict__ partials, int num_pages, float softcap = 0.0f,
-                        const float* __restrict__ bias_table = nullptr, int max_dist = 0, const float* __restrict__ sinks = nullptr) {
+                        const float* __restrict__ bias_table = nullptr, int max_dist = 0, const float* __restrict__ sinks = nullptr,
+                        int keep_first = 0) {
     constexpr int KPP = 64 / LPK;  // keys per wave and pass
     __shared__ float lds2[2][AD_WAVES][LPK][10];  // the waves' sums, for the first wave to merge; two of them in turn, so that one barrier a split is enough
     const int t = tok_list != nullptr ? tok_list[blockIdx.x] : blockIdx.x;
@@ -122,7 +124,8 @@ attention_decode_kernel(T* __restrict__ out, int64_t out_stride, const T* __rest
         for (int e = 0; e < 8; ++e) qf[e] = 0.0f;
     }
     __syncthreads();
-    const int first = window > 0 ? max(0, pos - window + 1) : 0;
+    const int first_seen = window > 0 ? max(0, pos - window + 1) : 0;  // the window's first position
+    const int first = SCORED ? first_seen - min(keep_first, first_seen) : first_seen;  // the walk's first place
     const int n_keys = pos - first + 1;
     // Splits by position launched as one (chunk > 0, n_splits == 1): the workgroup walks the token's
     // splits one after the other, keeps each one's sums apart and merges them at the end as the merge
@@ -152,7 +155,8 @@ attention_decode_kernel(T* __restrict__ out, int64_t out_stride, const T* __rest
         for (int u = 0; u < AD_U; ++u) {
             const int j = j0 + u * AD_WAVES * KPP + kg;
             valid[u] = j < k_end;
-            const int jc = valid[u] ? j : pos;  // a mapped position; its values are not used
+            int jc = valid[u] ? j : pos;  // a mapped position; its values are not used
+            if constexpr (SCORED) jc = jc < first_seen ? jc - first : jc;
             // no branch around the loads: a load under a branch is waited for where the branch ends
             const int lp = page_shift >= 0 ? jc >> page_shift : jc / page_size;
             const int off = page_shift >= 0 ? jc & (page_size - 1) : jc % page_size;
@@ -174,8 +178,10 @@ attention_decode_kernel(T* __restrict__ out, int64_t out_stride, const T* __rest
             if constexpr (SCORED) {
                 if (valid[u]) {
                     if (softcap > 0.0f) s[u] = softcap * tanhf(s[u] / softcap);
-                    if (bias_table != nullptr)
-                        s[u] += bias_table[static_cast<int64_t>(min(pos - (j0 + u * AD_WAVES * KPP + kg), max_dist)) * n_head + h];
+                    if (bias_table != nullptr) {
+                        const int place = j0 + u * AD_WAVES * KPP + kg;
+                        s[u] += bias_table[static_cast<int64_t>(min(pos - (place < first_seen ? place - first : place), max_dist)) * n_head + h];
+                    }
                 }
             }
             m_new = fmaxf(m_new, s[u]);
@@ -327,7 +333,7 @@ int launch_attention_decode(void* out, int64_t out_stride, const void* q, int64_
                             const int* tok_pos, int n, float scale, int window, int n_head, int n_kv_head, int hd,
                             int page_size, int n_splits, int chunk, int waves, int rows_are_requests, float* partials,
                             int leave_splits, int num_pages, hipStream_t stream, float softcap = 0.0f, const float* bias_table = nullptr,
-                            int max_dist = 0, const float* sinks = nullptr) {
+                            int max_dist = 0, const float* sinks = nullptr, int keep_first = 0) {
     int page_shift = -1;
     for (int b = 0; b < 31; ++b)
         if ((1 << b) == page_size) page_shift = b;
@@ -341,15 +347,15 @@ int launch_attention_decode(void* out, int64_t out_stride, const void* q, int64_
         if (waves == 4)                                                                                              \
             attention_decode_kernel<T, L, 4, 4, SCORED><<<grid, 256, 0, stream>>>(o, out_stride, pq, q_stride, pk, pv, block_tables, \
                                                                     max_blocks, tok_list, tok_seq, tok_pos, scale,   \
-                                                                    window, n_head, n_kv_head, hd, page_size, page_shift, rows_are_requests, n_splits, chunk, partials, num_pages, softcap, bias_table, max_dist, sinks); \
+                                                                    window, n_head, n_kv_head, hd, page_size, page_shift, rows_are_requests, n_splits, chunk, partials, num_pages, softcap, bias_table, max_dist, sinks, keep_first); \
         else if (waves == 8)                                                                                         \
             attention_decode_kernel<T, L, 8, 4, SCORED><<<grid, 512, 0, stream>>>(o, out_stride, pq, q_stride, pk, pv, block_tables, \
                                                                     max_blocks, tok_list, tok_seq, tok_pos, scale,   \
-                                                                    window, n_head, n_kv_head, hd, page_size, page_shift, rows_are_requests, n_splits, chunk, partials, num_pages, softcap, bias_table, max_dist, sinks); \
+                                                                    window, n_head, n_kv_head, hd, page_size, page_shift, rows_are_requests, n_splits, chunk, partials, num_pages, softcap, bias_table, max_dist, sinks, keep_first); \
         else                                                                                                         \
             attention_decode_kernel<T, L, 16, sizeof(T) == 2 ? 8 : 4, SCORED><<<grid, 1024, 0, stream>>>(o, out_stride, pq, q_stride, pk, pv, block_tables, \
                                                                       max_blocks, tok_list, tok_seq, tok_pos, scale, \
-                                                                      window, n_head, n_kv_head, hd, page_size, page_shift, rows_are_requests, n_splits, chunk, partials, num_pages, softcap, bias_table, max_dist, sinks); \
+                                                                      window, n_head, n_kv_head, hd, page_size, page_shift, rows_are_requests, n_splits, chunk, partials, num_pages, softcap, bias_table, max_dist, sinks, keep_first); \
     } while (0)
     if (hd <= 8) LIYAB_GO(1);
     else if (hd <= 16) LIYAB_GO(2);
@@ -381,8 +387,7 @@ using namespace liyab;
 static int check_attention_decode(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* kc, const void* vc, int dtype,
                                   const int* block_tables, int max_blocks, const int* tok_list, const int* tok_seq, const int* tok_pos, int n,
                                   int window, int n_head, int n_kv_head, int hd, int page_size, int n_splits, int chunk, int waves,
-                                  int rows_are_requests, float* partials, int leave_splits, int num_pages) {
-
+                                  int rows_are_requests, float* partials, int leave_splits, int num_pages, int keep_first) {
     LIYAB_REQUIRE(num_pages > 0, "attention_decode: the caches hold %d pages", num_pages);
     LIYAB_REQUIRE((out || leave_splits) && q && kc && vc && block_tables && tok_seq && tok_pos, "attention_decode: null pointer");
     LIYAB_REQUIRE(dtype == kBF16 || dtype == kF32, "attention_decode: unknown dtype %d", dtype);
@@ -398,9 +403,9 @@ static int check_attention_decode(void* out, int64_t out_stride, const void* q, 
                   "attention_decode: row strides are shorter than heads x head size");
     LIYAB_REQUIRE(n_splits >= 1 && n_splits <= 64 && (n_splits == 1 || partials != nullptr), "attention_decode: bad split count %d", n_splits);
     LIYAB_REQUIRE(window >= 0 && n_head <= 65535, "attention_decode: bad window or head count");
-    LIYAB_REQUIRE(chunk >= 0, "attention_decode: a negative number of keys a split");
+    LIYAB_REQUIRE(chunk >= 0 && keep_first >= 0, "attention_decode: a negative number of keys a split, or of kept positions");
     LIYAB_REQUIRE(chunk == 0 || n_splits > 1 || static_cast<int64_t>(chunk) * AD_LOOP_CHUNKS >= static_cast<int64_t>(max_blocks) * page_size ||
-                      (window > 0 && static_cast<int64_t>(chunk) * AD_LOOP_CHUNKS >= window),
+                      (window > 0 && static_cast<int64_t>(chunk) * AD_LOOP_CHUNKS >= static_cast<int64_t>(window) + keep_first),
                   "attention_decode: one workgroup walks at most %d splits of %d keys; contexts of %lld need a launch in splits", AD_LOOP_CHUNKS,
                   chunk, static_cast<long long>(max_blocks) * page_size);
     LIYAB_REQUIRE(max_blocks <= AD_MAX_BLOCKS, "attention_decode: block tables of %d pages; at most %d are taken", max_blocks, AD_MAX_BLOCKS);
@@ -415,7 +420,7 @@ extern "C" int liyab_attention_decode(void* out, int64_t out_stride, const void*
                                       int n_head, int n_kv_head, int hd, int page_size, int n_splits, int chunk, int waves,
                                       int rows_are_requests, float* partials, int leave_splits, int num_pages, hipStream_t stream) {
     if (int rc = check_attention_decode(out, out_stride, q, q_stride, kc, vc, dtype, block_tables, max_blocks, tok_list, tok_seq, tok_pos, n, window,
-                                        n_head, n_kv_head, hd, page_size, n_splits, chunk, waves, rows_are_requests, partials, leave_splits, num_pages))
+                                        n_head, n_kv_head, hd, page_size, n_splits, chunk, waves, rows_are_requests, partials, leave_splits, num_pages, 0))
         return rc;
     if (n == 0) return 0;
     if (dtype == kF32)
@@ -429,15 +434,15 @@ extern "C" int liyab_attention_decode(void* out, int64_t out_stride, const void*
 
 // The same with the scores worked on before the softmax: softcap > 0 caps them, cap * tanh(score / cap); bias_table (float
 // [max_dist + 1, n_head]) adds table[min(position - key, max_dist), head]; sinks (float [n_head], or null): exp(sinks[head])
-// is added to the softmax's denominator.
+// is added to the softmax's denominator; keep_first: positions below it stay visible behind the window.
 extern "C" int liyab_attention_decode_scored(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* kc,
                                              const void* vc, int dtype, const int* block_tables, int max_blocks, const int* tok_list,
                                              const int* tok_seq, const int* tok_pos, int n, float scale, int window,
                                              int n_head, int n_kv_head, int hd, int page_size, int n_splits, int chunk, int waves,
                                              int rows_are_requests, float* partials, int leave_splits, int num_pages, float softcap,
-                                             const float* bias_table, int max_dist, const float* sinks, hipStream_t stream) {
+                                             const float* bias_table, int max_dist, const float* sinks, int keep_first, hipStream_t stream) {
     if (int rc = check_attention_decode(out, out_stride, q, q_stride, kc, vc, dtype, block_tables, max_blocks, tok_list, tok_seq, tok_pos, n, window,
-                                        n_head, n_kv_head, hd, page_size, n_splits, chunk, waves, rows_are_requests, partials, leave_splits, num_pages))
+                                        n_head, n_kv_head, hd, page_size, n_splits, chunk, waves, rows_are_requests, partials, leave_splits, num_pages, keep_first))
         return rc;
     LIYAB_REQUIRE(softcap >= 0.0f && (bias_table == nullptr || max_dist >= 0), "attention_decode_scored: a negative cap or distance");
     LIYAB_REQUIRE(sinks == nullptr || !leave_splits, "attention_decode_scored: splits left unmerged take no sink");
@@ -445,10 +450,10 @@ extern "C" int liyab_attention_decode_scored(void* out, int64_t out_stride, cons
     if (dtype == kF32)
         return launch_attention_decode<float, true>(out, out_stride, q, q_stride, kc, vc, block_tables, max_blocks, tok_list, tok_seq,
                                                     tok_pos, n, scale, window, n_head, n_kv_head, hd, page_size, n_splits, chunk, waves,
-                                                    rows_are_requests, partials, leave_splits, num_pages, stream, softcap, bias_table, max_dist, sinks);
+                                                    rows_are_requests, partials, leave_splits, num_pages, stream, softcap, bias_table, max_dist, sinks, keep_first);
     return launch_attention_decode<bf16_t, true>(out, out_stride, q, q_stride, kc, vc, block_tables, max_blocks, tok_list, tok_seq,
                                                  tok_pos, n, scale, window, n_head, n_kv_head, hd, page_size, n_splits, chunk, waves,
-                                                 rows_are_requests, partials, leave_splits, num_pages, stream, softcap, bias_table, max_dist, sinks);
+                                                 rows_are_requests, partials, leave_splits, num_pages, stream, softcap, bias_table, max_dist, sinks, keep_first);
 }
 
 // out[m, h * hd + e] = the splits of (m, h) merged in split order: for splits that

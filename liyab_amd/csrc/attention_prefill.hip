@@ -61,7 +61,9 @@ constexpr int AP_MAX_BLOCKS = 2048;  // page ids of a tile's keys are kept in LD
 
 // SCORED: the scores are worked on before the softmax: scale * q . k, capped as cap * tanh(. / cap) when softcap > 0, plus
 // bias_table[min(query position - key position, max_dist), head] when a table is given; the exponentials then take the
-// scores as they are; `sinks` (one logit a head) join the denominator once the row's sums are final. Without SCORED these
+// scores as they are; `sinks` (one logit a head) join the denominator once the row's sums are final; with a window, positions
+// below `keep_first` stay visible: where the window has left them behind, the walk takes their steps first and goes on at the
+// window's first block (its steps are counted from `kb0v`, which lies as many steps ahead of that block). Without SCORED these
 // arguments are not read, and the kernel is the one it was.
 template <int DB, int QG, int KS, int NS = 1, bool SCORED = false>  // head dimension padded to 32 * DB; 32 * QG queries a tile; KS x NS blocks of keys a step, NS a wave
 __global__ void __launch_bounds__(64 * QG * KS)
@@ -70,7 +72,7 @@ attention_prefill_kernel(bf16_t* __restrict__ out, int64_t out_stride, const bf1
                          const int* __restrict__ block_tables, int max_blocks, const int* __restrict__ work, float scale,
                          int window, int n_head, int n_kv_head, int hd, int page_size, int page_shift, int num_pages,
                          float softcap = 0.0f, const float* __restrict__ bias_table = nullptr, int max_dist = 0,
-                         const float* __restrict__ sinks = nullptr) {
+                         const float* __restrict__ sinks = nullptr, int keep_first = 0) {
     constexpr int HDP = 32 * DB;
     constexpr int LDK = HDP + 8;  // padded row: 16-byte reads of 16 lanes fall in distinct banks
     constexpr int WAVES = QG * KS, THREADS = 64 * WAVES;
@@ -134,10 +136,25 @@ attention_prefill_kernel(bf16_t* __restrict__ out, int64_t out_stride, const bf1
     }
 
     const int k_hi = pos0 + nq - 1;  // last key any query of the tile sees
-    const int k_lo = window > 0 ? max(0, pos0 - window + 1) : 0;
+    int k_lo = window > 0 ? max(0, pos0 - window + 1) : 0;
+    // steps ahead of the window's for positions below keep_first; none if the window's first block is not past them (one walk from 0 then)
+    const int w_lo = k_lo;  // the first position the tile's windows hold
+    int kept_steps = 0;
+    if constexpr (SCORED) {
+        if (keep_first > 0 && k_lo > 0) {
+            kept_steps = (min(keep_first, k_lo) + STEP_KEYS - 1) / STEP_KEYS;
+            if (kept_steps * STEP_KEYS > (k_lo / AP_KEYS) * AP_KEYS) {
+                kept_steps = 0;
+                k_lo = 0;
+            }
+        }
+    }
+    const int kept = kept_steps > 0 ? min(keep_first, k_lo) : 0;  // positions the first steps hold
     const int64_t page_stride = static_cast<int64_t>(n_kv_head) * page_size * hd;
     const int64_t head_off = static_cast<int64_t>(hkv) * page_size * hd;
     constexpr int CHUNKS = 4 * DB;  // 16-byte pieces per padded row
+    const int kb0 = (k_lo / AP_KEYS) * AP_KEYS;          // the window's first block
+    const int kb0v = SCORED ? kb0 - kept_steps * STEP_KEYS : kb0;  // where the walk's count starts
     // a block's keys and values go global -> registers -> LDS (zeros past the head dimension,
     // before the window and past the last key). AP_DEPTH register sets form a ring: a block is
     // fetched AP_DEPTH - 1 blocks before it is multiplied, which covers the latency of the pages.
@@ -149,17 +166,23 @@ attention_prefill_kernel(bf16_t* __restrict__ out, int64_t out_stride, const bf1
     __shared__ int sbt[AP_MAX_BLOCKS];
     const int first_page = k_lo / page_size, n_pages = k_hi / page_size - first_page + 1;
     // (the host has checked that they fit; an id outside the caches' pages becomes one that exists)
-    for (int i = tid; i < n_pages; i += THREADS) sbt[i] = min(max(bt[first_page + i], 0), num_pages - 1);
+    // (kept positions' pages stand ahead of the window's, as many as lie before its first page)
+    const int kept_pages = SCORED && kept > 0 ? min((kept + page_size - 1) / page_size, first_page) : 0;
+    for (int i = tid; i < n_pages; i += THREADS) sbt[kept_pages + i] = min(max(bt[first_page + i], 0), num_pages - 1);
+    if constexpr (SCORED) {
+        for (int i = tid; i < kept_pages; i += THREADS) sbt[i] = min(max(bt[i], 0), num_pages - 1);
+    }
     __syncthreads();
     auto fetch = [&](int kb, u32x4 (&fk)[PER], u32x4 (&fv)[PER]) {
 #pragma unroll
         for (int i = 0; i < PER; ++i) {
             const int c = min(tid + THREADS * i, STEP_KEYS * CHUNKS - 1), key = c / CHUNKS, col = min((c % CHUNKS) * 8, hd - 8);
-            const int kp = min(max(kb + key, k_lo), k_hi);
+            const bool early = SCORED && kb < kb0;  // a step of kept positions (the same for every thread)
+            const int kp = early ? min(kb - kb0v + key, kept - 1) : min(max(kb + key, k_lo), k_hi);
             // page_shift >= 0: the page size is a power of two (no integer division)
             const int lp = page_shift >= 0 ? kp >> page_shift : kp / page_size;
             const int off = page_shift >= 0 ? kp & (page_size - 1) : kp % page_size;
-            const int64_t page = sbt[lp - first_page];
+            const int64_t page = sbt[SCORED && lp < first_page ? lp : kept_pages + lp - first_page];
             const int64_t at = page * page_stride + head_off + static_cast<int64_t>(off) * hd + col;
             fk[i] = *reinterpret_cast<const u32x4*>(kc + at);
             fv[i] = *reinterpret_cast<const u32x4*>(vc + at);
@@ -171,27 +194,28 @@ attention_prefill_kernel(bf16_t* __restrict__ out, int64_t out_stride, const bf1
             const int c = tid + THREADS * i, key = c / CHUNKS, col = (c % CHUNKS) * 8;
             if (c < STEP_KEYS * CHUNKS) {
                 const int kp = kb + key;
-                const bool ok = kp >= k_lo && kp <= k_hi && col < hd;
+                // (between the kept positions and the window lie pages that may have been given back: whatever they hold is not multiplied)
+                const bool ok = (SCORED && kb < kb0 ? kp - kb0v < kept : (kp >= w_lo || (SCORED && kp < keep_first)) && kp >= k_lo && kp <= k_hi) && col < hd;
                 const u32x4 zero = {0, 0, 0, 0};
                 *reinterpret_cast<u32x4*>(&Kb[buf * STAGE + key * LDK + col]) = ok ? fk[i] : zero;
                 *reinterpret_cast<u32x4*>(&Vb[buf * VSTAGE + key * LDK + col]) = ok ? fv[i] : zero;
             }
         }
     };
-    const int kb0 = (k_lo / AP_KEYS) * AP_KEYS;
 #pragma unroll
-    for (int d = 0; d < AP_DEPTH; ++d) fetch(kb0 + d * STEP_KEYS, rk[d], rv[d]);
-    stash(0, kb0, rk[0], rv[0]);
+    for (int d = 0; d < AP_DEPTH; ++d) fetch(kb0v + d * STEP_KEYS, rk[d], rv[d]);
+    stash(0, kb0v, rk[0], rv[0]);
     __syncthreads();
     int cur = 0;
-    for (int kbase = kb0; kbase <= k_hi; kbase += AP_DEPTH * STEP_KEYS) {
+    for (int kbase = kb0v; kbase <= k_hi; kbase += AP_DEPTH * STEP_KEYS) {
 #pragma unroll
       for (int ring = 0; ring < AP_DEPTH; ++ring) {
         const int kb_step = kbase + ring * STEP_KEYS;
         if (kb_step > k_hi) break;
         const bool more = kb_step + STEP_KEYS <= k_hi;
         fetch(kb_step + AP_DEPTH * STEP_KEYS, rk[ring], rv[ring]);  // this set's keys are in LDS already
-        const int kb0w = kb_step + ks * NS * AP_KEYS;  // this wave's first block of the step; its NS blocks are consecutive
+        // this wave's first block of the step; its NS blocks are consecutive
+        const int kb0w = (SCORED && kb_step < kb0 ? kb_step - kb0v : kb_step) + ks * NS * AP_KEYS;
         const bf16_t* Ks = Kb + cur * STAGE + ks * NS * AP_KEYS * LDK;
         const bf16_t* Vs = Vb + cur * VSTAGE + ks * NS * AP_KEYS * LDK;
         if (wave_has && kb0w <= wave_last) {
@@ -250,7 +274,7 @@ attention_prefill_kernel(bf16_t* __restrict__ out, int64_t out_stride, const bf1
 #pragma unroll
             for (int z = 0; z < NS; ++z) {
                 const int kb = kb0w + z * AP_KEYS;
-                const bool whole = kb + AP_KEYS - 1 <= pos0 + 32 * qg && (window <= 0 || kb > wave_last - window);
+                const bool whole = kb + AP_KEYS - 1 <= pos0 + 32 * qg && (window <= 0 || kb > wave_last - window || (SCORED && kb + AP_KEYS <= keep_first));
                 bm[z] = -INFINITY;
                 if (whole) {
 #pragma unroll
@@ -259,7 +283,7 @@ attention_prefill_kernel(bf16_t* __restrict__ out, int64_t out_stride, const bf1
 #pragma unroll
                     for (int r = 0; r < 16; ++r) {
                         const int kp = kb + 8 * (r / 4) + 4 * g2 + r % 4;
-                        const bool ok = kp <= qpos && (window <= 0 || kp > qpos - window);
+                        const bool ok = kp <= qpos && (window <= 0 || kp > qpos - window || (SCORED && kp < keep_first));
                         st[z][r] = ok ? st[z][r] : -INFINITY;
                         bm[z] = fmaxf(bm[z], st[z][r]);
                     }
@@ -422,7 +446,7 @@ static int run_attention_prefill(void* out, int64_t out_stride, const void* q, i
                                  const void* vc, const int* block_tables, int max_blocks, const int* work,
                                  int n_tiles, int tile, int ksplit, float scale, int window, int n_head, int n_kv_head, int hd,
                                  int page_size, int num_pages, float softcap, const float* bias_table, int max_dist, const float* sinks,
-                                 hipStream_t stream) {
+                                 int keep_first, hipStream_t stream) {
     LIYAB_REQUIRE(out && q && kc && vc && block_tables && work, "attention_prefill: null pointer");
     LIYAB_REQUIRE(num_pages > 0, "attention_prefill: the caches hold %d pages", num_pages);
     LIYAB_REQUIRE(n_tiles >= 0 && n_head > 0 && n_kv_head > 0 && page_size > 0 && max_blocks > 0, "attention_prefill: bad sizes");
@@ -434,7 +458,7 @@ static int run_attention_prefill(void* out, int64_t out_stride, const void* q, i
                   "attention_prefill: operands must be 16-byte aligned with strides that are multiples of 8");
     LIYAB_REQUIRE(out_stride >= static_cast<int64_t>(n_head) * hd && q_stride >= static_cast<int64_t>(n_head) * hd,
                   "attention_prefill: row strides are shorter than heads x head size");
-    LIYAB_REQUIRE(window >= 0, "attention_prefill: negative window");
+    LIYAB_REQUIRE(window >= 0 && keep_first >= 0, "attention_prefill: negative window or kept positions");
     LIYAB_REQUIRE(scale > 0.0f, "attention_prefill: the scale must be positive (the maximum is taken before scaling), not %g", scale);
     LIYAB_REQUIRE(tile == 64 || tile == 128, "attention_prefill: tiles of %d queries; 64 or 128 are taken", tile);
     LIYAB_REQUIRE(ksplit == 1 || ksplit == 2 || (ksplit == 4 && tile == 64), "attention_prefill: %d waves a query group do not go with tiles of %d", ksplit, tile);
@@ -451,7 +475,7 @@ static int run_attention_prefill(void* out, int64_t out_stride, const void* q, i
     auto* pv = static_cast<const bf16_t*>(vc);
 #define LIYAB_RUN(D, Q, S)                                                                                          \
     attention_prefill_kernel<D, Q, S, (D <= 2 && Q == 4 && S <= 2) ? 2 : 1, SCORED><<<grid, 64 * Q * S, 0, stream>>>(                          \
-        o, out_stride, pq, q_stride, pk, pv, block_tables, max_blocks, work, scale, window, n_head, n_kv_head, hd, page_size, page_shift, num_pages, softcap, bias_table, max_dist, sinks)
+        o, out_stride, pq, q_stride, pk, pv, block_tables, max_blocks, work, scale, window, n_head, n_kv_head, hd, page_size, page_shift, num_pages, softcap, bias_table, max_dist, sinks, keep_first)
 #define LIYAB_RUN4(D) LIYAB_RUN(D, 2, 4)
 #define LIYAB_SKIP4(D) (void)0  // four stages of 128 keys do not fit LDS at these head sizes (refused above)
 #define LIYAB_GO(D, FOUR)                           \
@@ -481,18 +505,18 @@ extern "C" int liyab_attention_prefill(void* out, int64_t out_stride, const void
                                        int n_tiles, int tile, int ksplit, float scale, int window, int n_head, int n_kv_head, int hd,
                                        int page_size, int num_pages, hipStream_t stream) {
     return run_attention_prefill<false>(out, out_stride, q, q_stride, kc, vc, block_tables, max_blocks, work, n_tiles, tile, ksplit, scale, window,
-                                        n_head, n_kv_head, hd, page_size, num_pages, 0.0f, nullptr, 0, nullptr, stream);
+                                        n_head, n_kv_head, hd, page_size, num_pages, 0.0f, nullptr, 0, nullptr, 0, stream);
 }
 
 // The same with the scores worked on before the softmax: softcap > 0 caps them, cap * tanh(score / cap); bias_table (float
 // [max_dist + 1, n_head]) adds table[min(query position - key position, max_dist), head]; sinks (float [n_head], or null):
-// exp(sinks[head]) is added to the softmax's denominator.
+// exp(sinks[head]) is added to the softmax's denominator; keep_first: positions below it stay visible behind the window.
 extern "C" int liyab_attention_prefill_scored(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* kc,
                                               const void* vc, const int* block_tables, int max_blocks, const int* work,
                                               int n_tiles, int tile, int ksplit, float scale, int window, int n_head, int n_kv_head, int hd,
                                               int page_size, int num_pages, float softcap, const float* bias_table, int max_dist,
-                                              const float* sinks, hipStream_t stream) {
+                                              const float* sinks, int keep_first, hipStream_t stream) {
     LIYAB_REQUIRE(softcap >= 0.0f && (bias_table == nullptr || max_dist >= 0), "attention_prefill_scored: a negative cap or distance");
     return run_attention_prefill<true>(out, out_stride, q, q_stride, kc, vc, block_tables, max_blocks, work, n_tiles, tile, ksplit, scale, window,
-                                       n_head, n_kv_head, hd, page_size, num_pages, softcap, bias_table, max_dist, sinks, stream);
+                                       n_head, n_kv_head, hd, page_size, num_pages, softcap, bias_table, max_dist, sinks, keep_first, stream);
 }

@@ -12,9 +12,13 @@
 // Values may be shared between layers of a step: `v_keep` (float [n, G * dv]) gets this layer's values as projected;
 // `v_first` (such rows of an earlier layer) and `v_lam` (one float on the device) make the cached values (1 - lam) v + lam v_first.
 //
+// liyab_qk_prepare_rows: the same for norms taken over all of a token's queries (and all of its keys) at once, before they are
+// heads: a weight an entry, q_norm [H * dk] and k_norm [G * dk]. A workgroup a token: both sums in one pass over the row, the
+// token's cosines and sines once for all heads. Without pages (kc null) only the queries: keys and values of another layer are used.
+//
 // liyab_attention_scored: one workgroup a (token, query head). score = scale * q . k, then, each optional:
 // a soft cap, cap * tanh(score / cap); a learned bias by distance, table[min(i - j, max_dist), head].
-// Causal, with an optional window; ordinary softmax in 32-bit over tiles of 256 keys in position order
+// Causal, with an optional window, beside which the first `keep_first` positions may stay visible; ordinary softmax in 32-bit over tiles of 256 keys in position order
 // with a running maximum and sum, so that a row's rounding follows from its position alone. Values are
 // `dv` wide (keys `dk`). `sinks` (one logit a head, optional): exp(sink) joins the softmax's denominator, with no value.
 // The result may be multiplied by the logistic function of a gate's logits before it is rounded to the compute type.
@@ -114,13 +118,87 @@ qk_prepare_kernel(const float* __restrict__ src, int64_t ld, int q_off, int k_of
     }
 }
 
+constexpr int QR_MAX_PAIRS = 256;  // turned pairs of a head (heads of up to 512)
+
+template <typename T>
+__global__ void __launch_bounds__(AS_THREADS)
+qk_prepare_rows_kernel(const float* __restrict__ src, int64_t ld, int q_off, int k_off, int v_off, int H, int G, int dk, int dv, int dk_out,
+                       int dv_out, T* __restrict__ q_out, T* __restrict__ kc, T* __restrict__ vc, const int* __restrict__ slots, int page_size,
+                       int num_pages, const float* __restrict__ q_norm, const float* __restrict__ k_norm, float eps,
+                       const double* __restrict__ freqs, int rot_dims, const int* __restrict__ positions, int rot_halves) {
+    __shared__ float2 turn[QR_MAX_PAIRS];
+    __shared__ float red[2][AS_THREADS / kWave];
+    const int t = blockIdx.x, tid = threadIdx.x;
+    const float* row = src + static_cast<int64_t>(t) * ld;
+    const float *q = row + q_off, *k = row + k_off;
+    const int n_turned = rot_dims / 2, p = positions[t];
+    const bool keys = kc != nullptr;
+    float sq = 0.0f, sk = 0.0f;
+    for (int i = tid; i < H * dk; i += AS_THREADS) sq = fmaf(q[i], q[i], sq);
+    if (keys)
+        for (int i = tid; i < G * dk; i += AS_THREADS) sk = fmaf(k[i], k[i], sk);
+    for (int i = tid; i < n_turned; i += AS_THREADS) {
+        const float angle = turn_angle(p, freqs[i]);
+        turn[i] = float2{cosf(angle), sinf(angle)};
+    }
+    sq = wave_sum(sq);
+    sk = wave_sum(sk);
+    if (tid % kWave == 0) {
+        red[0][tid / kWave] = sq;
+        red[1][tid / kWave] = sk;
+    }
+    __syncthreads();
+    sq = sk = 0.0f;
+#pragma unroll
+    for (int i = 0; i < AS_THREADS / kWave; ++i) {
+        sq += red[0][i];
+        sk += red[1][i];
+    }
+    const float fq = 1.0f / sqrtf(sq / static_cast<float>(H * dk) + eps), fk = 1.0f / sqrtf(sk / static_cast<float>(G * dk) + eps);
+    const int64_t slot = keys ? slots[t] : -1;
+    const bool stored = slot >= 0 && slot < static_cast<int64_t>(num_pages) * page_size;
+    // entries in pairs, those of the heads' rows behind their last entry included (zeros)
+    const int per = (dk_out + 1) / 2;
+    const int items = (H + (stored ? G : 0)) * per;
+    for (int item = tid; item < items; item += AS_THREADS) {
+        const int hh = item / per, u = item % per;
+        const bool is_q = hh < H;
+        const int head = is_q ? hh : hh - H;
+        int e0 = 2 * u, e1 = e0 + 1;
+        if (rot_halves && u < n_turned) {
+            e0 = u;
+            e1 = u + n_turned;
+        }
+        const int at = head * dk;
+        const float* x = (is_q ? q : k) + at;
+        const float* w = (is_q ? q_norm : k_norm) + at;
+        const float f = is_q ? fq : fk;
+        float a = e0 < dk ? x[e0] * f * w[e0] : 0.0f, b = e1 < dk ? x[e1] * f * w[e1] : 0.0f;
+        if (u < n_turned) {
+            const float2 cs = turn[u];
+            const float ra = a * cs.x - b * cs.y, rb = b * cs.x + a * cs.y;
+            a = ra;
+            b = rb;
+        }
+        T* dst = is_q ? q_out + (static_cast<int64_t>(t) * H + head) * dk_out
+                      : kc + (((slot / page_size) * G + head) * page_size + slot % page_size) * dk_out;
+        dst[e0] = from_float<T>(a);
+        if (e1 < dk_out) dst[e1] = from_float<T>(b);
+    }
+    if (!stored) return;
+    for (int item = tid; item < G * dv_out; item += AS_THREADS) {
+        const int head = item / dv_out, i = item % dv_out;
+        vc[(((slot / page_size) * G + head) * page_size + slot % page_size) * dv_out + i] = from_float<T>(i < dv ? row[v_off + head * dv + i] : 0.0f);
+    }
+}
+
 template <typename T>
 __global__ void __launch_bounds__(AS_THREADS)
 attention_scored_kernel(T* __restrict__ out, int64_t out_stride, const T* __restrict__ q, int64_t q_stride, const T* __restrict__ kc,
                         const T* __restrict__ vc, const int* __restrict__ block_tables, int max_blocks, const int* __restrict__ tok_seq,
                         const int* __restrict__ tok_pos, float scale, float softcap, int window, const float* __restrict__ bias_table,
                         int max_dist, const float* __restrict__ gate, int64_t gate_stride, int n_head, int n_kv_head, int dk, int dv,
-                        int page_size, int num_pages, const float* __restrict__ sinks) {
+                        int page_size, int num_pages, const float* __restrict__ sinks, int keep_first) {
     extern __shared__ float smem[];
     float* qs = smem;                          // [dk]
     float* sc = qs + dk;                       // [AS_THREADS]
@@ -133,6 +211,8 @@ attention_scored_kernel(T* __restrict__ out, int64_t out_stride, const T* __rest
     const int* bt = block_tables + static_cast<int64_t>(tok_seq[t]) * max_blocks;
     const int hkv = h / (n_head / n_kv_head);
     const int first = window > 0 ? max(0, pos - window + 1) : 0;
+    // the kept first positions stand ahead of the window's: place j0 .. first - 1 of the walk are positions 0 .. kept - 1
+    const int kept = min(keep_first, first), walk0 = first - kept;
     const T* qrow = q + static_cast<int64_t>(t) * q_stride + static_cast<int64_t>(h) * dk;
     for (int e = tid; e < dk; e += AS_THREADS) qs[e] = to_float<T>(qrow[e]);
     __syncthreads();
@@ -143,10 +223,11 @@ attention_scored_kernel(T* __restrict__ out, int64_t out_stride, const T* __rest
     const float inv_cap = softcap > 0.0f ? 1.0f / softcap : 0.0f;
     float m = -INFINITY, l = 0.0f, acc = 0.0f;
 
-    for (int j0 = first; j0 <= pos; j0 += AS_THREADS) {
-        const int j = j0 + tid;
+    for (int j0 = walk0; j0 <= pos; j0 += AS_THREADS) {
+        const int place = j0 + tid;
+        const int j = place < first ? place - walk0 : place;
         float s = -INFINITY;
-        if (j <= pos) {
+        if (place <= pos) {
             const int64_t page = min(max(bt[j / page_size], 0), num_pages - 1);
             const T* kr = kc + ((page * n_kv_head + hkv) * page_size + j % page_size) * dk;
             float dot = 0.0f;
@@ -162,7 +243,7 @@ attention_scored_kernel(T* __restrict__ out, int64_t out_stride, const T* __rest
 #pragma unroll
         for (int i = 1; i < AS_THREADS / kWave; ++i) tm = fmaxf(tm, red[i]);
         const float m_new = fmaxf(m, tm);
-        const float p = j <= pos ? expf(s - m_new) : 0.0f;
+        const float p = place <= pos ? expf(s - m_new) : 0.0f;
         sc[tid] = p;
         float ps = wave_sum(p);
         __syncthreads();
@@ -178,7 +259,7 @@ attention_scored_kernel(T* __restrict__ out, int64_t out_stride, const T* __rest
         if (vthread) {
             const int len = min(AS_THREADS, pos - j0 + 1);
             for (int jj = g; jj < len; jj += G) {
-                const int jv = j0 + jj;
+                const int jv = j0 + jj < first ? j0 + jj - walk0 : j0 + jj;
                 const int64_t page = min(max(bt[jv / page_size], 0), num_pages - 1);
                 const T* vr = vc + ((page * n_kv_head + hkv) * page_size + jv % page_size) * dv;
                 acc = fmaf(sc[jj], to_float<T>(vr[e]), acc);
@@ -239,16 +320,42 @@ extern "C" int liyab_qk_prepare(const float* src, int64_t ld, int q_off, int k_o
     return check_launch("qk_prepare");
 }
 
+extern "C" int liyab_qk_prepare_rows(const float* src, int64_t ld, int q_off, int k_off, int v_off, int H, int G, int dk, int dv, int dk_out,
+                                     int dv_out, void* q_out, void* kc, void* vc, int dtype, const int* slots, int page_size, int num_pages,
+                                     const float* q_norm, const float* k_norm, float eps, const double* freqs, int rot_dims, const int* positions,
+                                     int n, int rot_halves, hipStream_t stream) {
+    LIYAB_REQUIRE(src && q_out && positions && q_norm && (kc == nullptr) == (vc == nullptr), "qk_prepare_rows: null pointer");
+    LIYAB_REQUIRE(n >= 0 && H > 0 && G > 0 && dk > 0 && dv > 0 && dk <= 512, "qk_prepare_rows: bad sizes");
+    LIYAB_REQUIRE(kc == nullptr || (slots && k_norm && page_size > 0 && num_pages > 0), "qk_prepare_rows: keys need their weight and pages");
+    LIYAB_REQUIRE(dk_out >= dk && dv_out >= dv, "qk_prepare_rows: rows of %d / %d do not hold heads of %d / %d", dk_out, dv_out, dk, dv);
+    LIYAB_REQUIRE(q_off >= 0 && q_off + static_cast<int64_t>(H) * dk <= ld, "qk_prepare_rows: the queries' columns pass the source's rows");
+    LIYAB_REQUIRE(kc == nullptr || (k_off >= 0 && v_off >= 0 && k_off + static_cast<int64_t>(G) * dk <= ld && v_off + static_cast<int64_t>(G) * dv <= ld),
+                  "qk_prepare_rows: the keys' or values' columns pass the source's rows");
+    LIYAB_REQUIRE(rot_dims >= 0 && rot_dims <= dk && rot_dims % 2 == 0 && (rot_dims == 0 || freqs != nullptr), "qk_prepare_rows: %d turned entries of heads of %d", rot_dims, dk);
+    if (n == 0) return 0;
+    if (dtype == kF32)
+        qk_prepare_rows_kernel<float><<<n, AS_THREADS, 0, stream>>>(src, ld, q_off, k_off, v_off, H, G, dk, dv, dk_out, dv_out, static_cast<float*>(q_out),
+                                                                    static_cast<float*>(kc), static_cast<float*>(vc), slots, page_size, num_pages, q_norm,
+                                                                    k_norm, eps, freqs, rot_dims, positions, rot_halves);
+    else if (dtype == kBF16)
+        qk_prepare_rows_kernel<bf16_t><<<n, AS_THREADS, 0, stream>>>(src, ld, q_off, k_off, v_off, H, G, dk, dv, dk_out, dv_out, static_cast<bf16_t*>(q_out),
+                                                                     static_cast<bf16_t*>(kc), static_cast<bf16_t*>(vc), slots, page_size, num_pages, q_norm,
+                                                                     k_norm, eps, freqs, rot_dims, positions, rot_halves);
+    else return fail(1, "qk_prepare_rows: unknown dtype %d", dtype);
+    return check_launch("qk_prepare_rows");
+}
+
 extern "C" int liyab_attention_scored(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* kc, const void* vc, int dtype,
                                       const int* block_tables, int max_blocks, const int* tok_seq, const int* tok_pos, int n, float scale,
                                       float softcap, int window, const float* bias_table, int max_dist, const float* gate, int64_t gate_stride,
-                                      int n_head, int n_kv_head, int dk, int dv, int page_size, int num_pages, const float* sinks, hipStream_t stream) {
+                                      int n_head, int n_kv_head, int dk, int dv, int page_size, int num_pages, const float* sinks, int keep_first,
+                                      hipStream_t stream) {
     LIYAB_REQUIRE(out && q && kc && vc && block_tables && tok_seq && tok_pos, "attention_scored: null pointer");
     LIYAB_REQUIRE(num_pages > 0 && n >= 0 && n_head > 0 && n_kv_head > 0 && page_size > 0 && max_blocks > 0, "attention_scored: bad sizes");
     LIYAB_REQUIRE(n_head % n_kv_head == 0, "attention_scored: %d query heads are no multiple of %d key/value heads", n_head, n_kv_head);
     LIYAB_REQUIRE(dk > 0 && dk <= 512 && dv > 0 && dv <= AS_THREADS, "attention_scored: heads of %d / %d are outside 1..512 / 1..256", dk, dv);
     LIYAB_REQUIRE(out_stride >= static_cast<int64_t>(n_head) * dv && q_stride >= static_cast<int64_t>(n_head) * dk, "attention_scored: row strides are shorter than the heads");
-    LIYAB_REQUIRE(window >= 0 && softcap >= 0.0f, "attention_scored: negative window or cap");
+    LIYAB_REQUIRE(window >= 0 && softcap >= 0.0f && keep_first >= 0, "attention_scored: negative window, cap or kept positions");
     LIYAB_REQUIRE(bias_table == nullptr || max_dist >= 0, "attention_scored: a bias table needs its largest distance");
     LIYAB_REQUIRE(gate == nullptr || gate_stride >= static_cast<int64_t>(n_head) * dv, "attention_scored: the gate's rows are shorter than the heads");
     LIYAB_REQUIRE(n_head <= 65535, "attention_scored: too many heads");
@@ -260,12 +367,12 @@ extern "C" int liyab_attention_scored(void* out, int64_t out_stride, const void*
         attention_scored_kernel<float><<<grid, AS_THREADS, smem, stream>>>(
             static_cast<float*>(out), out_stride, static_cast<const float*>(q), q_stride, static_cast<const float*>(kc), static_cast<const float*>(vc),
             block_tables, max_blocks, tok_seq, tok_pos, scale, softcap, window, bias_table, max_dist, gate, gate_stride, n_head, n_kv_head, dk, dv,
-            page_size, num_pages, sinks);
+            page_size, num_pages, sinks, keep_first);
     else if (dtype == kBF16)
         attention_scored_kernel<bf16_t><<<grid, AS_THREADS, smem, stream>>>(
             static_cast<bf16_t*>(out), out_stride, static_cast<const bf16_t*>(q), q_stride, static_cast<const bf16_t*>(kc), static_cast<const bf16_t*>(vc),
             block_tables, max_blocks, tok_seq, tok_pos, scale, softcap, window, bias_table, max_dist, gate, gate_stride, n_head, n_kv_head, dk, dv,
-            page_size, num_pages, sinks);
+            page_size, num_pages, sinks, keep_first);
     else return fail(1, "attention_scored: unknown dtype %d", dtype);
     return check_launch("attention_scored");
 }

@@ -15,18 +15,16 @@
 //   A step with long portions (seg_tokens > 0) runs in segments of that many tokens side by side, in three launches. The
 //   recurrence is linear in S, S_t = A_t S_(t-1) + k_t v_t^T with A_t = diag(w_t) - (a_t * u_t) u_t^T, so a segment's end is
 //   P S_start + Z: every segment but a request's last walks twice side by side, from a zero state for Z and, without the outer
-//   products, from the unit matrix for P (the product of its A_t); delta_combine_kernel strings a request's segments together
-//   and leaves each the state it starts from; then every segment walks from that state and writes its outputs.
-// liyab_head_norm_gate: out = o / sqrt(mean(o^2 over the head) + eps) * weight * sigmoid(gate), rounded once.
+//   products, from the unit matrix for P (the product of its A_t); delta_combine_kernel (delta_segments.h) strings a request's segments
+//   together and leaves each the state it starts from; then every segment walks from that state and writes its outputs.
+// liyab_head_norm_gate: out = o / sqrt(mean(o^2 over the head) + eps) * weight * sigmoid(gate) (silu: * gate * sigmoid(gate)), rounded
+//   once; a weight an entry of the row, or one of a head's width for all heads (shared_w).
 // liyab_delta_single: all three for a step of single tokens and heads of up to 64, in one kernel.
 #include "common.h"
+#include "delta_segments.h"
 #include "launchers.h"
 
 namespace liyab {
-
-constexpr int kDeltaCols = 16;    // columns of S a wave
-constexpr int kDeltaSplit = 4;    // lanes that share a column's rows
-constexpr int kDeltaWaves = 4;    // waves a workgroup, each with work of its own
 
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
 
@@ -72,22 +70,6 @@ struct DeltaArgs {
     float* seg_start;         // [segments][H][D][D]: the state a segment starts from (the combining pass writes it)
 };
 
-// segment `g` of the step in the order of the requests: its request and rows; false past the last segment
-__device__ __forceinline__ bool delta_segment(const DeltaArgs& a, int g, int& s, int& begin, int& end, bool& last) {
-    for (s = 0; s < a.n_seqs; ++s) {
-        const int b = a.seq_starts[s], len = a.seq_starts[s + 1] - b;
-        const int n_seg = (len + a.seg_tokens - 1) / a.seg_tokens;
-        if (g < n_seg) {
-            begin = b + g * a.seg_tokens;
-            end = min(begin + a.seg_tokens, b + len);
-            last = g == n_seg - 1;
-            return true;
-        }
-        g -= n_seg;
-    }
-    return false;
-}
-
 // REG: rows a lane holds (D <= 4 * REG); a lane's rows are i0 .. i0 + REG - 1, i0 = (lane % 4) * REG. The waves of a workgroup
 // are column blocks of one (request, head) and share its tokens' vectors: CH tokens at a time go through LDS (w, a * u, u, k, r
 // padded to DP = 4 * REG entries, v), the next CH fetched into registers while these are computed.
@@ -112,7 +94,7 @@ delta_scan_kernel(DeltaArgs a) {
     int s = item, begin, end;
     bool last_seg = true;
     if (a.seg_tokens > 0) {
-        if (!delta_segment(a, item, s, begin, end, last_seg)) return;
+        if (!find_segment(a.seq_starts, a.n_seqs, a.seg_tokens, item, s, begin, end, last_seg)) return;
         if (a.phase == 1 && last_seg) return;  // (nobody needs the end of a request's last segment from zero)
     } else {
         begin = a.seq_starts[s];
@@ -213,114 +195,6 @@ delta_scan_kernel(DeltaArgs a) {
 #pragma unroll
         for (int ii = 0; ii < REG; ++ii)
             if (mine[ii]) Sg[static_cast<int64_t>(i0 + ii) * D + j] = S[ii];
-    }
-}
-
-// Between the two passes over the segments: the state each segment starts from. A workgroup a (request, head, block of 16
-// columns) walks the request's segments in order, S <- P S + Z, and leaves in seg_start what each segment starts from (the
-// first: the slot's state, or zeros at position 0); an array of its own, named as such to the compiler, so that no load of a
-// later segment's Z or P has to wait behind a store. A thread holds rows ib, ib + 16, ... of one column; the columns' block
-// of S lies in LDS; P goes through LDS in tiles of 64 x 64, the next tile fetched into registers while this one is used.
-constexpr int kCombTile = 64, kCombStride = kCombTile + 4;  // (rows 68 floats apart: four rows read together fall into different banks)
-constexpr int kCombMaxD = 256;
-
-__global__ void __launch_bounds__(256)
-delta_combine_kernel(DeltaArgs a, const float* __restrict__ seg_z, const float* __restrict__ seg_p, float* __restrict__ seg_start) {
-    __shared__ __attribute__((aligned(16))) float Pt[kCombTile * kCombStride];
-    __shared__ float Sl[2][kCombMaxD * kDeltaCols];
-    const int s = blockIdx.x, h = blockIdx.y, cb = blockIdx.z, tid = threadIdx.x;
-    const int D = a.D, H = a.H;
-    int g0 = 0;
-    for (int q = 0; q < s; ++q) g0 += (a.seq_starts[q + 1] - a.seq_starts[q] + a.seg_tokens - 1) / a.seg_tokens;
-    const int begin = a.seq_starts[s];
-    const int n_seg = (a.seq_starts[s + 1] - begin + a.seg_tokens - 1) / a.seg_tokens;
-    if (n_seg <= 0) return;
-    const int slot = a.state_slots[s];
-    const bool from_slot = slot >= 0 && slot < a.n_slots && a.positions[begin] != 0;
-    const int jj = tid % kDeltaCols, ib = tid / kDeltaCols, j = cb * kDeltaCols + jj;
-    const int64_t DD = static_cast<int64_t>(D) * D;
-    const float* S0 = a.state + static_cast<int64_t>(from_slot ? slot : 0) * a.state_stride + h * DD;
-    for (int m = ib; m < kCombMaxD; m += 256 / kDeltaCols) {  // (rows past the head's last stay zero: they meet zeros of P)
-        Sl[0][m * kDeltaCols + jj] = (from_slot && m < D && j < D) ? S0[static_cast<int64_t>(m) * D + j] : 0.0f;
-        Sl[1][m * kDeltaCols + jj] = 0.0f;
-    }
-    const int nb = (D + kCombTile - 1) / kCombTile, per_seg = nb * nb;
-    const int n_tiles = (n_seg - 1) * per_seg;
-    constexpr int NPRE = kCombTile * kCombTile / 256;
-    float pre[NPRE];
-    auto fetch = [&](int T) {
-        const int g = T / per_seg, ibk = (T % per_seg) / nb, mbk = T % nb;
-        const float* P = seg_p + (static_cast<int64_t>(g0 + g) * H + h) * DD;
-#pragma unroll
-        for (int q = 0; q < NPRE; ++q) {
-            const int e = tid + q * 256;
-            const int i = ibk * kCombTile + e / kCombTile, m = mbk * kCombTile + e % kCombTile;
-            const float val = P[static_cast<int64_t>(min(i, D - 1)) * D + min(m, D - 1)];
-            pre[q] = (i < D && m < D) ? val : 0.0f;
-        }
-    };
-    // a segment's own end, for the rows of block ibk of step g * nb + ibk; asked for one step ahead, like the tiles (the barriers
-    // below wait for LDS only, so what is on its way from memory stays on its way)
-    auto fetch_z = [&](int step, float (&z)[4]) {
-        const int g = step / nb, ibk = step % nb;
-        const bool live = g + 1 < n_seg;  // (a request's last segment has none)
-        const float* Zg = seg_z + (static_cast<int64_t>(g0 + g) * H + h) * DD;
-#pragma unroll
-        for (int q = 0; q < 4; ++q) {
-            const int i = ibk * kCombTile + ib + 16 * q;
-            z[q] = (live && i < D && j < D) ? Zg[static_cast<int64_t>(i) * D + j] : 0.0f;
-        }
-    };
-    float z_next[4];
-    fetch_z(0, z_next);
-    if (n_tiles > 0) fetch(0);
-    __syncthreads();
-    typedef __attribute__((ext_vector_type(4))) float f32x4;
-    int cur = 0;
-    for (int g = 0; g < n_seg; ++g) {
-        float* Sg = seg_start + (static_cast<int64_t>(g0 + g) * H + h) * DD;
-        const bool more = g + 1 < n_seg;
-        for (int ibk = 0; ibk < nb; ++ibk) {
-            float acc[4];
-#pragma unroll
-            for (int q = 0; q < 4; ++q) acc[q] = z_next[q];
-            if (g * nb + ibk + 1 < n_seg * nb) fetch_z(g * nb + ibk + 1, z_next);
-            if (more) {
-                for (int mbk = 0; mbk < nb; ++mbk) {
-                    const int T = (g * nb + ibk) * nb + mbk;
-#pragma unroll
-                    for (int q = 0; q < NPRE; ++q) {
-                        const int e = tid + q * 256;
-                        Pt[(e / kCombTile) * kCombStride + e % kCombTile] = pre[q];
-                    }
-                    lds_barrier();
-                    if (T + 1 < n_tiles) fetch(T + 1);
-                    const float* Sc = Sl[cur] + mbk * kCombTile * kDeltaCols + jj;
-#pragma unroll 4
-                    for (int c = 0; c < kCombTile; c += 4) {
-                        float sv[4];
-#pragma unroll
-                        for (int e = 0; e < 4; ++e) sv[e] = Sc[(c + e) * kDeltaCols];
-#pragma unroll
-                        for (int q = 0; q < 4; ++q) {
-                            const f32x4 p4 = *reinterpret_cast<const f32x4*>(Pt + (ib + 16 * q) * kCombStride + c);
-#pragma unroll
-                            for (int e = 0; e < 4; ++e) acc[q] += p4[e] * sv[e];
-                        }
-                    }
-                    lds_barrier();  // (the next tile takes this one's place)
-                }
-            }
-#pragma unroll
-            for (int q = 0; q < 4; ++q) {
-                const int i = ibk * kCombTile + ib + 16 * q;
-                if (i < D) Sl[cur ^ 1][i * kDeltaCols + jj] = acc[q];
-            }
-        }
-        if (j < D)
-            for (int m = ib; m < D; m += 256 / kDeltaCols) Sg[static_cast<int64_t>(m) * D + j] = Sl[cur][m * kDeltaCols + jj];
-        lds_barrier();
-        cur ^= 1;
     }
 }
 
@@ -440,7 +314,7 @@ delta_single_kernel(DeltaSingleArgs a) {
 template <typename T>
 __global__ void __launch_bounds__(256)
 head_norm_gate_kernel(T* __restrict__ out, const float* __restrict__ o, const float* __restrict__ gate, int64_t ldg, const float* __restrict__ w,
-                      float eps, int n, int H, int D) {
+                      int w_step, float eps, int n, int H, int D, int silu) {
     const int item = blockIdx.x * 4 + threadIdx.x / kWave, lane = threadIdx.x % kWave;
     if (item >= n * H) return;
     const int t = item / H, h = item % H;
@@ -450,8 +324,11 @@ head_norm_gate_kernel(T* __restrict__ out, const float* __restrict__ o, const fl
     const float scale = 1.0f / sqrtf(wave_sum(ss) / static_cast<float>(D) + eps);
     for (int i = lane; i < D; i += kWave) {
         float v = row[i] * scale;
-        if (w != nullptr) v *= w[h * D + i];
-        if (gate != nullptr) v *= sigmoid_f(gate[static_cast<int64_t>(t) * ldg + h * D + i]);
+        if (w != nullptr) v *= w[h * w_step + i];
+        if (gate != nullptr) {
+            const float g = gate[static_cast<int64_t>(t) * ldg + h * D + i];
+            v *= silu ? g * sigmoid_f(g) : sigmoid_f(g);
+        }
         out[(static_cast<int64_t>(t) * H + h) * D + i] = from_float<T>(v);
     }
 }
@@ -506,7 +383,8 @@ extern "C" int liyab_delta_scan(float* out, const float* r, const float* k, cons
         DeltaArgs p = a;
         p.phase = 1;
         walk(p, static_cast<int64_t>(max_segs) * 2, false);
-        delta_combine_kernel<<<dim3(n_seqs, H, n_cb), 256, 0, stream>>>(p, seg_state, seg_trans, seg_start);
+        const DeltaSegments segs{state, state_stride, n_slots, seq_starts, positions, state_slots, n_seqs, H, D, D, seg_tokens};
+        delta_combine_kernel<<<dim3(n_seqs, H, n_cb), 256, 0, stream>>>(segs, seg_state, seg_trans, seg_start);
         p.phase = 3;
         walk(p, max_segs, true);
         return check_launch("delta_scan");
@@ -541,14 +419,14 @@ extern "C" int liyab_delta_single(void* out, int out_dtype, const float* r, cons
     return check_launch("delta_single");
 }
 
-extern "C" int liyab_head_norm_gate(void* out, int out_dtype, const float* o, const float* gate, int64_t ldg, const float* w, float eps, int n,
-                                    int H, int D, hipStream_t stream) {
+extern "C" int liyab_head_norm_gate(void* out, int out_dtype, const float* o, const float* gate, int64_t ldg, const float* w, int shared_w,
+                                    float eps, int n, int H, int D, int silu, hipStream_t stream) {
     LIYAB_REQUIRE(out && o, "head_norm_gate: null pointer");
     LIYAB_REQUIRE(n >= 0 && H > 0 && D > 0 && (gate == nullptr || ldg >= static_cast<int64_t>(H) * D), "head_norm_gate: bad sizes");
     LIYAB_REQUIRE(out_dtype == kF32 || out_dtype == kBF16, "head_norm_gate: unknown dtype %d", out_dtype);
     if (n == 0) return 0;
     const unsigned grid = static_cast<unsigned>((static_cast<int64_t>(n) * H + 3) / 4);
-    if (out_dtype == kF32) head_norm_gate_kernel<float><<<grid, 256, 0, stream>>>(static_cast<float*>(out), o, gate, ldg, w, eps, n, H, D);
-    else head_norm_gate_kernel<bf16_t><<<grid, 256, 0, stream>>>(static_cast<bf16_t*>(out), o, gate, ldg, w, eps, n, H, D);
+    if (out_dtype == kF32) head_norm_gate_kernel<float><<<grid, 256, 0, stream>>>(static_cast<float*>(out), o, gate, ldg, w, shared_w ? 0 : D, eps, n, H, D, silu);
+    else head_norm_gate_kernel<bf16_t><<<grid, 256, 0, stream>>>(static_cast<bf16_t*>(out), o, gate, ldg, w, shared_w ? 0 : D, eps, n, H, D, silu);
     return check_launch("head_norm_gate");
 }

@@ -8,6 +8,8 @@
 // they meet: g = min(G, limit), u = clamp(U, -limit, limit), y = g * sigmoid(slope * g) * (u + shift),
 // from one 32-bit product [G | U] a row.
 //
+// liyab_glu: the inner rows of a plain gated feed-forward, y = act(G) * U with act = silu or the tanh form of gelu, from such a product.
+//
 // liyab_activate: tanh, silu, the logistic function or the squared positive part of 32-bit rows, rounded to the output type.
 //
 // liyab_gate_rows: x *= scale * sigmoid(g) in place, a gate on a mixer's rows from 32-bit logits (and a constant factor).
@@ -54,6 +56,17 @@ glu_clamped_kernel(T* __restrict__ out, const float* __restrict__ gu, int64_t ld
     const float g = fminf(row[i], limit);
     const float u = fminf(fmaxf(row[ff + i], -limit), limit);
     out[static_cast<int64_t>(t) * ff + i] = from_float<T>(g * logistic(slope * g) * (u + shift));
+}
+
+template <typename T>
+__global__ void __launch_bounds__(EW_THREADS)
+glu_kernel(T* __restrict__ out, const float* __restrict__ gu, int64_t ld, int ff, int act) {
+    const int t = blockIdx.y;
+    const int i = blockIdx.x * EW_THREADS + threadIdx.x;
+    if (i >= ff) return;
+    const float* row = gu + static_cast<int64_t>(t) * ld;
+    const float g = row[i];
+    out[static_cast<int64_t>(t) * ff + i] = from_float<T>((act == 0 ? g * logistic(g) : sizeof(T) == 2 ? gelu_tanh_fast(g) : gelu_tanh(g)) * row[ff + i]);
 }
 
 template <typename T>
@@ -145,6 +158,19 @@ extern "C" int liyab_glu_clamped(void* out, int out_dtype, const float* gu, int6
     else if (out_dtype == kBF16) glu_clamped_kernel<bf16_t><<<grid, EW_THREADS, 0, stream>>>(static_cast<bf16_t*>(out), gu, ld, ff, limit, slope, shift);
     else return fail(1, "glu_clamped: unknown dtype %d", out_dtype);
     return check_launch("glu_clamped");
+}
+
+// out[t, i] = act(gu[t, i]) * gu[t, ff + i]; act 0: silu, 1: the tanh form of gelu.
+extern "C" int liyab_glu(void* out, int out_dtype, const float* gu, int64_t ld, int n, int ff, int act, hipStream_t stream) {
+    LIYAB_REQUIRE(out && gu, "glu: null pointer");
+    LIYAB_REQUIRE(n >= 0 && n <= 65535 && ff > 0 && ld >= 2 * static_cast<int64_t>(ff), "glu: bad sizes");
+    LIYAB_REQUIRE(act == 0 || act == 1, "glu: unknown activation %d", act);
+    if (n == 0) return 0;
+    dim3 grid((ff + EW_THREADS - 1) / EW_THREADS, n);
+    if (out_dtype == kF32) glu_kernel<float><<<grid, EW_THREADS, 0, stream>>>(static_cast<float*>(out), gu, ld, ff, act);
+    else if (out_dtype == kBF16) glu_kernel<bf16_t><<<grid, EW_THREADS, 0, stream>>>(static_cast<bf16_t*>(out), gu, ld, ff, act);
+    else return fail(1, "glu: unknown dtype %d", out_dtype);
+    return check_launch("glu");
 }
 
 extern "C" int liyab_activate(void* out, int out_dtype, int64_t ldo, const float* in, int64_t ldi, int op, int n, int d, hipStream_t stream) {

@@ -28,7 +28,7 @@ int liyab_pool_free_pages(void* p) { return static_cast<PagePool*>(p)->free_page
 int liyab_pool_peak(void* p) { return static_cast<PagePool*>(p)->peak_in_use(); }
 
 // -- the manager ------------------------------------------------------------------
-void* liyab_cm_create(int n_groups, const int* windows, const int* num_pages, int page_size, int max_requests,
+void* liyab_cm_create(int n_groups, const int* windows, const int* keep_first, const int* num_pages, int page_size, int max_requests,
                       int max_positions) {
     if (n_groups < 0 || page_size <= 0 || max_requests <= 0 || max_positions <= 0) {
         g_error = "cache manager: page_size, max_requests and max_positions must be positive";
@@ -40,7 +40,7 @@ void* liyab_cm_create(int n_groups, const int* windows, const int* num_pages, in
             g_error = "a page pool needs at least one page";
             return nullptr;
         }
-        groups.push_back({windows[g], num_pages[g]});
+        groups.push_back({windows[g], num_pages[g], keep_first[g]});
     }
     return new CacheManager(groups, page_size, max_requests, max_positions);
 }

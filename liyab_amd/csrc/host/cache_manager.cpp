@@ -58,6 +58,7 @@ CacheManager::CacheManager(const std::vector<GroupConfig>& groups, int page_size
       max_blocks_(std::max(1, (max_positions + page_size - 1) / page_size)), reqs_(static_cast<size_t>(max_requests)) {
     for (const GroupConfig& g : groups) {
         windows_.push_back(g.window);
+        keep_first_.push_back(g.window > 0 ? std::max(0, g.keep_first) : 0);
         pools_.emplace_back(g.num_pages);
         table_rows_.emplace_back(static_cast<size_t>(max_requests) * max_blocks_, kUnmapped);
     }
@@ -140,8 +141,9 @@ Status CacheManager::commit(int slot, int new_length, std::string* err) {
         if (windows_[g] <= 0) continue;
         const int first_needed = std::max(0, new_length - windows_[g] + 1);
         const int keep_from = std::min(first_needed / page_size_, r.mapped[g]);
+        if (keep_from <= kept_pages(g)) continue;  // (the window still touches the pages that stay)
         int32_t* t = row(g, slot);
-        for (int lp = r.first_kept[g]; lp < keep_from; ++lp) {
+        for (int lp = std::max(r.first_kept[g], kept_pages(g)); lp < keep_from; ++lp) {
             if (t[lp] != kUnmapped) {
                 if (Status s = pools_[g].release(&t[lp], 1, err)) return s;
                 t[lp] = kUnmapped;

@@ -57,6 +57,7 @@ private:
 struct GroupConfig {
     int window;     // 0: every position is kept; W > 0: only the last W are read
     int num_pages;
+    int keep_first = 0;  // with a window: the first `keep_first` positions are read too, however far back
 };
 
 class CacheManager {
@@ -81,7 +82,7 @@ public:
     // Maps pages so that each request can hold new_lengths[i] positions: all or nothing.
     Status reserve(const int* slots, const int* new_lengths, int n, std::string* err);
     // The request now holds new_length positions; windowed groups give back the pages no
-    // later query can see (a query at p >= length reads [p - W + 1, p]).
+    // later query can see (a query at p >= length reads [p - W + 1, p] and, where the group keeps them, the first positions).
     Status commit(int slot, int new_length, std::string* err);
     // Forgets positions >= length; pages wholly past it are given back (kv_cache.cpp:418-439).
     Status truncate(int slot, int length, std::string* err);
@@ -95,14 +96,15 @@ private:
         bool open = false;
         int length = 0;                 // positions committed
         std::vector<int> mapped;        // per group: logical pages in the table (mapped or released)
-        std::vector<int> first_kept;    // per group: first logical page still mapped
+        std::vector<int> first_kept;    // per group: first logical page still mapped (behind the pages that are always kept)
     };
+    int kept_pages(int g) const { return pages_for(keep_first_[g]); }  // logical pages that no window passes
     int pages_for(int n_positions) const { return (n_positions + page_size_ - 1) / page_size_; }
     int32_t* row(int g, int slot) { return table_rows_[g].data() + static_cast<size_t>(slot) * max_blocks_; }
     const int32_t* row(int g, int slot) const { return table_rows_[g].data() + static_cast<size_t>(slot) * max_blocks_; }
 
     int page_size_, max_requests_, max_positions_, max_blocks_;
-    std::vector<int> windows_;
+    std::vector<int> windows_, keep_first_;
     std::vector<PagePool> pools_;
     std::vector<Request> reqs_;
     std::vector<int> free_slots_;

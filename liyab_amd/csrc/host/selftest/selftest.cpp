@@ -35,7 +35,7 @@ static int run(unsigned seed, int n_steps) {
     const int windowed = pick(0, 1), window = pick(5, 60);
     const int need_alone = (max_positions + page - 1) / page;
     std::vector<GroupConfig> groups{{0, need_alone + pick(0, 2 * need_alone)}};
-    if (windowed) groups.push_back({window, need_alone + pick(0, need_alone)});
+    if (windowed) groups.push_back({window, need_alone + pick(0, need_alone), pick(0, 1) * pick(0, 40)});
     CacheManager m(groups, page, max_requests, max_positions);
     Scheduler s(&m, pick(1, max_requests), pick(4, 96), pick(2, 64));
     std::string err;

@@ -63,7 +63,7 @@ int liyab_rmsnorm(void* out, int out_dtype, const float* x, const float* w, cons
 int liyab_gated_norm_add(float* x, void* cast_out, int cast_dtype, const float* y, int n_sum, const float* gate, int64_t gate_stride,
                          const float* w, float eps, int normalize, int n, int d, float* state, int ring, int n_slots,
                          const int* tok_seq, const int* positions, const int* context_lens, const int* state_slots, const int* n_real,
-                         const float* next_w, float next_eps, hipStream_t stream);
+                         const float* next_w, float next_eps, const float* b, hipStream_t stream);
 int liyab_causal_conv(void* out, void* cast_out, int dtype, const float* x, const float* w, int taps, const float* state, int n_slots,
                       const int* tok_seq, const int* positions, const int* seq_starts, const int* state_slots, int n, int d,
                       hipStream_t stream);
@@ -76,9 +76,10 @@ int liyab_grouped_product(const void* a, int64_t lda, int a_div, int a_group_col
                           int block, int n_groups, const float* row_scale, const void* gate, int gate_dtype, int64_t gate_stride, int M, int N,
                           int K, int act, int out_div, int out_extra, hipStream_t stream);
 int liyab_moe_route(const float* logits, int64_t ld, int n, int n_experts, int top, int* ids, float* weights, int mode, int n_groups, int keep,
-                    hipStream_t stream);
+                    const float* correction, hipStream_t stream);
 int liyab_moe_route_align(const float* logits, int64_t ld, int n, int n_experts, int top, int* ids, float* weights, int block,
-                          int* rows_list, int* tile_group, int max_tiles, int mode, int n_groups, int keep, hipStream_t stream);
+                          int* rows_list, int* tile_group, int max_tiles, int mode, int n_groups, int keep, const float* correction,
+                          hipStream_t stream);
 int liyab_moe_align(const int* ids, int n_entries, int n_experts, int block, int* rows_list, int* tile_group, int max_tiles,
                     hipStream_t stream);
 
@@ -86,16 +87,17 @@ int liyab_attention_decode_scored(void* out, int64_t out_stride, const void* q, 
                                   const int* block_tables, int max_blocks, const int* tok_list, const int* tok_seq, const int* tok_pos, int n,
                                   float scale, int window, int n_head, int n_kv_head, int hd, int page_size, int n_splits, int chunk,
                                   int waves, int rows_are_requests, float* partials, int leave_splits, int num_pages, float softcap,
-                                  const float* bias_table, int max_dist, const float* sinks, hipStream_t stream);
+                                  const float* bias_table, int max_dist, const float* sinks, int keep_first, hipStream_t stream);
 int liyab_attention_prefill_scored(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* kc, const void* vc,
                                    const int* block_tables, int max_blocks, const int* work, int n_tiles, int tile, int ksplit, float scale,
                                    int window, int n_head, int n_kv_head, int hd, int page_size, int num_pages, float softcap,
-                                   const float* bias_table, int max_dist, const float* sinks, hipStream_t stream);
+                                   const float* bias_table, int max_dist, const float* sinks, int keep_first, hipStream_t stream);
 int liyab_gate_rows(void* x, int dtype, int64_t ldx, const float* gate, int64_t ldg, int n, int d, float scale, hipStream_t stream);
 int liyab_dyt(void* out, int out_dtype, const float* x, const float* w, const float* b, const float* alpha, const int* rows, int n, int d,
               hipStream_t stream);
 int liyab_glu_clamped(void* out, int out_dtype, const float* gu, int64_t ld, int n, int ff, float limit, float slope, float shift,
                       hipStream_t stream);
+int liyab_glu(void* out, int out_dtype, const float* gu, int64_t ld, int n, int ff, int act, hipStream_t stream);
 int liyab_activate(void* out, int out_dtype, int64_t ldo, const float* in, int64_t ldi, int op, int n, int d, hipStream_t stream);
 int liyab_mean_norm_add(float* x, const float* a, const float* b, const float* wa, const float* wb, float eps, float weight, int n, int d,
                         hipStream_t stream);
@@ -110,6 +112,16 @@ int liyab_ssd_scan(float* y, int64_t ldy, const float* xbc, int64_t ldx, const f
                    int64_t keep_ld, int keep_width, int keep_ring, int64_t keep_off, const int* seq_starts, const int* positions,
                    const int* state_slots, int n_seqs, int H, int P, int N, int G, int seg_tokens, int max_segs, float* seg_state,
                    float* seg_decay, hipStream_t stream);
+int liyab_gla_decay(float* out, const float* low, int64_t ldl, const float* w2t, const float* bias, float tau, int n, int C, int rank,
+                    hipStream_t stream);
+int liyab_gla_scan(void* out, int out_dtype, const float* q, const float* k, const float* v, const float* gate, int64_t ld, const float* decay,
+                   int64_t ldw, const float* norm_w, float eps, float q_scale, float* state, int64_t state_stride, int n_slots,
+                   const int* seq_starts, const int* positions, const int* state_slots, int n_seqs, int H, int R, int C, int seg_tokens,
+                   int max_segs, float* seg_state, float* seg_decay, hipStream_t stream);
+int liyab_gla_single(void* out, int out_dtype, const float* q, const float* k, const float* v, const float* gate, int64_t ld, const float* low,
+                     int64_t ldl, const float* w2t, const float* bias, float tau, const float* norm_w, float eps, float q_scale, float* state,
+                     int64_t state_stride, int n_slots, const int* seq_starts, const int* positions, const int* state_slots, int n_seqs, int H,
+                     int R, int C, int rank, hipStream_t stream);
 int liyab_token_shift(void* out, int dtype, const void* h, const float* mu, int n_mix, const float* state, int64_t state_stride, int n_slots,
                       const int* tok_seq, const int* positions, const int* seq_starts, const int* state_slots, int n, int d,
                       hipStream_t stream);
@@ -122,10 +134,15 @@ int liyab_qk_prepare(const float* src, int64_t ld, int q_off, int k_off, int v_o
                      void* q_out, void* kc, void* vc, int dtype, const int* slots, int page_size, int num_pages, const float* q_norm, const float* k_norm,
                      float eps, const double* freqs, int rot_dims, float temp_coef, int temp_every, const int* positions, int n,
                      int rot_halves, float rot_mag, float* v_keep, const float* v_first, const float* v_lam, hipStream_t stream);
+int liyab_qk_prepare_rows(const float* src, int64_t ld, int q_off, int k_off, int v_off, int H, int G, int dk, int dv, int dk_out, int dv_out,
+                          void* q_out, void* kc, void* vc, int dtype, const int* slots, int page_size, int num_pages, const float* q_norm,
+                          const float* k_norm, float eps, const double* freqs, int rot_dims, const int* positions, int n, int rot_halves,
+                          hipStream_t stream);
 int liyab_attention_scored(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* kc, const void* vc, int dtype,
                            const int* block_tables, int max_blocks, const int* tok_seq, const int* tok_pos, int n, float scale,
                            float softcap, int window, const float* bias_table, int max_dist, const float* gate, int64_t gate_stride,
-                           int n_head, int n_kv_head, int dk, int dv, int page_size, int num_pages, const float* sinks, hipStream_t stream);
+                           int n_head, int n_kv_head, int dk, int dv, int page_size, int num_pages, const float* sinks, int keep_first,
+                           hipStream_t stream);
 
 int liyab_norm_shift(void* out, int out_dtype, float* hbuf, const float* x, const float* w, float offset, float eps, const float* cw, int taps,
                      float* state, int64_t state_stride, int n_slots, const int* tok_seq, const int* positions, const int* seq_starts,
@@ -145,8 +162,20 @@ int liyab_delta_single(void* out, int out_dtype, const float* r, const float* k,
                        const float* wraw, int64_t ldw, const float* w0, const float* a_bias, const float* norm_w, float eps, float decay_scale,
                        float key_eps, float* state, int64_t state_stride, int n_slots, const int* seq_starts, const int* positions,
                        const int* state_slots, int n_seqs, int H, int D, hipStream_t stream);
-int liyab_head_norm_gate(void* out, int out_dtype, const float* o, const float* gate, int64_t ldg, const float* w, float eps, int n, int H, int D,
-                         hipStream_t stream);
+int liyab_head_norm_gate(void* out, int out_dtype, const float* o, const float* gate, int64_t ldg, const float* w, int shared_w, float eps, int n,
+                         int H, int D, int silu, hipStream_t stream);
+int liyab_gated_delta_takes(int D, int V);
+int liyab_gated_delta_prepare(float* prep, const float* src, int64_t ld, const float* cw, int taps, const float* ring, int64_t state_stride, int n_slots,
+                              const float* a_log, const float* dt_bias, int b_off, int a_off, float key_eps, float q_scale, const int* tok_seq,
+                              const int* positions, const int* seq_starts, const int* state_slots, int n, int H, int G, int D, int V,
+                              hipStream_t stream);
+int liyab_gated_delta_scan(float* out, const float* prep, const float* src, int64_t ld, int taps, float* state, int64_t state_stride, int n_slots,
+                           const int* seq_starts, const int* positions, const int* state_slots, int n_seqs, int H, int G, int D, int V,
+                           int seg_tokens, int max_segs, float* seg_state, float* seg_trans, float* seg_start, hipStream_t stream);
+int liyab_gated_delta_single(void* out, int out_dtype, const float* src, int64_t ld, const float* cw, int taps, const float* a_log,
+                             const float* dt_bias, int g_off, int b_off, int a_off, const float* norm_w, float eps, float key_eps, float q_scale,
+                             float* state, int64_t state_stride, int n_slots, const int* seq_starts, const int* positions, const int* state_slots,
+                             int n_seqs, int H, int G, int D, int V, hipStream_t stream);
 int liyab_maps_store(const float* src, int64_t ld, const float* cw, int taps, float* state, int64_t state_stride, int n_slots, void* q_out,
                      void* k1, void* k2, void* vc, int dtype, const int* slots, int page_size, int num_pages, const int* tok_seq,
                      const int* positions, const int* seq_starts, const int* state_slots, int n, int H, int G, int D, int V, int P,

@@ -1,16 +1,18 @@
 // Mixers that carry a matrix of state from token to token instead of keys: the recurrence itself and
 // what stands around it.
 //
-// Both recurrences here keep, a head, a matrix S [rows, cols] of 32-bit floats a request:
+// The recurrences here keep, a head, a matrix S [rows, cols] of 32-bit floats a request:
 //   decayed outer products with a bonus (a "wkv" head; rows = key channels, cols = value channels):
 //       o_t = (S + diag(u) k_t v_t^T)^T r_t,      S <- diag(w_t) S + k_t v_t^T,   w_t = exp(-exp(wraw_t + w0))
 //   a selective state space (rows = state size, cols = the head's channels), a = exp(-exp(A_log) dt_t):
 //       S <- a S + dt_t B_t x_t^T,                y_t = S^T C_t + D x_t,          dt_t = softplus(dtraw_t + dt_bias)
-// One kernel serves both: a workgroup a (request, head) walks the request's tokens of the step in order.
+//   gated linear attention (rows = key channels, cols = value channels, of widths of their own), a decay a key channel:
+//       S <- diag(w_t) S + k_t v_t^T,             o_t = S^T (q_t * q_scale),      w_t = sigmoid(z_t)^(1 / tau) (liyab_gla_decay)
+// One kernel serves all three: a workgroup a (request, head) walks the request's tokens of the step in order.
 // A thread owns one column of a block of rows of S in registers, so nothing of the state moves between
 // threads; a token's vectors are staged through LDS sixteen tokens at a time (one trip to memory a
 // chunk, not a token), the threads leave partial sums of the outputs in LDS, and after the chunk the
-// workgroup adds them up and finishes the rows (a wkv head: unit root mean square over the head, the
+// workgroup adds them up and finishes the rows (a wkv or gated-linear head: unit root mean square over the head, the
 // weight, the gate silu(g); a state-space head: + D x). The state comes from the request's slot (zeros
 // at position 0 whatever the slot still holds) and goes back to it. The workgroup of head 0 also keeps
 // the request's last input rows for the next step (the previous token's input of a token shift, the last
@@ -21,6 +23,8 @@
 // strings a request's segments together and leaves each the state it starts from; every segment again from that state,
 // with outputs. Decays are only ever multiplied, and the grids follow from the step's rows and requests alone.
 //
+// liyab_gla_decay: the decays of gated linear attention from a low-rank product, z = W2 low + b in 32-bit, w = sigmoid(z)^(1 / tau).
+// liyab_gla_single: a step of single tokens of gated linear attention (decays included) in one kernel, a workgroup a (request, head).
 // liyab_token_shift: m_c[t] = h[t] + (h[t - 1] - h[t]) * mu_c for each of n_mix learned mixes (a token's mixes side by side
 //   in its row of the output, [n, n_mix * d]), the previous
 //   row taken from the step's rows, from the request's slot, or zero at position 0.
@@ -61,7 +65,7 @@ struct ScanArgs {
     const float *r, *k, *v, *wraw, *gate;
     int64_t ld;
     const float *w0, *u, *norm_w;
-    float eps;
+    float eps, q_scale;     // (q_scale: gated linear attention; its decays are wraw, rows of ldp floats)
     void* out;              // wkv: rows in the compute type [n, H * cols]; ssd: float [n, ldy]
     // ssd
     const float* xbc;       // [n, ldx]: x at 0, B at inner, C at inner + G * rows
@@ -148,6 +152,11 @@ scan_kernel(ScanArgs a) {
             d = a.wraw[at] + a.w0[h * R + ic];
             x = a.k[at];
             q = a.r[at];
+        } else if (MODE == 2) {
+            const int64_t at = t * a.ld + h * R + ic;
+            d = a.wraw[t * a.ldp + h * R + ic];
+            x = a.k[at];
+            q = a.r[at] * a.q_scale;
         } else {
             d = a.dtraw[t * a.ldp + h];
             x = a.xbc[t * a.ldx + a.inner + g * R + ic];
@@ -157,7 +166,7 @@ scan_kernel(ScanArgs a) {
     auto raw_val = [&](int c0, int len, int tt, int jj) {
         const int64_t t = c0 + min(tt, len - 1);
         const int jc = min(jj, C - 1);
-        return MODE == 0 ? a.v[t * a.ld + h * C + jc] : a.xbc[t * a.ldx + h * C + jc];
+        return MODE != 1 ? a.v[t * a.ld + h * C + jc] : a.xbc[t * a.ldx + h * C + jc];
     };
     auto raw_gate = [&](int c0, int len, int tt, int jj) {
         return a.gate[static_cast<int64_t>(c0 + min(tt, len - 1)) * a.ld + h * C + min(jj, C - 1)];
@@ -168,6 +177,9 @@ scan_kernel(ScanArgs a) {
             const bool real = i < R;
             if (MODE == 0) {
                 decay[e] = real ? expf(-expf(d)) : 0.0f;
+                inr[e] = real ? x : 0.0f;
+            } else if (MODE == 2) {
+                decay[e] = real ? d : 0.0f;
                 inr[e] = real ? x : 0.0f;
             } else {
                 const float dt = softplus_f(d + dtb);
@@ -189,7 +201,7 @@ scan_kernel(ScanArgs a) {
         vt[k] = e >> cl_shift;
         vc[k] = e & (CL - 1);
     }
-    float* gates = part + SCAN_CHUNK * SCAN_THREADS;  // [CHUNK][CL] (wkv): silu of the gate's logits
+    float* gates = part + SCAN_CHUNK * SCAN_THREADS;  // [CHUNK][CL] (not the state space): silu of the gate's logits
     auto fetch = [&](int from) {  // (past the request's last token: its last token once more, never staged)
         const int c0 = min(from, end - 1);
         const int len = min(SCAN_CHUNK, end - c0);
@@ -197,7 +209,7 @@ scan_kernel(ScanArgs a) {
         for (int k = 0; k < NPF; ++k) {
             raw_rows(c0, len, rt[k], ri[k], pd[k], px[k], pq[k]);
             pv[k] = raw_val(c0, len, vt[k], vc[k]);
-            if (MODE == 0) pg[k] = raw_gate(c0, len, vt[k], vc[k]);
+            if (MODE != 1) pg[k] = raw_gate(c0, len, vt[k], vc[k]);
         }
     };
     if (PF > 0) fetch(begin);
@@ -211,7 +223,7 @@ scan_kernel(ScanArgs a) {
                 put_rows(len, rt[k], ri[k], pd[k], px[k], pq[k]);
                 if (vt[k] < len) {
                     val[vt[k] * CL + vc[k]] = vc[k] < C ? pv[k] : 0.0f;
-                    if (MODE == 0) gates[vt[k] * CL + vc[k]] = silu_f(pg[k]);
+                    if (MODE != 1) gates[vt[k] * CL + vc[k]] = silu_f(pg[k]);
                 }
             }
         } else {
@@ -222,7 +234,7 @@ scan_kernel(ScanArgs a) {
             }
             for (int e = tid; e < len * CL; e += SCAN_THREADS) {
                 val[e] = (e & (CL - 1)) < C ? raw_val(c0, len, e >> cl_shift, e & (CL - 1)) : 0.0f;
-                if (MODE == 0) gates[e] = silu_f(raw_gate(c0, len, e >> cl_shift, e & (CL - 1)));
+                if (MODE != 1) gates[e] = silu_f(raw_gate(c0, len, e >> cl_shift, e & (CL - 1)));
             }
         }
         __syncthreads();
@@ -289,7 +301,7 @@ scan_kernel(ScanArgs a) {
         else tokens(std::false_type{});
         __syncthreads();
         if (a.phase == 1) continue;  // (no outputs in pass 1)
-        if (MODE == 0) {
+        if (MODE != 1) {
             // a wave a token: the head's outputs, their root mean square, the weight and the gate
             const int wave = tid / kWave, lane = tid % kWave;
             for (int tt = wave; tt < len; tt += SCAN_THREADS / kWave) {
@@ -305,7 +317,7 @@ scan_kernel(ScanArgs a) {
                     float o = 0.0f;
                     for (int b = 0; b < n_rb; ++b) o += part[(tt * n_rb + b) * CL + jj];
                     const int col = h * C + jj;
-                    const float y = o * rinv * a.norm_w[col] * gates[tt * CL + jj];
+                    const float y = o * rinv * a.norm_w[MODE == 2 ? jj : col] * gates[tt * CL + jj];
                     static_cast<OutT*>(a.out)[t * (static_cast<int64_t>(a.H) * C) + col] = from_float<OutT>(y);
                 }
             }
@@ -446,6 +458,129 @@ static void launch_scan(const ScanArgs& a, int n_seqs, int reg, int pf, size_t s
     if (pf == 4) launch_scan_pf<MODE, OutT, 4>(a, n_seqs, reg, smem, stream);
     else if (pf == 8) launch_scan_pf<MODE, OutT, 8>(a, n_seqs, reg, smem, stream);
     else launch_scan_pf<MODE, OutT, 0>(a, n_seqs, reg, smem, stream);
+}
+
+// Decays of gated linear attention: a thread a channel, eight tokens at a time, so that a weight is read once for eight sums.
+constexpr int kGlaTokens = 8;
+
+__device__ __forceinline__ float gla_decay_of(float z, float inv_tau) {
+    // sigmoid(z)^(1 / tau) through its logarithm, -softplus(-z), which loses nothing at either end
+    return expf((fminf(z, 0.0f) - log1pf(expf(-fabsf(z)))) * inv_tau);
+}
+
+__global__ void __launch_bounds__(256)
+gla_decay_kernel(float* __restrict__ out, const float* __restrict__ low, int64_t ldl, const float* __restrict__ w2t, const float* __restrict__ bias,
+                 float inv_tau, int n, int C, int rank) {
+    const int c = blockIdx.x * 256 + threadIdx.x, t0 = blockIdx.y * kGlaTokens;
+    if (c >= C) return;
+    float acc[kGlaTokens];
+    const float b = bias[c];
+#pragma unroll
+    for (int i = 0; i < kGlaTokens; ++i) acc[i] = b;
+    for (int r = 0; r < rank; ++r) {
+        const float w = w2t[static_cast<int64_t>(r) * C + c];
+#pragma unroll
+        for (int i = 0; i < kGlaTokens; ++i) acc[i] = fmaf(w, low[static_cast<int64_t>(min(t0 + i, n - 1)) * ldl + r], acc[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < kGlaTokens; ++i)
+        if (t0 + i < n) out[static_cast<int64_t>(t0 + i) * C + c] = gla_decay_of(acc[i], inv_tau);
+}
+
+struct GlaSingleArgs {
+    void* out;                        // [n, H * C], the compute type
+    const float *q, *k, *v, *gate;    // rows of ld floats
+    int64_t ld;
+    const float* low;                 // rows of ldl floats, `rank` of them used
+    int64_t ldl;
+    const float *w2t, *bias, *norm_w; // [rank, H * R], [H * R], [C]
+    float inv_tau, eps, q_scale;
+    float* state;
+    int64_t state_stride;
+    int n_slots;
+    const int* seq_starts;
+    const int* positions;
+    const int* state_slots;
+    int H, R, C, rank;
+};
+
+// Four lanes side by side share a column of S, each with a quarter of its rows in registers; four waves take 64 columns at a time.
+constexpr int kGlaMax = 256;
+
+template <typename T, int REG>
+__global__ void __launch_bounds__(256)
+gla_single_kernel(GlaSingleArgs a) {
+    constexpr int RP = 4 * REG;
+    __shared__ __attribute__((aligned(16))) float vec[3 * RP];  // decays, keys, scaled queries, zeros behind the last row
+    __shared__ float o_s[kGlaMax];
+    __shared__ float red[4];
+    const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave;
+    const int h = blockIdx.x % a.H, s = blockIdx.x / a.H;
+    const int t = a.seq_starts[s];
+    if (a.seq_starts[s + 1] - t != 1) return;  // (the host sends steps of single tokens only)
+    const int R = a.R, C = a.C;
+    const int slot = a.state_slots[s];
+    const bool slot_ok = slot >= 0 && slot < a.n_slots;
+    const bool fresh = a.positions[t] == 0;
+    float* Sg = a.state + static_cast<int64_t>(slot_ok ? slot : 0) * a.state_stride + static_cast<int64_t>(h) * R * C;
+    const int rb = lane % 4, i0 = rb * REG, j0 = wave * 16 + lane / 4;
+    // the first block of columns is on its way while the vectors are made
+    float S[REG];
+    auto load = [&](int j) {
+#pragma unroll
+        for (int ii = 0; ii < REG; ++ii) {
+            const float val = Sg[static_cast<int64_t>(min(i0 + ii, R - 1)) * C + min(j, C - 1)];
+            S[ii] = (i0 + ii < R && j < C && slot_ok && !fresh) ? val : 0.0f;
+        }
+    };
+    load(j0);
+    for (int i = tid; i < RP; i += 256) {
+        const bool in = i < R;
+        const int64_t at = static_cast<int64_t>(t) * a.ld + h * R + (in ? i : 0);
+        float z = a.bias[h * R + (in ? i : 0)];
+        for (int r = 0; r < a.rank; ++r)
+            z = fmaf(a.w2t[static_cast<int64_t>(r) * a.H * R + h * R + (in ? i : 0)], a.low[static_cast<int64_t>(t) * a.ldl + r], z);
+        const float k = a.k[at], q = a.q[at];
+        vec[i] = in ? gla_decay_of(z, a.inv_tau) : 0.0f;
+        vec[RP + i] = in ? k : 0.0f;
+        vec[2 * RP + i] = in ? q * a.q_scale : 0.0f;
+    }
+    __syncthreads();
+    float ss = 0.0f;
+    for (int c0 = 0; c0 < C; c0 += 64) {
+        const int j = c0 + j0;
+        if (c0 > 0) load(j);
+        const float v = j < C ? a.v[static_cast<int64_t>(t) * a.ld + h * C + j] : 0.0f;
+        float acc[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+        for (int q4 = 0; q4 < REG / 4; ++q4) {
+            const f32x4_t w4 = *reinterpret_cast<const f32x4_t*>(vec + i0 + 4 * q4), k4 = *reinterpret_cast<const f32x4_t*>(vec + RP + i0 + 4 * q4),
+                          r4 = *reinterpret_cast<const f32x4_t*>(vec + 2 * RP + i0 + 4 * q4);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                float& x = S[4 * q4 + e];
+                x = fmaf(w4[e], x, k4[e] * v);
+                acc[e] = fmaf(r4[e], x, acc[e]);
+            }
+        }
+        const float o = group_sum<4>((acc[0] + acc[1]) + (acc[2] + acc[3]));
+        if (rb == 0 && j < C) {
+            o_s[j] = o;
+            ss = fmaf(o, o, ss);
+        }
+        if (slot_ok) {
+#pragma unroll
+            for (int ii = 0; ii < REG; ++ii)
+                if (i0 + ii < R && j < C) Sg[static_cast<int64_t>(i0 + ii) * C + j] = S[ii];
+        }
+    }
+    ss = wave_sum(ss);
+    if (lane == 0) red[wave] = ss;
+    __syncthreads();
+    const float rinv = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / static_cast<float>(C) + a.eps);
+    if (tid < C)
+        static_cast<T*>(a.out)[(static_cast<int64_t>(t) * a.H + h) * C + tid] =
+            from_float<T>(o_s[tid] * rinv * a.norm_w[tid] * silu_f(a.gate[static_cast<int64_t>(t) * a.ld + h * C + tid]));
 }
 
 template <typename T>
@@ -589,6 +724,66 @@ extern "C" int liyab_ssd_scan(float* y, int64_t ldy, const float* xbc, int64_t l
     a.G = G; a.inner = static_cast<int>(inner);
     launch_scan<1, float>(a, n_seqs, reg, pf, smem, stream);
     return check_launch("ssd_scan");
+}
+
+extern "C" int liyab_gla_decay(float* out, const float* low, int64_t ldl, const float* w2t, const float* bias, float tau, int n, int C, int rank,
+                               hipStream_t stream) {
+    LIYAB_REQUIRE(out && low && w2t && bias, "gla_decay: null pointer");
+    LIYAB_REQUIRE(n >= 0 && C > 0 && rank > 0 && ldl >= rank && tau > 0.0f, "gla_decay: bad sizes");
+    LIYAB_REQUIRE((n + kGlaTokens - 1) / kGlaTokens <= 65535, "gla_decay: too many tokens");
+    if (n == 0) return 0;
+    gla_decay_kernel<<<dim3((C + 255) / 256, (n + kGlaTokens - 1) / kGlaTokens), 256, 0, stream>>>(out, low, ldl, w2t, bias, 1.0f / tau, n, C, rank);
+    return check_launch("gla_decay");
+}
+
+extern "C" int liyab_gla_scan(void* out, int out_dtype, const float* q, const float* k, const float* v, const float* gate, int64_t ld,
+                              const float* decay, int64_t ldw, const float* norm_w, float eps, float q_scale, float* state, int64_t state_stride,
+                              int n_slots, const int* seq_starts, const int* positions, const int* state_slots, int n_seqs, int H, int R, int C,
+                              int seg_tokens, int max_segs, float* seg_state, float* seg_decay, hipStream_t stream) {
+    LIYAB_REQUIRE(out && q && k && v && gate && decay && norm_w && state && seq_starts && positions && state_slots, "gla_scan: null pointer");
+    LIYAB_REQUIRE(n_seqs >= 0 && H > 0 && R > 0 && C > 0 && n_slots > 0, "gla_scan: bad sizes");
+    LIYAB_REQUIRE(ld >= static_cast<int64_t>(H) * R && ld >= static_cast<int64_t>(H) * C && ldw >= static_cast<int64_t>(H) * R, "gla_scan: rows shorter than the heads");
+    LIYAB_REQUIRE(state_stride >= static_cast<int64_t>(H) * R * C, "gla_scan: a slot of %lld floats does not hold the state", static_cast<long long>(state_stride));
+    ScanArgs a = {};
+    size_t smem;
+    int reg, pf;
+    LIYAB_REQUIRE(scan_shape(R, C, &a.col_lanes, &a.rows_per, &reg, &pf, &smem), "gla_scan: a state of %d x %d a head is not taken", R, C);
+    if (n_seqs == 0) return 0;
+    LIYAB_REQUIRE(seg_tokens >= 0 && (seg_tokens == 0 || (max_segs > 0 && seg_state && seg_decay)), "scan: segments need their count and scratch");
+    a.n_seqs = n_seqs; a.seg_tokens = seg_tokens; a.max_segs = max_segs; a.seg_state = seg_state; a.seg_decay = seg_decay;
+    a.state = state; a.state_stride = state_stride; a.n_slots = n_slots;
+    a.seq_starts = seq_starts; a.positions = positions; a.state_slots = state_slots;
+    a.H = H; a.rows = R; a.cols = C;
+    a.r = q; a.k = k; a.v = v; a.gate = gate; a.ld = ld; a.wraw = decay; a.ldp = ldw; a.norm_w = norm_w; a.eps = eps; a.q_scale = q_scale; a.out = out;
+    if (out_dtype == kF32) launch_scan<2, float>(a, n_seqs, reg, pf, smem, stream);
+    else if (out_dtype == kBF16) launch_scan<2, bf16_t>(a, n_seqs, reg, pf, smem, stream);
+    else return fail(1, "gla_scan: unknown dtype %d", out_dtype);
+    return check_launch("gla_scan");
+}
+
+extern "C" int liyab_gla_single(void* out, int out_dtype, const float* q, const float* k, const float* v, const float* gate, int64_t ld,
+                                const float* low, int64_t ldl, const float* w2t, const float* bias, float tau, const float* norm_w, float eps,
+                                float q_scale, float* state, int64_t state_stride, int n_slots, const int* seq_starts, const int* positions,
+                                const int* state_slots, int n_seqs, int H, int R, int C, int rank, hipStream_t stream) {
+    LIYAB_REQUIRE(out && q && k && v && gate && low && w2t && bias && norm_w && state && seq_starts && positions && state_slots, "gla_single: null pointer");
+    LIYAB_REQUIRE(n_seqs >= 0 && H > 0 && R > 0 && C > 0 && R <= kGlaMax && C <= kGlaMax && rank > 0 && n_slots > 0 && tau > 0.0f, "gla_single: bad sizes");
+    LIYAB_REQUIRE(ld >= static_cast<int64_t>(H) * R && ld >= static_cast<int64_t>(H) * C && ldl >= rank, "gla_single: rows shorter than the heads");
+    LIYAB_REQUIRE(state_stride >= static_cast<int64_t>(H) * R * C, "gla_single: a slot of %lld floats does not hold the state", static_cast<long long>(state_stride));
+    LIYAB_REQUIRE(out_dtype == kF32 || out_dtype == kBF16, "gla_single: unknown dtype %d", out_dtype);
+    if (n_seqs == 0) return 0;
+    const GlaSingleArgs a{out, q, k, v, gate, ld, low, ldl, w2t, bias, norm_w, 1.0f / tau, eps, q_scale, state, state_stride, n_slots,
+                          seq_starts, positions, state_slots, H, R, C, rank};
+    const unsigned grid = static_cast<unsigned>(n_seqs) * static_cast<unsigned>(H);
+    auto run = [&](auto zero) {
+        using T = decltype(zero);
+        if (R <= 32) gla_single_kernel<T, 8><<<grid, 256, 0, stream>>>(a);
+        else if (R <= 64) gla_single_kernel<T, 16><<<grid, 256, 0, stream>>>(a);
+        else if (R <= 128) gla_single_kernel<T, 32><<<grid, 256, 0, stream>>>(a);
+        else gla_single_kernel<T, 64><<<grid, 256, 0, stream>>>(a);
+    };
+    if (out_dtype == kF32) run(float{});
+    else run(bf16_t{});
+    return check_launch("gla_single");
 }
 
 extern "C" int liyab_token_shift(void* out, int dtype, const void* h, const float* mu, int n_mix, const float* state, int64_t state_stride,

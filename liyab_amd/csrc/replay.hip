@@ -102,14 +102,19 @@ static const Entry kEntries[] = {
     LIYAB_ENTRY(liyab_gate_rows),
     LIYAB_ENTRY(liyab_dyt),
     LIYAB_ENTRY(liyab_glu_clamped),
+    LIYAB_ENTRY(liyab_glu),
     LIYAB_ENTRY(liyab_activate),
     LIYAB_ENTRY(liyab_mean_norm_add),
     LIYAB_ENTRY(liyab_wkv_scan),
     LIYAB_ENTRY(liyab_ssd_scan),
+    LIYAB_ENTRY(liyab_gla_decay),
+    LIYAB_ENTRY(liyab_gla_scan),
+    LIYAB_ENTRY(liyab_gla_single),
     LIYAB_ENTRY(liyab_token_shift),
     LIYAB_ENTRY(liyab_conv_act),
     LIYAB_ENTRY(liyab_gated_group_norm),
     LIYAB_ENTRY(liyab_qk_prepare),
+    LIYAB_ENTRY(liyab_qk_prepare_rows),
     LIYAB_ENTRY(liyab_attention_scored),
     LIYAB_ENTRY(liyab_norm_shift),
     LIYAB_ENTRY(liyab_ring_keep),
@@ -119,6 +124,9 @@ static const Entry kEntries[] = {
     LIYAB_ENTRY(liyab_delta_scan),
     LIYAB_ENTRY(liyab_delta_single),
     LIYAB_ENTRY(liyab_head_norm_gate),
+    LIYAB_ENTRY(liyab_gated_delta_prepare),
+    LIYAB_ENTRY(liyab_gated_delta_scan),
+    LIYAB_ENTRY(liyab_gated_delta_single),
     LIYAB_ENTRY(liyab_maps_store),
     LIYAB_ENTRY(liyab_maps_join),
     LIYAB_ENTRY(liyab_weighted_sum),

@@ -8,7 +8,8 @@
 //   s = (y_0 + ... + y_{n_sum-1}) * sigmoid(g),   x += w * s / sqrt(mean(s^2) + eps)
 // y: the sublayer's 32-bit result, one row a token or n_sum consecutive rows a token that are
 // added in their order (a routed feed-forward leaves one row for each expert a token took);
-// without `normalize` the sum is added as it is (x += s);
+// without `normalize` the sum is added as it is (x += s); with normalize = 2 the norm takes the mean off first and adds a bias,
+// x += w * (s - mean(s)) / sqrt(mean((s - mean(s))^2) + eps) + b, the mean and the mean square in two passes over the row;
 // g: the gate's 32-bit logits (a pointer and a row stride, so that they may be columns of a wider
 // product), or none. The new row may also be written rounded to the compute type for the next
 // product (`cast_out`), or, with `next_w`, what the next sublayer reads of it: the new row's own root-mean-square norm under that
@@ -72,7 +73,7 @@ template <typename T, int THREADS, int MAXV>
 __global__ void __launch_bounds__(THREADS)
 gated_norm_add_kernel(float* __restrict__ x, T* __restrict__ cast_out, const float* __restrict__ y, int n_sum,
                       const float* __restrict__ gate, int64_t gate_stride, const float* __restrict__ w, float eps, int normalize, int d, KeepRows keep,
-                      const float* __restrict__ next_w, float next_eps) {
+                      const float* __restrict__ next_w, float next_eps, const float* __restrict__ b) {
     __shared__ float red[THREADS / kWave];
     const int t = blockIdx.x;
     float* xr = x + static_cast<int64_t>(t) * d;
@@ -88,7 +89,7 @@ gated_norm_add_kernel(float* __restrict__ x, T* __restrict__ cast_out, const flo
     const float* gr = gate != nullptr ? gate + static_cast<int64_t>(t) * gate_stride : nullptr;
     const bool held = d <= THREADS * MAXV;
     float sv[MAXV];
-    float ss = 0.0f;
+    float ss = 0.0f, mean = 0.0f;
     auto value = [&](int i) {
         float s = yr[i];
         for (int k = 1; k < n_sum; ++k) s += yr[static_cast<int64_t>(k) * d + i];
@@ -100,12 +101,28 @@ gated_norm_add_kernel(float* __restrict__ x, T* __restrict__ cast_out, const flo
         for (int j = 0; j < MAXV; ++j) {
             const int i = threadIdx.x + j * THREADS;
             sv[j] = i < d ? value(i) : 0.0f;
-            ss += sv[j] * sv[j];
+            ss += normalize == 2 ? sv[j] : sv[j] * sv[j];
         }
     } else {
         for (int i = threadIdx.x; i < d; i += THREADS) {
             const float s = value(i);
-            ss += s * s;
+            ss += normalize == 2 ? s : s * s;
+        }
+    }
+    if (normalize == 2) {
+        mean = rms_block_sum<THREADS>(ss, red) / static_cast<float>(d);
+        ss = 0.0f;
+        if (held) {
+#pragma unroll
+            for (int j = 0; j < MAXV; ++j) {
+                sv[j] -= mean;
+                if (threadIdx.x + j * THREADS < d) ss += sv[j] * sv[j];
+            }
+        } else {
+            for (int i = threadIdx.x; i < d; i += THREADS) {
+                const float s = value(i) - mean;
+                ss += s * s;
+            }
         }
     }
     const float scale = normalize ? 1.0f / sqrtf(rms_block_sum<THREADS>(ss, red) / static_cast<float>(d) + eps) : 1.0f;
@@ -115,6 +132,7 @@ gated_norm_add_kernel(float* __restrict__ x, T* __restrict__ cast_out, const flo
     auto finish = [&](int i, float s) {
         float v = s * scale;
         if (w != nullptr) v *= w[i];
+        if (b != nullptr) v += b[i];
         v += xr[i];
         xr[i] = v;
         if (norm_next) ss_new += v * v;
@@ -128,7 +146,7 @@ gated_norm_add_kernel(float* __restrict__ x, T* __restrict__ cast_out, const flo
             if (i < d) sv[j] = finish(i, sv[j]);
         }
     } else {
-        for (int i = threadIdx.x; i < d; i += THREADS) finish(i, value(i));
+        for (int i = threadIdx.x; i < d; i += THREADS) finish(i, value(i) - mean);
     }
     if (norm_next) {
         const float next_scale = 1.0f / sqrtf(rms_block_sum<THREADS>(ss_new, red) / static_cast<float>(d) + next_eps);
@@ -164,8 +182,9 @@ extern "C" int liyab_rmsnorm(void* out, int out_dtype, const float* x, const flo
 extern "C" int liyab_gated_norm_add(float* x, void* cast_out, int cast_dtype, const float* y, int n_sum, const float* gate,
                                     int64_t gate_stride, const float* w, float eps, int normalize, int n, int d, float* state, int ring, int n_slots,
                                     const int* tok_seq, const int* positions, const int* context_lens, const int* state_slots,
-                                    const int* n_real, const float* next_w, float next_eps, hipStream_t stream) {
+                                    const int* n_real, const float* next_w, float next_eps, const float* b, hipStream_t stream) {
     LIYAB_REQUIRE(x && y, "gated_norm_add: null pointer");
+    LIYAB_REQUIRE(normalize >= 0 && normalize <= 2, "gated_norm_add: unknown norm %d", normalize);
     LIYAB_REQUIRE(next_w == nullptr || cast_out != nullptr, "gated_norm_add: the next norm's rows need a place");
     LIYAB_REQUIRE(n >= 0 && d > 0 && n_sum >= 1, "gated_norm_add: bad sizes n=%d d=%d n_sum=%d", n, d, n_sum);
     LIYAB_REQUIRE(cast_dtype == kF32 || cast_dtype == kBF16, "gated_norm_add: unknown dtype %d", cast_dtype);
@@ -175,8 +194,8 @@ extern "C" int liyab_gated_norm_add(float* x, void* cast_out, int cast_dtype, co
     if (n == 0) return 0;
     const KeepRows keep{state, ring, n_slots, tok_seq, positions, context_lens, state_slots, n_real};
     if (cast_dtype == kF32)
-        gated_norm_add_kernel<float, 256, 8><<<n, 256, 0, stream>>>(x, static_cast<float*>(cast_out), y, n_sum, gate, gate_stride, w, eps, normalize, d, keep, next_w, next_eps);
+        gated_norm_add_kernel<float, 256, 8><<<n, 256, 0, stream>>>(x, static_cast<float*>(cast_out), y, n_sum, gate, gate_stride, w, eps, normalize, d, keep, next_w, next_eps, b);
     else
-        gated_norm_add_kernel<bf16_t, 256, 8><<<n, 256, 0, stream>>>(x, static_cast<bf16_t*>(cast_out), y, n_sum, gate, gate_stride, w, eps, normalize, d, keep, next_w, next_eps);
+        gated_norm_add_kernel<bf16_t, 256, 8><<<n, 256, 0, stream>>>(x, static_cast<bf16_t*>(cast_out), y, n_sum, gate, gate_stride, w, eps, normalize, d, keep, next_w, next_eps, b);
     return check_launch("gated_norm_add");
 }

@@ -41,7 +41,7 @@ _SIGNATURES = {
     "liyab_pool_check": ([c_void_p], c_int),
     "liyab_pool_free_pages": ([c_void_p], c_int),
     "liyab_pool_peak": ([c_void_p], c_int),
-    "liyab_cm_create": ([c_int, IP, IP, c_int, c_int, c_int], c_void_p),
+    "liyab_cm_create": ([c_int, IP, IP, IP, c_int, c_int, c_int], c_void_p),
     "liyab_cm_destroy": ([c_void_p], None),
     "liyab_cm_open": ([c_void_p, IP], c_int),
     "liyab_cm_close": ([c_void_p, c_int], c_int),

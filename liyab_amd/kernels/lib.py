@@ -74,35 +74,43 @@ _SIGNATURES = {
     "liyab_argmax_static": [P, P, c_int64, c_int, c_int, P, P, P],
     "liyab_sample": [P, P, c_int64, c_int, c_int, P, P, P, P, P, P, P],
     "liyab_rmsnorm": [P, c_int, P, P, P, c_int, c_int, c_float, P],
-    "liyab_gated_norm_add": [P, P, c_int, P, c_int, P, c_int64, P, c_float, c_int, c_int, c_int, P, c_int, c_int, P, P, P, P, P, P, c_float, P],
+    "liyab_gated_norm_add": [P, P, c_int, P, c_int, P, c_int64, P, c_float, c_int, c_int, c_int, P, c_int, c_int, P, P, P, P, P, P, c_float, P, P],
     "liyab_causal_conv": [P, P, c_int, P, P, c_int, P, c_int, P, P, P, P, c_int, c_int, P],
     "liyab_keep_rows": [P, c_int, c_int, P, P, P, P, P, P, c_int, c_int, P],
     "liyab_latent_store": [P, c_int, P, c_int64, c_int, P, c_float, P, c_int, c_int, c_int, c_int, P],
     "liyab_grouped_product": [P, c_int64, c_int, c_int, P, P, c_int, P, c_int, c_int64, c_int, P, P, c_int, c_int, c_int, P, P, c_int, c_int64,
                               c_int, c_int, c_int, c_int, c_int, c_int, P],
-    "liyab_moe_route": [P, c_int64, c_int, c_int, c_int, P, P, c_int, c_int, c_int, P],
+    "liyab_moe_route": [P, c_int64, c_int, c_int, c_int, P, P, c_int, c_int, c_int, P, P],
     "liyab_moe_align": [P, c_int, c_int, c_int, P, P, c_int, P],
-    "liyab_moe_route_align": [P, c_int64, c_int, c_int, c_int, P, P, c_int, P, P, c_int, c_int, c_int, c_int, P],
+    "liyab_moe_route_align": [P, c_int64, c_int, c_int, c_int, P, P, c_int, P, P, c_int, c_int, c_int, c_int, P, P],
     "liyab_attention_decode_scored": [P, c_int64, P, c_int64, P, P, c_int, P, c_int, P, P, P, c_int, c_float, c_int, c_int, c_int,
-                                      c_int, c_int, c_int, c_int, c_int, c_int, P, c_int, c_int, c_float, P, c_int, P, P],
+                                      c_int, c_int, c_int, c_int, c_int, c_int, P, c_int, c_int, c_float, P, c_int, P, c_int, P],
     "liyab_attention_prefill_scored": [P, c_int64, P, c_int64, P, P, P, c_int, P, c_int, c_int, c_int, c_float, c_int, c_int,
-                                       c_int, c_int, c_int, c_int, c_float, P, c_int, P, P],
+                                       c_int, c_int, c_int, c_int, c_float, P, c_int, P, c_int, P],
     "liyab_gate_rows": [P, c_int, c_int64, P, c_int64, c_int, c_int, c_float, P],
     "liyab_dyt": [P, c_int, P, P, P, P, P, c_int, c_int, P],
     "liyab_glu_clamped": [P, c_int, P, c_int64, c_int, c_int, c_float, c_float, c_float, P],
+    "liyab_glu": [P, c_int, P, c_int64, c_int, c_int, c_int, P],
     "liyab_activate": [P, c_int, c_int64, P, c_int64, c_int, c_int, c_int, P],
     "liyab_mean_norm_add": [P, P, P, P, P, c_float, c_float, c_int, c_int, P],
     "liyab_wkv_scan": [P, c_int, P, P, P, P, P, c_int64, P, P, P, c_float, P, c_int64, c_int, P, c_int, c_int64, c_int, c_int64, P, P, P,
                        c_int, c_int, c_int, c_int, c_int, P, P, P],
     "liyab_ssd_scan": [P, c_int64, P, c_int64, P, c_int64, P, P, P, P, c_int64, c_int, P, c_int64, c_int, c_int, c_int64, P, P, P, c_int,
                        c_int, c_int, c_int, c_int, c_int, c_int, P, P, P],
+    "liyab_gla_decay": [P, P, c_int64, P, P, c_float, c_int, c_int, c_int, P],
+    "liyab_gla_scan": [P, c_int, P, P, P, P, c_int64, P, c_int64, P, c_float, c_float, P, c_int64, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int,
+                       c_int, P, P, P],
+    "liyab_gla_single": [P, c_int, P, P, P, P, c_int64, P, c_int64, P, P, c_float, P, c_float, c_float, P, c_int64, c_int, P, P, P, c_int, c_int, c_int,
+                         c_int, c_int, P],
     "liyab_token_shift": [P, c_int, P, P, c_int, P, c_int64, c_int, P, P, P, P, c_int, c_int, P],
     "liyab_conv_act": [P, c_int64, P, c_int64, P, P, c_int, P, c_int64, c_int, P, P, P, P, c_int, c_int, c_int, P],
     "liyab_gated_group_norm": [P, c_int, P, c_int64, P, c_int64, P, c_float, c_int, c_int, c_int, P],
     "liyab_qk_prepare": [P, c_int64, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, P, P, P, c_int, P, c_int, c_int, P, P, c_float, P,
                          c_int, c_float, c_int, P, c_int, c_int, c_float, P, P, P, P],
+    "liyab_qk_prepare_rows": [P, c_int64, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, P, P, P, c_int, P, c_int, c_int, P, P, c_float, P,
+                              c_int, P, c_int, c_int, P],
     "liyab_attention_scored": [P, c_int64, P, c_int64, P, P, c_int, P, c_int, P, P, c_int, c_float, c_float, c_int, P, c_int, P, c_int64,
-                               c_int, c_int, c_int, c_int, c_int, c_int, P, P],
+                               c_int, c_int, c_int, c_int, c_int, c_int, P, c_int, P],
     "liyab_norm_shift": [P, c_int, P, P, P, c_float, c_float, P, c_int, P, c_int64, c_int, P, P, P, P, c_int, c_int, c_int, c_int, P],
     "liyab_ring_keep": [P, c_int64, c_int, c_int, P, c_int64, c_int, P, P, P, P, P, c_int, P],
     "liyab_normed_powers": [P, c_int, P, c_int64, c_int, c_int, P, c_float, P],
@@ -111,7 +119,12 @@ _SIGNATURES = {
     "liyab_delta_single": [P, c_int, P, P, P, P, P, c_int64, P, c_int64, P, P, P, c_float, c_float, c_float, P, c_int64, c_int, P, P, P, c_int, c_int,
                            c_int, P],
     "liyab_delta_scan": [P, P, P, P, c_int64, P, P, c_int64, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, P, P, P, P],
-    "liyab_head_norm_gate": [P, c_int, P, P, c_int64, P, c_float, c_int, c_int, c_int, P],
+    "liyab_head_norm_gate": [P, c_int, P, P, c_int64, P, c_int, c_float, c_int, c_int, c_int, c_int, P],
+    "liyab_gated_delta_prepare": [P, P, c_int64, P, c_int, P, c_int64, c_int, P, P, c_int, c_int, c_float, c_float, P, P, P, P, c_int, c_int, c_int,
+                                  c_int, c_int, P],
+    "liyab_gated_delta_scan": [P, P, P, c_int64, c_int, P, c_int64, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, P, P, P, P],
+    "liyab_gated_delta_single": [P, c_int, P, c_int64, P, c_int, P, P, c_int, c_int, c_int, P, c_float, c_float, c_float, P, c_int64, c_int, P, P, P,
+                                 c_int, c_int, c_int, c_int, c_int, P],
     "liyab_maps_store": [P, c_int64, P, c_int, P, c_int64, c_int, P, P, P, P, c_int, P, c_int, c_int, P, P, P, P, c_int, c_int, c_int,
                          c_int, c_int, c_int, c_int, P],
     "liyab_maps_join": [P, P, P, c_int64, c_int, c_float, c_float, c_float, c_int, c_int, c_int, c_int, P],

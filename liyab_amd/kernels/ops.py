@@ -783,7 +783,7 @@ def attention_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, 
                      tok_list: Optional[torch.Tensor] = None, n_tokens: Optional[int] = None, waves: int = 4,
                      rows_are_requests: bool = False, leave_splits: bool = False, chunk: int = 0,
                      num_pages: Optional[int] = None, softcap: float = 0.0, bias_table: Optional[torch.Tensor] = None,
-                     sinks: Optional[torch.Tensor] = None) -> None:
+                     sinks: Optional[torch.Tensor] = None, keep_first: int = 0) -> None:
     """Each token on its own over its request's cache (bfloat16, or float32 throughout), its keys cut into `n_splits`.
     With `tok_list` (int32) only those rows are computed. `rows_are_requests`: row t belongs to
     request t (every request brings one token), which saves the kernel a lookup. With
@@ -793,7 +793,7 @@ def attention_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, 
     token's keys instead of an equal share (`n_splits * chunk` must cover the longest context): a token's
     sums then follow from its position alone. `softcap` > 0: scores become cap * tanh(score / cap); `bias_table` (float32
     [distances, heads]): + table[min(position - key, distances - 1), head]; `sinks` (float32 [heads]): exp(sinks[head]) joins
-    the softmax's denominator (a learned logit with no key and no value)."""
+    the softmax's denominator (a learned logit with no key and no value); `keep_first`: with a window, positions below it stay visible."""
     if k_cache.dim() != 4 or k_cache.shape != v_cache.shape or not k_cache.is_contiguous() or not v_cache.is_contiguous():
         raise KernelError("attention: caches must be contiguous [pages, kv_heads, page_size, head_dim] of one shape")
     _, hkv, page, hd = k_cache.shape
@@ -824,10 +824,11 @@ def attention_decode(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, 
             n, float(scale), int(window), n_head, hkv, hd, page, n_splits, int(chunk), waves, 1 if rows_are_requests else 0,
             _ptr(partials), 1 if leave_splits else 0, _pages(k_cache, num_pages))
     _f32vec(sinks, "sinks", n_head)
-    if softcap > 0 or bias_table is not None or sinks is not None:
+    if softcap > 0 or bias_table is not None or sinks is not None or (keep_first > 0 and window > 0):
         if sinks is not None and leave_splits:
             raise KernelError("attention_decode: splits left unmerged take no sink")
-        _lib.call("liyab_attention_decode_scored", *args, float(softcap), _ptr(bias_table), _bias_rows(bias_table, n_head) - 1, _ptr(sinks), _stream())
+        _lib.call("liyab_attention_decode_scored", *args, float(softcap), _ptr(bias_table), _bias_rows(bias_table, n_head) - 1, _ptr(sinks), int(keep_first),
+                  _stream())
     else:
         _lib.call("liyab_attention_decode", *args, _stream())
 
@@ -858,7 +859,7 @@ def attention_merge(out: torch.Tensor, partials: torch.Tensor) -> None:
 def attention_prefill(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                       block_tables: torch.Tensor, work: torch.Tensor, n_tiles: int, *, n_head: int, scale: float,
                       window: int = 0, tile: int = 128, ksplit: int = 1, num_pages: Optional[int] = None, softcap: float = 0.0,
-                      bias_table: Optional[torch.Tensor] = None, sinks: Optional[torch.Tensor] = None) -> None:
+                      bias_table: Optional[torch.Tensor] = None, sinks: Optional[torch.Tensor] = None, keep_first: int = 0) -> None:
     """Tiles of up to `tile` (64 or 128) consecutive queries of one request over its bfloat16
     cache, on the matrix cores; `ksplit` waves (1, 2, or 4 with tiles of 64) share the keys of
     32 queries. work: int32 [n_tiles, 4] = (request index, first row, first
@@ -881,8 +882,9 @@ def attention_prefill(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
             block_tables.data_ptr(), block_tables.shape[1], work.data_ptr(), n_tiles, int(tile), int(ksplit), float(scale), int(window),
             n_head, hkv, hd, page, _pages(k_cache, num_pages))
     _f32vec(sinks, "sinks", n_head)
-    if softcap > 0 or bias_table is not None or sinks is not None:  # (see attention_decode)
-        _lib.call("liyab_attention_prefill_scored", *args, float(softcap), _ptr(bias_table), _bias_rows(bias_table, n_head) - 1, _ptr(sinks), _stream())
+    if softcap > 0 or bias_table is not None or sinks is not None or (keep_first > 0 and window > 0):  # (see attention_decode)
+        _lib.call("liyab_attention_prefill_scored", *args, float(softcap), _ptr(bias_table), _bias_rows(bias_table, n_head) - 1, _ptr(sinks), int(keep_first),
+                  _stream())
     else:
         _lib.call("liyab_attention_prefill", *args, _stream())
 
@@ -969,17 +971,20 @@ def attention_takes(head_dim: int) -> bool:
 def attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
               block_tables: torch.Tensor, ctx, *, n_head: int, scale: float, window: int = 0,
               splits_ok: bool = False, softcap: float = 0.0, bias_table: Optional[torch.Tensor] = None,
-              sinks: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+              sinks: Optional[torch.Tensor] = None, keep_first: int = 0) -> Optional[torch.Tensor]:
     """Attention of the step's tokens over their requests' cached keys and values; the kernel
     is chosen from the step's shape (`ctx` is the step's StepContext; `ctx.plans["attention"]`
     says how the step's tokens are cut, see parts/attention.py; without it every token goes to
     the plain kernel). With `splits_ok`, a step of few tokens may leave `out` unwritten and
     return the splits of each (token, head) pair instead, float32 [tokens, heads, splits, head
     size + 4], for `gemm_att_parts`. `softcap`, `bias_table`: what is done to the scores before the softmax, `sinks`: a learned
-    logit a head in its denominator (see `attention_decode`); every kernel below does the same."""
+    logit a head in its denominator, `keep_first`: positions that stay visible behind the window (see `attention_decode`); every kernel
+    below does the same."""
     hd = k_cache.shape[3]
     host = ctx.host
-    scored = dict(softcap=softcap, bias_table=bias_table, sinks=sinks) if softcap > 0 or bias_table is not None or sinks is not None else {}
+    keep_first = keep_first if window > 0 else 0
+    scored = (dict(softcap=softcap, bias_table=bias_table, sinks=sinks, keep_first=keep_first)
+              if softcap > 0 or bias_table is not None or sinks is not None or keep_first else {})
     if sinks is not None and splits_ok:
         raise KernelError("attention: splits left to the caller take no sink")
     plan = ctx.plans.get("attention")
@@ -987,7 +992,7 @@ def attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache
             and out.stride(0) % 8 == 0)
 
     def decode(tok_list, n):
-        splits, waves = decode_plan(n, n_head, min(plan.context_bucket, window) if window > 0 else plan.context_bucket)
+        splits, waves = decode_plan(n, n_head, min(plan.context_bucket, window + keep_first) if window > 0 else plan.context_bucket)
         partials = None
         if splits > 1:
             partials = ctx.workspace.get("attn_partials", (n * n_head * splits * (hd + 4),), torch.float32)
@@ -1005,7 +1010,7 @@ def attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache
         # a split's keys follow from what a request can reach at most (the table's width, the window): a
         # constant of the engine, never of the step; at most 16 splits, so that one workgroup can walk them
         # all and the merge's arrays hold them (contexts past 4,096 keys take longer splits)
-        reach = block_tables.shape[1] * k_cache.shape[2] if window <= 0 else min(window, block_tables.shape[1] * k_cache.shape[2])
+        reach = block_tables.shape[1] * k_cache.shape[2] if window <= 0 else min(window + keep_first, block_tables.shape[1] * k_cache.shape[2])
         chunk = invariant_chunk(reach)
         splits = max(1, -(-min(plan.context_bucket, reach) // chunk))
         # many tokens: a workgroup walks its token's splits in turn (the same bits: the kernel merges them
@@ -1086,14 +1091,15 @@ def _keep_args(keep, d: int):
 
 def gated_norm_add(x: torch.Tensor, y: torch.Tensor, weight: Optional[torch.Tensor], eps: float, *, n_sum: int = 1,
                    gate: Optional[torch.Tensor] = None, cast_out: Optional[torch.Tensor] = None, keep=None,
-                   normalize: bool = True, next_norm=None) -> None:
+                   normalize: bool = True, next_norm=None, bias: Optional[torch.Tensor] = None, centred: bool = False) -> None:
     """x[t] += weight * s / sqrt(mean(s^2) + eps) with s = (y[t * n_sum] + ... + y[t * n_sum + n_sum - 1]) *
     sigmoid(gate[t]); x float32 [n, d] in place, y float32 [n * n_sum, d], gate float32 [n, d] (rows may
     be strided: columns of a wider product) or None. `cast_out` [n, d] (float32 or bfloat16) gets the new
     rows rounded. `keep` = (state, ctx): before the update, the last rows of each request go to its input
     history, state[slot, position % ring] (the rows behind the step's tokens are left out). Without
     `normalize`: x[t] += s. `next_norm` = (weight float32 [d], eps): `cast_out` gets the new row's root-mean-square norm under
-    that weight instead of the row itself (what the next sublayer reads)."""
+    that weight instead of the row itself (what the next sublayer reads). `centred`: a layer norm instead, x[t] += weight * (s - mean(s)) /
+    sqrt(var(s) + eps) + bias."""
     _dev(x, "x")
     _dev(y, "y")
     n, d = x.shape
@@ -1102,6 +1108,7 @@ def gated_norm_add(x: torch.Tensor, y: torch.Tensor, weight: Optional[torch.Tens
     if y.dtype != torch.float32 or not y.is_contiguous() or y.numel() != n * n_sum * d or n_sum < 1:
         raise KernelError(f"gated_norm_add: y must be contiguous float32 with {n_sum} rows of {d} a token, got {tuple(y.shape)} {y.dtype}")
     _f32vec(weight, "norm weight", d)
+    _f32vec(bias, "norm bias", d)
     gs = 0
     if gate is not None:
         gs = _rows(gate, "gate")
@@ -1120,7 +1127,7 @@ def gated_norm_add(x: torch.Tensor, y: torch.Tensor, weight: Optional[torch.Tens
     if next_w is not None and cast_out is None:
         raise KernelError("gated_norm_add: the next norm's rows need a place (cast_out)")
     _lib.call("liyab_gated_norm_add", x.data_ptr(), _ptr(cast_out), code, y.data_ptr(), n_sum, _ptr(gate), gs, _ptr(weight), float(eps),
-              1 if normalize else 0, n, d, *_keep_args(keep, d), _ptr(next_w), float(next_eps), _stream())
+              (2 if centred else 1) if normalize else 0, n, d, *_keep_args(keep, d), _ptr(next_w), float(next_eps), _ptr(bias), _stream())
 
 
 def keep_rows(x: torch.Tensor, state: torch.Tensor, ctx) -> None:
@@ -1241,16 +1248,21 @@ def moe_block(n_entries: int, n_experts: int, dtype: torch.dtype, *inner_sizes: 
 
 
 MOE_MAX_GROUPS = 64
+MOE_MAX_WAVE_EXPERTS = 2048  # with logistic scores (csrc/moe.hip: kMaxWaveExperts)
+MOE_WAVE_TOKENS = 64  # tokens such a choice and its lists take in one launch (kWaveRouteTokens)
 
 
 def moe_route(logits: torch.Tensor, top: int, ids: torch.Tensor, weights: torch.Tensor, rows_list: torch.Tensor,
-              tile_group: torch.Tensor, block: int = GROUPED_ROWS, groups: Optional[tuple] = None) -> None:
+              tile_group: torch.Tensor, block: int = GROUPED_ROWS, groups: Optional[tuple] = None, logistic: bool = False,
+              correction: Optional[torch.Tensor] = None) -> None:
     """From float32 router logits [n, experts] (rows may be strided): ids int32 and weights float32 [n,
     top] (the experts with the largest logits, softmax over those alone), and the entries t * top + k
     listed by expert in tiles of `block` places: rows_list int32 [tiles * block] (-1: empty), tile_group
     int32 [tiles] (-1: unused), tiles = moe_tiles(n * top, experts, block). `groups` = (count, keep): the choice among groups
     of experts instead: softmax over all experts, the experts in `count` equal groups of neighbours, only those of the `keep`
-    groups with the largest member can be chosen, the weights the chosen scores divided by their sum."""
+    groups with the largest member can be chosen, the weights the chosen scores divided by their sum. `logistic`: scores s = sigmoid(logit),
+    the choice by s + correction (float32 [experts], or None); a group's score is then the sum of its two largest, and the weights are the
+    chosen s as they are."""
     ld = _rows(logits, "logits")
     n, E = logits.shape
     if logits.dtype != torch.float32:
@@ -1271,11 +1283,18 @@ def moe_route(logits: torch.Tensor, top: int, ids: torch.Tensor, weights: torch.
         mode, count, keep = 1, int(groups[0]), int(groups[1])
         if not (1 <= count <= MOE_MAX_GROUPS and E % count == 0 and 1 <= keep <= count and top <= keep * (E // count)):
             raise KernelError(f"moe_route: {keep} of {count} groups of {E} experts do not hold {top} choices (at most {MOE_MAX_GROUPS} groups)")
-    if n <= 1024:  # one launch: a thread routes a token, then the workgroup lists the entries
+    if logistic:
+        mode = 2
+        if E > MOE_MAX_WAVE_EXPERTS:
+            raise KernelError(f"moe_route: {E} experts with logistic scores (at most {MOE_MAX_WAVE_EXPERTS})")
+        _f32vec(correction, "the choice's correction", E)
+    elif correction is not None:
+        raise KernelError("moe_route: a correction goes with logistic scores")
+    if n <= (1024 if mode != 2 else MOE_WAVE_TOKENS if E <= 512 else 0):  # one launch: the tokens are routed, then the workgroup lists the entries
         _lib.call("liyab_moe_route_align", logits.data_ptr(), ld, n, E, top, ids.data_ptr(), weights.data_ptr(), block,
-                  rows_list.data_ptr(), tile_group.data_ptr(), tiles, mode, count, keep, _stream())
+                  rows_list.data_ptr(), tile_group.data_ptr(), tiles, mode, count, keep, _ptr(correction), _stream())
         return
-    _lib.call("liyab_moe_route", logits.data_ptr(), ld, n, E, top, ids.data_ptr(), weights.data_ptr(), mode, count, keep, _stream())
+    _lib.call("liyab_moe_route", logits.data_ptr(), ld, n, E, top, ids.data_ptr(), weights.data_ptr(), mode, count, keep, _ptr(correction), _stream())
     _lib.call("liyab_moe_align", ids.data_ptr(), n * top, E, block, rows_list.data_ptr(), tile_group.data_ptr(), tiles, _stream())
 
 
@@ -1344,6 +1363,19 @@ def glu_clamped(out: torch.Tensor, gu: torch.Tensor, limit: float, slope: float,
     if gu.dtype != torch.float32 or tuple(gu.shape) != (n, 2 * ff) or not out.is_contiguous():
         raise KernelError(f"glu_clamped: needs float32 [n, {2 * ff}] and a contiguous out [n, {ff}], got {tuple(gu.shape)} {gu.dtype}")
     _lib.call("liyab_glu_clamped", out.data_ptr(), dtype_code(out.dtype), gu.data_ptr(), ld, n, ff, float(limit), float(slope), float(shift), _stream())
+
+
+GLU_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
+
+
+def glu(out: torch.Tensor, gu: torch.Tensor, activation: str) -> None:
+    """out = act(G) * U; gu float32 [n, 2 * ff] = [G | U], out contiguous [n, ff] float32 or bfloat16; act "silu" or "gelu_tanh"."""
+    _dev(out, "out")
+    ld = _rows(gu, "gu")
+    n, ff = out.shape
+    if gu.dtype != torch.float32 or tuple(gu.shape) != (n, 2 * ff) or not out.is_contiguous():
+        raise KernelError(f"glu: needs float32 [n, {2 * ff}] and a contiguous out [n, {ff}], got {tuple(gu.shape)} {gu.dtype}")
+    _lib.call("liyab_glu", out.data_ptr(), dtype_code(out.dtype), gu.data_ptr(), ld, n, ff, GLU_ACTIVATIONS[activation], _stream())
 
 
 ACTIVATE = {"tanh": 0, "silu": 1, "sigmoid": 2, "relu2": 3}
@@ -1593,13 +1625,59 @@ def qk_prepare(src: torch.Tensor, q_out: torch.Tensor, k_cache: torch.Tensor, v_
               1 if rot_halves else 0, float(rot_mag), _ptr(v_keep), _ptr(v_first), _ptr(v_lam), _stream())
 
 
+def qk_prepare_rows(src: torch.Tensor, q_out: torch.Tensor, k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor], slots: torch.Tensor,
+                    positions: torch.Tensor, *, q_off: int, k_off: int, v_off: int, n_head: int, n_kv_head: int, head_dim: int, value_dim: int,
+                    q_norm: torch.Tensor, k_norm: Optional[torch.Tensor], eps: float, freqs: Optional[torch.Tensor] = None, rot_dims: int = 0,
+                    rot_halves: bool = False, num_pages: Optional[int] = None) -> None:
+    """`qk_prepare` with the norms taken over all of a token's queries (and all of its keys) at once, a weight an entry: q_norm float32
+    [n_head * head_dim], k_norm [n_kv_head * head_dim]. Without caches (None) only the queries are made: the layer's keys and values are
+    another layer's. q_out [n, n_head * row], row the caches' row width (at least head_dim; zeros behind the heads)."""
+    ld = _rows(src, "src")
+    n = src.shape[0]
+    H, G = n_head, n_kv_head
+    _dev(q_out, "q_out")
+    if src.dtype != torch.float32 or q_out.dim() != 2 or q_out.shape[0] != n or q_out.shape[1] % H or not q_out.is_contiguous() or head_dim > 512:
+        raise KernelError("qk_prepare_rows: src must be float32 rows and q_out contiguous [n, heads * row], heads of up to 512")
+    dk_out = q_out.shape[1] // H
+    dv_out, page, pages = max(value_dim, 1), 1, 1
+    if q_off < 0 or q_off + H * head_dim > src.shape[1] or dk_out < head_dim:
+        raise KernelError("qk_prepare_rows: the queries' columns pass the source's rows, or the heads their rows")
+    _f32vec(q_norm, "query norm weight", H * head_dim)
+    if k_cache is not None:
+        _dev(k_cache, "k_cache")
+        _dev(v_cache, "v_cache")
+        if k_cache.dim() != 4 or v_cache.dim() != 4 or k_cache.shape[:3] != v_cache.shape[:3] or k_cache.shape[1] != G or not k_cache.is_contiguous() or not v_cache.is_contiguous():
+            raise KernelError(f"qk_prepare_rows: caches must be contiguous [pages, {G}, page_size, width] with the same pages")
+        page, dv_out, pages = k_cache.shape[2], v_cache.shape[3], _pages(k_cache, num_pages)
+        if not (q_out.dtype == k_cache.dtype == v_cache.dtype) or k_cache.shape[3] != dk_out or dv_out < value_dim:
+            raise KernelError("qk_prepare_rows: queries and caches share a dtype and the keys' row width, which hold the heads")
+        if min(k_off, v_off) < 0 or k_off + G * head_dim > src.shape[1] or v_off + G * value_dim > src.shape[1]:
+            raise KernelError("qk_prepare_rows: the keys' or values' columns pass the source's rows")
+        if k_norm is None:
+            raise KernelError("qk_prepare_rows: the keys have a norm too")
+        _f32vec(k_norm, "key norm weight", G * head_dim)
+        _i32(slots, "slots", n)
+    if rot_dims:
+        if rot_dims % 2 or rot_dims > head_dim or freqs is None:
+            raise KernelError(f"qk_prepare_rows: {rot_dims} turned entries of heads of {head_dim}")
+        _dev(freqs, "freqs")
+        if freqs.dtype != torch.float64 or not freqs.is_contiguous() or freqs.numel() != rot_dims // 2:
+            raise KernelError(f"qk_prepare_rows: the frequencies must be {rot_dims // 2} contiguous float64 values")
+    _i32(positions, "positions", n)
+    _lib.call("liyab_qk_prepare_rows", src.data_ptr(), ld, q_off, k_off, v_off, H, G, head_dim, value_dim, dk_out, dv_out, q_out.data_ptr(), _ptr(k_cache),
+              _ptr(v_cache), dtype_code(q_out.dtype), slots.data_ptr() if k_cache is not None else None, page, pages, q_norm.data_ptr(),
+              _ptr(k_norm) if k_cache is not None else None, float(eps), _ptr(freqs) if rot_dims else None, rot_dims, positions.data_ptr(), n,
+              1 if rot_halves else 0, _stream())
+
+
 def attention_scored(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor, ctx, *,
                      n_head: int, scale: float, softcap: float = 0.0, window: int = 0, bias_table: Optional[torch.Tensor] = None,
-                     gate: Optional[torch.Tensor] = None, num_pages: Optional[int] = None, sinks: Optional[torch.Tensor] = None) -> None:
+                     gate: Optional[torch.Tensor] = None, num_pages: Optional[int] = None, sinks: Optional[torch.Tensor] = None,
+                     keep_first: int = 0) -> None:
     """Causal attention of the step's rows over their requests' pages with score = scale * q . k, then cap * tanh(score / cap)
     (softcap > 0), then + bias_table[min(distance, rows - 1), head] (float32 [rows, heads]); softmax in 32-bit; values `dv` wide.
     out [n, heads * dv] = result * sigmoid(gate) (gate: float32 rows [n, heads * dv], or None). `sinks` (float32 [heads]):
-    exp(sinks[head]) joins the softmax's denominator."""
+    exp(sinks[head]) joins the softmax's denominator. `keep_first`: with a window, positions below it stay visible."""
     _dev(out, "out")
     _dev(q, "q")
     n = out.shape[0]
@@ -1631,7 +1709,8 @@ def attention_scored(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, 
     _f32vec(sinks, "sinks", n_head)
     _lib.call("liyab_attention_scored", out.data_ptr(), so, q.data_ptr(), sq, k_cache.data_ptr(), v_cache.data_ptr(), dtype_code(q.dtype),
               block_tables.data_ptr(), block_tables.shape[1], ctx.tok_seq.data_ptr(), ctx.positions.data_ptr(), n, float(scale), float(softcap),
-              int(window), _ptr(bias_table), max_dist, _ptr(gate), gs, n_head, G, dk, dv, page, _pages(k_cache, num_pages), _ptr(sinks), _stream())
+              int(window), _ptr(bias_table), max_dist, _ptr(gate), gs, n_head, G, dk, dv, page, _pages(k_cache, num_pages), _ptr(sinks), int(keep_first),
+              _stream())
 
 
 def gate_rows(x: torch.Tensor, gate: torch.Tensor, scale: float = 1.0) -> None:
@@ -1814,7 +1893,121 @@ def delta_rule(out: torch.Tensor, proj: torch.Tensor, wraw: torch.Tensor, w0: to
     _lib.call("liyab_delta_scan", o.data_ptr(), p, p + 4 * HD, p + 8 * HD, ld, prep.data_ptr(), state.data_ptr(), state.stride, state.n_slots,
               ctx.seq_starts.data_ptr(), ctx.positions.data_ptr(), ctx.state_slots.data_ptr(), ctx.n_seqs, H, D, *_delta_segments(ctx, n, H, D),
               _stream())
-    _lib.call("liyab_head_norm_gate", out.data_ptr(), dtype_code(out.dtype), o.data_ptr(), p + 16 * HD, ld, _ptr(norm_w), float(eps), n, H, D, _stream())
+    _lib.call("liyab_head_norm_gate", out.data_ptr(), dtype_code(out.dtype), o.data_ptr(), p + 16 * HD, ld, _ptr(norm_w), 0, float(eps), n, H, D, 0,
+              _stream())
+
+
+# -- a gated delta rule behind a short convolution ---------------------------------------------------------------
+def gated_delta_takes(head_dim: int, value_dim: int) -> bool:
+    """Whether the gated delta-rule kernels take heads of these sizes (csrc/gated_delta.hip)."""
+    return 1 <= head_dim <= 256 and 1 <= value_dim <= 256
+
+
+GATED_DELTA_MAX_TAPS = 16
+
+
+def gated_delta_floats(n_head: int, n_kv_head: int, head_dim: int, value_dim: int, taps: int) -> int:
+    """Floats a request's slot holds: the heads' matrices, then `taps` places of the channels before the convolution (none with one tap)."""
+    return n_head * head_dim * value_dim + (taps * (2 * n_kv_head * head_dim + n_head * value_dim) if taps > 1 else 0)
+
+
+def gated_delta(out: torch.Tensor, src: torch.Tensor, conv: torch.Tensor, a_log: torch.Tensor, dt_bias: torch.Tensor, norm_w: torch.Tensor, eps: float,
+                state: StateSlice, ctx, *, n_head: int, n_kv_head: int, head_dim: int, value_dim: int, key_eps: float, q_scale: float) -> None:
+    """The gated delta rule over each request's rows of the step. src float32 [n, >= C + H * V + 2 H] = [q | k | v | gate logits | rate
+    logits b, H | decay inputs a, H], C = 2 G D + H V; q, k, v = silu(conv(.)) a channel over time (conv float32 [taps, C], a tap's
+    channels side by side), q and k to length one a head (key_eps under the root), q times q_scale; beta = sigmoid(b), g = exp(-exp(a_log) *
+    softplus(a + dt_bias)); S <- g S, S <- S + k (beta (v - S^T k))^T, o = S^T q; out [n, H * V] (compute dtype) = o / rms(o over the head)
+    * norm_w [V] * silu(gate). `state`: `gated_delta_floats` of a slot."""
+    H, G, D, V = n_head, n_kv_head, head_dim, value_dim
+    C = 2 * G * D + H * V
+    _dev(out, "out")
+    n = out.shape[0]
+    ld = _rows(src, "src")
+    if src.dtype != torch.float32 or src.shape[0] != n or src.shape[1] < C + H * V + 2 * H or tuple(out.shape) != (n, H * V) or not out.is_contiguous() or ctx.n_tokens != n:
+        raise KernelError(f"gated_delta: needs the step's float32 rows of {C + H * V + 2 * H} columns and a contiguous out [n, {H * V}]")
+    if H % G or not gated_delta_takes(D, V):
+        raise KernelError(f"gated_delta: {H} heads over {G}, keys of {D}, values of {V} are not taken")
+    _dev(conv, "conv")
+    if conv.dtype != torch.float32 or conv.dim() != 2 or conv.shape[1] != C or not conv.is_contiguous() or not 1 <= conv.shape[0] <= GATED_DELTA_MAX_TAPS:
+        raise KernelError(f"gated_delta: the convolution's weights must be contiguous float32 [taps, {C}], 1 to {GATED_DELTA_MAX_TAPS} taps")
+    taps = conv.shape[0]
+    _f32vec(a_log, "A_log", H)
+    _f32vec(dt_bias, "dt_bias", H)
+    _f32vec(norm_w, "norm weight", V)
+    if state.size != gated_delta_floats(H, G, D, V, taps):
+        raise KernelError(f"gated_delta: a slot of {state.size} floats, {gated_delta_floats(H, G, D, V, taps)} are needed")
+    _step_lists(ctx, n)
+    g_off, b_off = C, C + H * V
+    a_off = b_off + H
+    if single_token_step(ctx):
+        _lib.call("liyab_gated_delta_single", out.data_ptr(), dtype_code(out.dtype), src.data_ptr(), ld, conv.data_ptr(), taps, a_log.data_ptr(),
+                  dt_bias.data_ptr(), g_off, b_off, a_off, norm_w.data_ptr(), float(eps), float(key_eps), float(q_scale), state.data_ptr(), state.stride,
+                  state.n_slots, ctx.seq_starts.data_ptr(), ctx.positions.data_ptr(), ctx.state_slots.data_ptr(), ctx.n_seqs, H, G, D, V, _stream())
+        return
+    ws = ctx.workspace
+    prep = ws.get("gated_delta_prep", (n, C + 2 * H), torch.float32)
+    o = ws.get("gated_delta_o", (n, H * V), torch.float32)
+    _lib.call("liyab_gated_delta_prepare", prep.data_ptr(), src.data_ptr(), ld, conv.data_ptr(), taps, state.data_ptr() + 4 * H * D * V, state.stride,
+              state.n_slots, a_log.data_ptr(), dt_bias.data_ptr(), b_off, a_off, float(key_eps), float(q_scale), ctx.tok_seq.data_ptr(),
+              ctx.positions.data_ptr(), ctx.seq_starts.data_ptr(), ctx.state_slots.data_ptr(), n, H, G, D, V, _stream())
+    seg = (0, 0, None, None, None)
+    if delta_segments_from(n, ctx.n_seqs):
+        most = -(-n // SCAN_SEGMENT) + ctx.n_seqs
+        ends = ws.get("gated_delta_ends", (most, H, D, V), torch.float32)
+        trans = ws.get("gated_delta_trans", (most, H, D, D), torch.float32)
+        starts = ws.get("gated_delta_starts", (most, H, D, V), torch.float32)
+        seg = (SCAN_SEGMENT, most, ends.data_ptr(), trans.data_ptr(), starts.data_ptr())
+    _lib.call("liyab_gated_delta_scan", o.data_ptr(), prep.data_ptr(), src.data_ptr(), ld, taps, state.data_ptr(), state.stride, state.n_slots,
+              ctx.seq_starts.data_ptr(), ctx.positions.data_ptr(), ctx.state_slots.data_ptr(), ctx.n_seqs, H, G, D, V, *seg, _stream())
+    _lib.call("liyab_head_norm_gate", out.data_ptr(), dtype_code(out.dtype), o.data_ptr(), src.data_ptr() + 4 * g_off, ld, norm_w.data_ptr(), 1, float(eps),
+              n, H, V, 1, _stream())
+
+
+# -- gated linear attention --------------------------------------------------------------------------------------
+GLA_SINGLE_MAX = 256  # the widest heads the one-kernel form for steps of single tokens takes (csrc/recurrent.hip: kGlaMax)
+
+
+def gla(out: torch.Tensor, proj: torch.Tensor, w2t: torch.Tensor, bias: torch.Tensor, norm_w: torch.Tensor, tau: float, eps: float, state: StateSlice, ctx,
+        *, n_head: int, head_dim: int, value_dim: int, q_scale: float) -> None:
+    """Gated linear attention over each request's rows of the step. proj float32 [n, >= 2 H D + 2 H V + rank] = [q | k | v | gate logits |
+    the decay's narrow product], w2t float32 [rank, H * D]; w = sigmoid(low . w2 + bias)^(1 / tau) a key channel; S <- diag(w) S + k v^T,
+    o = S^T q * q_scale a head; out [n, H * V] (compute dtype) = o / rms(o over the head) * norm_w [V] * silu(gate). `state`: the heads'
+    matrices [H, D, V] of a slot."""
+    H, D, V = n_head, head_dim, value_dim
+    _dev(out, "out")
+    n = out.shape[0]
+    ld = _rows(proj, "proj")
+    _dev(w2t, "w2t")
+    if w2t.dtype != torch.float32 or w2t.dim() != 2 or w2t.shape[1] != H * D or not w2t.is_contiguous():
+        raise KernelError(f"gla: the decay's second matrix must be contiguous float32 [rank, {H * D}]")
+    rank = w2t.shape[0]
+    low_off = 2 * H * D + 2 * H * V
+    if proj.dtype != torch.float32 or proj.shape[0] != n or proj.shape[1] < low_off + rank or tuple(out.shape) != (n, H * V) or not out.is_contiguous() or ctx.n_tokens != n:
+        raise KernelError(f"gla: needs the step's float32 rows of {low_off + rank} columns and a contiguous out [n, {H * V}]")
+    _f32vec(bias, "the decay's bias", H * D)
+    _f32vec(norm_w, "norm weight", V)
+    if not scan_takes(D, V) or state.size != H * D * V or not tau > 0:
+        raise KernelError(f"gla: a state of {D} x {V} a head ({state.size} floats a slot), tau {tau}")
+    _step_lists(ctx, n)
+    p = proj.data_ptr()
+    q, k, v, g, low = p, p + 4 * H * D, p + 8 * H * D, p + 4 * (2 * H * D + H * V), p + 4 * low_off
+    lists = (ctx.seq_starts.data_ptr(), ctx.positions.data_ptr(), ctx.state_slots.data_ptr(), ctx.n_seqs)
+    slots = (state.data_ptr(), state.stride, state.n_slots)
+    if single_token_step(ctx) and D <= GLA_SINGLE_MAX and V <= GLA_SINGLE_MAX:
+        _lib.call("liyab_gla_single", out.data_ptr(), dtype_code(out.dtype), q, k, v, g, ld, low, ld, w2t.data_ptr(), bias.data_ptr(), float(tau),
+                  norm_w.data_ptr(), float(eps), float(q_scale), *slots, *lists, H, D, V, rank, _stream())
+        return
+    ws = ctx.workspace
+    decay = ws.get("gla_decay", (n, H * D), torch.float32)
+    _lib.call("liyab_gla_decay", decay.data_ptr(), low, ld, w2t.data_ptr(), bias.data_ptr(), float(tau), n, H * D, rank, _stream())
+    seg = (0, 0, None, None)
+    if delta_segments_from(n, ctx.n_seqs):
+        most = -(-n // SCAN_SEGMENT) + ctx.n_seqs
+        ends = ws.get("scan_seg_state", (most, H, D, V), torch.float32)
+        prod = ws.get("scan_seg_decay", (most, H, D), torch.float32)
+        seg = (SCAN_SEGMENT, most, ends.data_ptr(), prod.data_ptr())
+    _lib.call("liyab_gla_scan", out.data_ptr(), dtype_code(out.dtype), q, k, v, g, ld, decay.data_ptr(), H * D, norm_w.data_ptr(), float(eps), float(q_scale),
+              *slots, *lists, H, D, V, *seg, _stream())
 
 
 # -- attention in two maps a head --------------------------------------------------------------------------------

@@ -142,8 +142,8 @@ class DecoderModel:
         self.head = build_part("head", plan.head, store, dtype)
         self.order = list(plan.order)
         # a block may take the first norm of the block that follows it into its own last update of the rows (`chain_norm`): offered
-        # where the order runs every layer once, on its own cache, with nothing done to the stream between the two
-        if [e.layer for e in self.order] == list(range(len(self.blocks))) and all(e.cache_of is None and e.writes_cache for e in self.order):
+        # where the order runs every layer once, with nothing done to the stream between the two
+        if [e.layer for e in self.order] == list(range(len(self.blocks))):
             for i in range(len(self.blocks) - 1):
                 if hasattr(self.blocks[i], "chain_norm") and (i + 1) not in self.entries:
                     self.blocks[i].chain_norm(self.blocks[i + 1])
@@ -185,6 +185,9 @@ class DecoderModel:
             spec = self.blocks[layer].mixer.cache_spec()
             if spec is None:
                 continue
+            for e in self.order:  # other layers that read this one's rows, under windows of their own
+                if e.cache_layer == layer and e.layer != layer:
+                    spec = spec.covering(self.blocks[e.layer].mixer.cache_spec())
             groups.setdefault(spec.key, (spec, []))[1].append(layer)
         return list(groups.values())
 

@@ -124,7 +124,7 @@ class PostNormGatedBlock:
     gets it (before the convolution); `conv`: what the mixer reads is x + a short causal convolution of
     x over time, whose last inputs are the layer's per-request state. Gates and the convolution are
     optional, the feed-forward too. The sum into the stream, the norms and the gates are 32-bit; the
-    sublayers and the gates' products read x rounded to the compute dtype.
+    sublayers and the gates' products read x rounded to the compute dtype. The norms are root-mean-square norms or layer norms.
 
     Kernels a sublayer beside its own: the convolution (which also rounds x), the gate's product, and
     one update of the rows (sum of the sublayer's rows a token, gate, norm, addition, the rounded rows
@@ -144,8 +144,9 @@ class PostNormGatedBlock:
             if part is not None and "out" not in part.forward.__code__.co_varnames:
                 raise ValueError(f"a post-norm block needs a {what} that can leave its result to the block (forward(..., out=))")
         for norm in (norm_mixer, norm_ffn if ffn is not None else norm_mixer):
-            if not getattr(norm, "root_mean_square", False):
-                raise ValueError("a post-norm block's row update applies a root-mean-square norm (kind 'rmsnorm')")
+            if not getattr(norm, "root_mean_square", False) and not getattr(norm, "centred", False):
+                raise ValueError("a post-norm block's row update applies a root-mean-square norm or a layer norm (kinds 'rmsnorm', 'layernorm')")
+        self.casts_last = self.input_cast = False  # see chain_norm
         if mixer.state_spec() is not None and self.conv is not None and self.conv.state_spec() is not None:
             raise ValueError("a mixer with state of its own under an input convolution: one state a layer")
         # The feed-forward's gate and its router read the same rows: one product [gate | router] instead of two
@@ -165,6 +166,19 @@ class PostNormGatedBlock:
             self.joint_weight, self.joint_bias = hit[0], hit[1]
             self.gate_ffn.weight = self.gate_ffn.bias = None
 
+    def chain_norm(self, following) -> bool:
+        """Called once, when the model is built, for a block that runs right before `following` in every pass: this block's last update
+        of the rows then also leaves them rounded to the compute dtype, which is what `following`'s mixer and gate read. True if the two
+        were chained (both blocks of this kind, `following` without a convolution, which rounds the rows itself)."""
+        if not isinstance(following, PostNormGatedBlock) or following.conv is not None or following.dtype != self.dtype:
+            return False
+        self.casts_last = following.input_cast = True
+        return True
+
+    @staticmethod
+    def _norm_of(norm) -> dict:
+        return {"centred": True, "bias": norm.bias} if getattr(norm, "centred", False) else {}
+
     def state_spec(self):
         return (self.conv.state_spec() if self.conv is not None else None) or self.mixer.state_spec()
 
@@ -177,14 +191,15 @@ class PostNormGatedBlock:
         if self.conv is not None:
             h = self.conv.forward(x, ctx, conv_state, cast_out=xh)
         else:
-            ops.gather_rows(xh, x)
+            if not self.input_cast:  # (the block before may have left the rows rounded already)
+                ops.gather_rows(xh, x)
             h = xh
         gate = self.gate_mixer.forward(xh, ctx, "gate_logits") if self.gate_mixer is not None else None
         y = ws.get("sublayer_out", (n, d), torch.float32)
         self.mixer.forward(h, ctx, cache, None if conv_state is not None else state, None, writes_cache=writes_cache, out=y)
         keep = (conv_state, ctx) if conv_state is not None and writes_cache else None
-        ops.gated_norm_add(x, y, self.norm_mixer.weight, self.norm_mixer.eps, gate=gate, cast_out=xh if self.ffn is not None else None,
-                           keep=keep)
+        ops.gated_norm_add(x, y, self.norm_mixer.weight, self.norm_mixer.eps, gate=gate,
+                           cast_out=xh if self.ffn is not None or self.casts_last else None, keep=keep, **self._norm_of(self.norm_mixer))
         if self.ffn is not None:
             if ctx.phases is not None:
                 ctx.phases.mark(self.ffn_phase)
@@ -198,7 +213,8 @@ class PostNormGatedBlock:
             else:
                 gate = self.gate_ffn.forward(xh, ctx, "gate_logits") if self.gate_ffn is not None else None
                 self.ffn.forward(xh, ctx, None, out=y)
-            ops.gated_norm_add(x, y, self.norm_ffn.weight, self.norm_ffn.eps, n_sum=k, gate=gate)
+            ops.gated_norm_add(x, y, self.norm_ffn.weight, self.norm_ffn.eps, n_sum=k, gate=gate, cast_out=xh if self.casts_last else None,
+                               **self._norm_of(self.norm_ffn))
         return None
 
 

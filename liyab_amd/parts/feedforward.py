@@ -97,6 +97,49 @@ class ClampedGLU:
 register_ffn("clamped_glu", ClampedGLU)
 
 
+class GatedFFN:
+    """down(act(gate h) * (up h)): the two projections run as one product [gate | up] whose 32-bit sums the activation kernel reads;
+    the inner rows are rounded once, for the second product."""
+
+    replayable = True
+    takes_padding_rows = True
+
+    def __init__(self, spec, store, dtype: torch.dtype):
+        from ..kernels import ops
+
+        self.dtype = dtype
+        self.width, self.inner, self.activation = spec.width, spec.inner, spec.activation
+        if self.activation not in ops.GLU_ACTIVATIONS:
+            raise ValueError(f"gated feed-forward: activation '{self.activation}' is not known")
+        t = spec.tensors
+        self.in_weight = store.fetch_joined([t["gate"], t["up"]], [(self.inner, self.width)] * 2, "matrix", "rows")
+        self.down_weight = store.fetch(t["down"], (self.width, self.inner), "matrix")
+
+    def begin(self, h, ctx: StepContext) -> torch.Tensor:
+        """The first product, [gate | up] of h in 32 bits: everything of the feed-forward that reads its input."""
+        gu = ctx.workspace.get("glu_in", (h.shape[0], 2 * self.inner), torch.float32)
+        linear(h, self.in_weight, None, out=gu)
+        return gu
+
+    def finish(self, gu: torch.Tensor, ctx: StepContext, residual: Optional[torch.Tensor], out: Optional[torch.Tensor] = None):
+        from ..kernels import ops
+
+        inner = ctx.workspace.get("ffn_inner", (gu.shape[0], self.inner), self.dtype)
+        ops.glu(inner, gu, self.activation)
+        if out is not None:
+            linear(inner, self.down_weight, None, out=out)
+        else:
+            linear(inner, self.down_weight, None, residual=settled(residual))
+        return None
+
+    def forward(self, h, ctx: StepContext, residual: Optional[torch.Tensor], out: Optional[torch.Tensor] = None):
+        """Adds the result into `residual` (float32 [n, width]), or leaves it in `out`."""
+        return self.finish(self.begin(h, ctx), ctx, residual, out=out)
+
+
+register_ffn("gated_ffn", GatedFFN)
+
+
 class NormedPowersFFN:
     """down(c1 N(z) + c2 N(z^2) + c3 N(z^3) + c4) with z = up h, powers entry by entry and N(v) = v / sqrt(mean(v^2) + eps) over the
     inner width: the first product leaves its 32-bit sums, one kernel takes the three means of a row and mixes the powers, and the inner

@@ -62,6 +62,7 @@ class LayerNorm:
         self.weight = store.fetch(w, (self.width,), "vector") if w is not None else None
         self.bias = store.fetch(b, (self.width,), "vector") if b is not None else None
 
+    centred = True  # (what `ops.gated_norm_add(centred=True)` applies, given this part's weight, bias and eps)
     fusable = "layernorm"  # product kernels know how to fold this norm into their operand
 
     def takes_planes(self, planes: torch.Tensor) -> bool:

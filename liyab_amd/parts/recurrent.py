@@ -10,6 +10,7 @@ from ..cache.pages import StateSpec
 from ..errors import Unsupported
 from ..kernels import ops
 from .base import StepContext, settled
+from .delta_rule import own_state
 from .linear import linear
 from .norms import as_tensor
 from .registry import register_mixer
@@ -137,5 +138,53 @@ class StateSpace:
         return None
 
 
+class GatedLinearAttention:
+    """q, k, v = W h a head (keys and values of widths of their own); a decay a key channel w = sigmoid(W2 (W1 h) + b)^(1 / tau);
+    S <- diag(w) S + k v^T, o = S^T q * q_scale; each head's o brought to unit root mean square, times a weight shared by the heads and
+    silu(Wg h), then the output projection. The five projections of h run as one product left in 32 bits; the decay's second, narrow
+    product runs in 32-bit multiply-adds on those sums, since a decay is multiplied by itself over hundreds of tokens. A request's slot
+    holds the heads' matrices [heads, key, value], 32-bit."""
+
+    replayable = True
+    takes_padding_rows = True
+
+    def __init__(self, spec, store, dtype: torch.dtype):
+        self.dtype = dtype
+        self.width, self.n_head, self.head_dim, self.value_dim = spec.width, spec.n_head, spec.head_dim, spec.value_dim
+        self.rank, self.tau, self.eps, self.q_scale = spec.decay_rank, float(spec.tau), float(spec.eps), float(spec.q_scale)
+        H, D, V, d, R = self.n_head, self.head_dim, self.value_dim, self.width, self.rank
+        if not ops.scan_takes(D, V):
+            raise Unsupported(f"gated linear attention: keys of {D} over values of {V} are not supported")
+        t = spec.tensors
+        self.in_weight = store.fetch_joined([t[c] for c in ("q", "k", "v", "g", "w1")], [(H * D, d), (H * D, d), (H * V, d), (H * V, d), (R, d)], "matrix", "rows")
+        w2 = store.fetch(t["w2"], (H * D, R), "vector")
+        self.w2 = store.derived(("rank_first", t["w2"].name), lambda: w2.t().contiguous())  # [rank, channels]
+        self.w2_bias = store.fetch(t["w2_bias"], (H * D,), "vector")
+        self.norm = store.fetch(t["norm"], (V,), "vector")
+        self.out_weight = store.fetch(t["out"], (d, H * V), "matrix")
+
+    def cache_spec(self):
+        return None
+
+    def state_spec(self) -> Optional[StateSpec]:
+        return StateSpec((self.n_head * self.head_dim * self.value_dim,))
+
+    def forward(self, h, ctx: StepContext, cache, state, residual: Optional[torch.Tensor], writes_cache: bool = True,
+                out: Optional[torch.Tensor] = None):
+        h = as_tensor(h)
+        n, ws = h.shape[0], ctx.workspace
+        proj = ws.get("gla_in", (n, self.in_weight.shape[0]), torch.float32)
+        linear(h, self.in_weight, None, out=proj)
+        y = ws.get("gla_out", (n, self.n_head * self.value_dim), self.dtype)
+        ops.gla(y, proj, self.w2, self.w2_bias, self.norm, self.tau, self.eps, own_state(state, self.n_head * self.head_dim * self.value_dim), ctx,
+                n_head=self.n_head, head_dim=self.head_dim, value_dim=self.value_dim, q_scale=self.q_scale)
+        if out is not None:
+            linear(y, self.out_weight, None, out=out)
+        else:
+            linear(y, self.out_weight, None, residual=settled(residual))
+        return None
+
+
 register_mixer("wkv", WKV)
+register_mixer("gated_linear_attention", GatedLinearAttention)
 register_mixer("state_space", StateSpace)

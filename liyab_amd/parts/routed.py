@@ -22,7 +22,7 @@ class RoutedFFN:
     with the router's weight; an entry's row is added to the others of its token by the reader.
     The spec's options: experts without a gate, Wdown_e act(Wup_e h), with act = the square of the positive part; the choice
     among groups of experts (scores by a softmax over all experts, the best groups only, weights divided by their sum:
-    `ops.moe_route(groups=)`); one more expert of the same form that every token takes with weight one, whose result is one
+    `ops.moe_route(groups=)`); scores by the logistic function with a correction on the choice (`ops.moe_route(logistic=)`); one more expert of the same form that every token takes with weight one, whose result is one
     more row a token for the reader to add."""
 
     replayable = True
@@ -34,6 +34,9 @@ class RoutedFFN:
         self.gated, self.activation = bool(getattr(spec, "gated", True)), spec.activation
         if (self.gated and self.activation != "silu") or (not self.gated and self.activation != "relu2"):
             raise ValueError(f"routed feed-forward: activation '{spec.activation}' of {'gated' if self.gated else 'ungated'} experts is not known")
+        self.logistic = getattr(spec, "scores", "softmax") == "logistic"
+        if not self.logistic and getattr(spec, "scores", "softmax") != "softmax":
+            raise ValueError(f"routed feed-forward: scores '{spec.scores}'")
         self.groups = tuple(int(v) for v in spec.groups) if getattr(spec, "groups", None) is not None else None
         self.shared_inner = int(getattr(spec, "shared_inner", 0) or 0)
         if not 1 <= self.top <= min(self.n_experts, ops.MOE_MAX_TOP):
@@ -41,6 +44,7 @@ class RoutedFFN:
         t, E, F, d = spec.tensors, self.n_experts, self.inner, self.width
         self.router = store.fetch(t["router"], (E, d), "matrix")
         self.router_bias = store.fetch(t["router_bias"], (E,), "vector") if "router_bias" in t else None
+        self.correction = store.fetch(t["correction"], (E,), "vector") if self.logistic and "correction" in t else None
         self.gate = store.fetch_joined([t[("gate", e)] for e in range(E)], [(F, d)] * E, "matrix", "stack") if self.gated else None
         self.up = store.fetch_joined([t[("up", e)] for e in range(E)], [(F, d)] * E, "matrix", "stack")
         self.down = store.fetch_joined([t[("down", e)] for e in range(E)], [(d, F)] * E, "matrix", "stack")
@@ -89,7 +93,7 @@ class RoutedFFN:
         weights = ws.get("routed_weights", (n * top,), torch.float32)
         rows_list = ws.get("routed_rows", (tiles * block,), torch.int32)
         tile_group = ws.get("routed_tiles", (tiles,), torch.int32)
-        ops.moe_route(logits, top, ids, weights, rows_list, tile_group, block=block, groups=self.groups)
+        ops.moe_route(logits, top, ids, weights, rows_list, tile_group, block=block, groups=self.groups, logistic=self.logistic, correction=self.correction)
         inner = ws.get("routed_inner", (n * top, self.inner), self.dtype)
         if self.gated:
             ops.moe_product(inner, h, self.gate, self.up, rows_list, tile_group, a_div=top, block=block)

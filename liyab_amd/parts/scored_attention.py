@@ -23,7 +23,7 @@ def rotary_frequencies(rot) -> np.ndarray:
     """f_i = base^(-2i / dims) for i < dims / 2, the long wavelengths stretched as `rot.scaling` = (factor, low, high,
     original) says: with wavelength l = 2 pi / f, f stays for l < original / high, becomes f / factor for l > original /
     low, and in between is (1 - s) f / factor + s f with s = (original / l - low) / (high - low); or as `rot.ramp` = (factor,
-    fast, slow, original) says, by the entry's number (see RotarySpec). float64."""
+    fast, slow, original) says, by the entry's number (see RotarySpec); all divided by `rot.linear`. float64."""
     f = np.array([float(rot.base) ** (-2.0 * i / rot.dims) for i in range(rot.dims // 2)], dtype=np.float64)
     if rot.scaling is not None:
         factor, low, high, original = (float(v) for v in rot.scaling)
@@ -47,7 +47,7 @@ def rotary_frequencies(rot) -> np.ndarray:
         for i, fi in enumerate(f):
             r = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
             f[i] = fi / factor * r + fi * (1.0 - r)
-    return f
+    return f / float(getattr(rot, "linear", 1.0) or 1.0)
 
 
 def rotary_magnitude(rot) -> float:
@@ -76,7 +76,8 @@ class ScoredAttention:
     kernel then norms, turns and scales the heads as the spec says and writes queries to a buffer and keys and values to
     their pages (keys `head_dim` wide, values `value_dim`: two planes of the cache with widths of their own); the attention
     kernel applies the soft cap and the bias by distance to the scores, and the gate to its result; then the output
-    projection. The bias by distance is looked up in a table a distance [distance_bias + 1, heads] made once from the learned
+    projection. Norms over a token's whole queries and keys (`qk_norm_rows`) are taken by a kernel with a workgroup a token. A layer
+    whose keys and values are another's (`kv_shared`) projects queries only and reads that layer's pages. The bias by distance is looked up in a table a distance [distance_bias + 1, heads] made once from the learned
     rows, so that no kernel computes a logarithm a key."""
 
     replayable = True
@@ -97,11 +98,21 @@ class ScoredAttention:
         self.values_are_keys, self.gated = bool(spec.values_are_keys), bool(spec.gated)
         H, G, D, V, d = self.n_head, self.n_kv_head, self.head_dim, self.value_dim, self.width
         t = spec.tensors
-        srcs, shapes = [t["q"], t["k"]], [(H * D, d), (G * D, d)]
+        self.kv_shared, self.norm_rows = bool(getattr(spec, "kv_shared", False)), bool(getattr(spec, "qk_norm_rows", False))
+        self.keep_first = int(getattr(spec, "keep_first", 0) or 0) if self.window > 0 else 0
+        if self.kv_shared and not (self.norm_rows and not spec.values_are_keys and not getattr(spec, "biased", False) and not getattr(spec, "value_mix", "")):
+            raise Unsupported("scored attention: another layer's keys and values go with norms over whole rows, and without biases or shared values")
+        if self.norm_rows and (spec.qk_norm or spec.q_temp or spec.values_are_keys or getattr(spec, "value_mix", "") or (spec.rotary is not None and spec.rotary.ramp is not None)):
+            raise Unsupported("scored attention: norms over whole rows do not go with norms a head, a query factor, shared values or a ramp")
+        srcs, shapes = [t["q"]], [(H * D, d)]
         self.q_off, self.k_off = 0, H * D
-        at = H * D + G * D
+        at = H * D
+        if not self.kv_shared:
+            srcs.append(t["k"])
+            shapes.append((G * D, d))
+            at += G * D
         self.v_off = self.k_off
-        if not self.values_are_keys:
+        if not self.values_are_keys and not self.kv_shared:
             srcs.append(t["v"])
             shapes.append((G * V, d))
             self.v_off, at = at, at + G * V
@@ -136,8 +147,10 @@ class ScoredAttention:
             P = self.row_dim = -(-max(D, V) // 8) * 8
             w = self.out_weight
             self.out_weight = store.derived(("padded_heads", t["out"].name, P), lambda: torch.nn.functional.pad(w.view(d, H, V), (0, P - V)).reshape(d, H * P).contiguous())
-        self.q_norm = store.fetch(t["q_norm"], (D,), "vector") if spec.qk_norm else None
-        self.k_norm = store.fetch(t["k_norm"], (D,), "vector") if spec.qk_norm else None
+        per_q, per_k = (H * D, G * D) if self.norm_rows else (D, D)
+        normed = spec.qk_norm or self.norm_rows
+        self.q_norm = store.fetch(t["q_norm"], (per_q,), "vector") if normed else None
+        self.k_norm = store.fetch(t["k_norm"], (per_k,), "vector") if normed and not self.kv_shared else None
         self.rot_dims, self.freqs, self.rot_halves, self.rot_mag = 0, None, False, 1.0
         if spec.rotary is not None:
             rot = spec.rotary
@@ -145,7 +158,7 @@ class ScoredAttention:
                 raise ValueError(f"rotary encoding over {rot.dims} of {D} entries")
             self.rot_dims = int(rot.dims)
             self.rot_halves, self.rot_mag = bool(getattr(rot, "halves", False)), rotary_magnitude(rot)
-            self.freqs = store.derived(("rotary", rot.dims, rot.base, rot.scaling, getattr(rot, "ramp", None)),
+            self.freqs = store.derived(("rotary", rot.dims, rot.base, rot.scaling, getattr(rot, "ramp", None), getattr(rot, "linear", 1.0)),
                                        lambda: torch.from_numpy(rotary_frequencies(rot).astype(np.float64)).to(self.out_weight.device))
         self.temp_coef, self.temp_every = (float(spec.q_temp[0]), int(spec.q_temp[1])) if spec.q_temp else (0.0, 0)
         self.bias_table = None
@@ -164,7 +177,7 @@ class ScoredAttention:
         return {"v_keep": rows} if self.value_mix == "first" else {"v_first": rows, "v_lam": self.v_lam}
 
     def cache_spec(self) -> Optional[KVSpec]:
-        return KVSpec(self.n_kv_head, self.head_dim, self.window,
+        return KVSpec(self.n_kv_head, self.head_dim, self.window, keep_first=self.keep_first,
                       rows=(("k", self.n_kv_head, self.row_dim or self.head_dim), ("v", self.n_kv_head, self.row_dim or self.value_dim)))
 
     def state_spec(self):
@@ -187,19 +200,24 @@ class ScoredAttention:
             linear(h, self.in_weight, self.in_bias, out=proj)
         P = self.row_dim
         q = ws.get("scored_q", (n, H * (P or D)), self.dtype)
-        if not writes_cache:
-            raise Unsupported("scored attention: a run that reads another run's cache is not supported")
-        ops.qk_prepare(proj, q, cache.k, cache.v, group.slots, ctx.positions, q_off=self.q_off, k_off=self.k_off, v_off=self.v_off,
-                       n_head=H, q_norm=self.q_norm, k_norm=self.k_norm, eps=self.eps, freqs=self.freqs, rot_dims=self.rot_dims,
-                       temp_coef=self.temp_coef, temp_every=self.temp_every, head_dim=D, value_dim=V, rot_halves=self.rot_halves,
-                       rot_mag=self.rot_mag, **self._shared_values(ws, n))
+        if writes_cache == self.kv_shared:
+            raise Unsupported("scored attention: a run that reads another run's cache needs a layer without keys and values of its own, and such a layer another's cache")
+        if self.norm_rows:
+            ops.qk_prepare_rows(proj, q, None if self.kv_shared else cache.k, None if self.kv_shared else cache.v, group.slots, ctx.positions, q_off=self.q_off,
+                                k_off=self.k_off, v_off=self.v_off, n_head=H, n_kv_head=self.n_kv_head, head_dim=D, value_dim=V, q_norm=self.q_norm,
+                                k_norm=self.k_norm, eps=self.eps, freqs=self.freqs, rot_dims=self.rot_dims, rot_halves=self.rot_halves)
+        else:
+            ops.qk_prepare(proj, q, cache.k, cache.v, group.slots, ctx.positions, q_off=self.q_off, k_off=self.k_off, v_off=self.v_off,
+                           n_head=H, q_norm=self.q_norm, k_norm=self.k_norm, eps=self.eps, freqs=self.freqs, rot_dims=self.rot_dims,
+                           temp_coef=self.temp_coef, temp_every=self.temp_every, head_dim=D, value_dim=V, rot_halves=self.rot_halves,
+                           rot_mag=self.rot_mag, **self._shared_values(ws, n))
         att = ws.get("scored_att", (n, H * (P or V)), self.dtype)
         gate = proj[:, self.gate_off:self.gate_off + H * V] if self.gated else None
         if D == V or P:
             # keys and values of one width: the paged attention kernels of the engine (tiles of a prompt's queries on the matrix
             # cores, single tokens in splits, the 32-bit form), which cap and bias the scores when asked to
             splits = ops.attention(att, q, cache.k, cache.v, group.block_tables, ctx, n_head=H, scale=self.scale, window=self.window,
-                                   softcap=self.softcap, bias_table=self.bias_table, sinks=self.sinks)
+                                   softcap=self.softcap, bias_table=self.bias_table, sinks=self.sinks, keep_first=self.keep_first)
             assert splits is None
             if gate is not None:
                 ops.gate_rows(att, gate, out_scale)
@@ -209,7 +227,7 @@ class ScoredAttention:
             if out_scale != 1.0:
                 raise Unsupported("scored attention: a factor on the result needs the gate's pass (can_scale_output)")
             ops.attention_scored(att, q, cache.k, cache.v, group.block_tables, ctx, n_head=H, scale=self.scale, softcap=self.softcap,
-                                 window=self.window, bias_table=self.bias_table, gate=gate, sinks=self.sinks)
+                                 window=self.window, bias_table=self.bias_table, gate=gate, sinks=self.sinks, keep_first=self.keep_first)
         if out is not None and add:
             linear(att, self.out_weight, None, residual=out)
         elif out is not None:
