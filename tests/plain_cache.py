@@ -25,6 +25,7 @@ class KVSpec:
     n_kv_head: int
     head_dim: int
     window: int = 0  # 0: every position is kept; W > 0: only the last W are read
+    keep_first: int = 0  # with a window: the first positions that are read too
 
     @property
     def key(self) -> Tuple[int, int, int]:
@@ -223,7 +224,10 @@ class CacheManager:
             keep_from = first_needed // self.page_size
             table = r.tables[gi]
             gone = []
-            for lp in range(r.first_kept[gi], min(keep_from, len(table))):
+            always = self._pages_for(g.spec.keep_first)  # pages no window passes
+            if min(keep_from, len(table)) <= always:
+                continue
+            for lp in range(max(r.first_kept[gi], always), min(keep_from, len(table))):
                 if table[lp] != UNMAPPED:
                     gone.append(table[lp])
                     table[lp] = UNMAPPED

@@ -176,7 +176,30 @@ def test_random_orders_lose_nothing(seed):
     assert m.pages_in_use(0) == 0 and m.pages_in_use(1) == 0 and m.free_slots() == 5
 
 
-@pytest.mark.parametrize("seed", range(8))
+def test_a_window_that_keeps_the_first_positions_keeps_their_pages():
+    """Pages of the kept first positions stay however far the window moves; pages between them and the window go; what a request
+    held comes back when it closes; a window that still touches the kept pages gives nothing back."""
+    m = CacheManager([(KVSpec(2, 16, 10, keep_first=5), [0])], page_size=4, num_pages=20, max_requests=2, max_positions=80)
+    m.open("r")
+    m.reserve([("r", 12)])
+    m.commit("r", 12)
+    assert UNMAPPED not in m.block_table("r")  # positions 3.. are in the window, page 0 holds kept ones
+    m.reserve([("r", 40)])
+    m.commit("r", 40)
+    table = m.block_table("r")  # a query at 40 reads 31..40 and 0..4: pages 0, 1 and 7..9
+    assert [i for i, page in enumerate(table) if page != UNMAPPED] == [0, 1, 7, 8, 9]
+    kept = table[:2]
+    for length in range(41, 77):
+        m.reserve([("r", length)])
+        m.commit("r", length)
+        assert m.block_table("r")[:2] == kept and m.pages_in_use() <= 2 + 4
+        m.check()
+    m.close("r")
+    assert m.pages_in_use() == 0
+    m.check()
+
+
+@pytest.mark.parametrize("seed", range(14))
 def test_native_manager_does_what_the_plain_one_does(seed):
     """The same random operations on the native manager and on the plain Python one: the same
     pages in the same places, the same counters, the same refusals."""
@@ -186,10 +209,11 @@ def test_native_manager_does_what_the_plain_one_does(seed):
     window = rng.choice([0, 24, 70])
     page_size = rng.choice([4, 16])
     pages = [rng.randint(10, 40), rng.randint(10, 40)]
-    specs = [(KVSpec(2, 16, 0), [0]), (KVSpec(2, 16, window), [1])]
+    keep = rng.choice([0, 3, 30]) if seed >= 8 else 0
+    specs = [(KVSpec(2, 16, 0), [0]), (KVSpec(2, 16, window, keep_first=keep), [1])]
     kw = dict(page_size=page_size, num_pages=pages, max_requests=4, max_positions=200)
     a = CacheManager(specs, **kw)
-    b = plain_cache.CacheManager([(plain_cache.KVSpec(2, 16, 0), [0]), (plain_cache.KVSpec(2, 16, window), [1])], **kw)
+    b = plain_cache.CacheManager([(plain_cache.KVSpec(2, 16, 0), [0]), (plain_cache.KVSpec(2, 16, window, keep), [1])], **kw)
     live, n = {}, 0
 
     def both(op):
