@@ -6,7 +6,7 @@
     python bench.py --workload medium16|xl64         # the continuous-batching and the batch-64 workloads of the larger sizes
     python bench.py --link-floor                     # what one dependent kernel of a replayed graph costs at least
     python bench.py --product 4096,4096,16384,8,15   # one product in tiles of 128 x 128 and of 256 x 256
-    python bench.py --design bokulix|mofulix|dopilorn|larulorn [--design-sizes small,medium,xl] [--layers L] [--phases]   # that design beside GPT-2 (dopilorn, larulorn: beside Mofulix) at equal sizes
+    python bench.py --design bokulix|mofulix|dopilorn|larulorn|lolulorn [--design-sizes small,medium,xl] [--layers L] [--phases]   # that design beside GPT-2 (dopilorn, larulorn: beside Mofulix; lolulorn: beside Larulorn) at equal sizes
 
 The default run has GPT-2 small's layer sizes (12 layers, width 768, 12 heads
 of 64, feed-forward 3072, vocabulary 50257, 1024 positions) with random
@@ -642,11 +642,92 @@ def larulorn_prefill_flops(cfg, prompt_lens, logit_rows):
     return flops
 
 
+# The Lolulorn of each size has GPT-2's width, layers, vocabulary and head count (heads of 64 everywhere); its layers take turns as a gated
+# delta rule (half as many query/key heads as value heads where the number is even, four taps) over a gated feed-forward two thirds as wide
+# as GPT-2's, gated linear attention (a decay of rank 16) over eight gated experts of a quarter of GPT-2's inner width in four groups of
+# which two stay, two a token, and attention under a window of half the positions behind which four first positions stay visible, over the
+# same dense feed-forward; every second attention layer reads the keys and values of the one before it. It stands beside Larulorn, the
+# engine's closest design: attention and recurrences, one sublayer after the other with a norm behind each, experts chosen among groups.
+def lolulorn_config(gpt2_cfg):
+    d, H, F, L = gpt2_cfg["n_embd"], gpt2_cfg["n_head"], gpt2_cfg["n_inner"], gpt2_cfg["n_layer"]
+    hd = d // H
+    dense = {"kind": "dense", "ff": max(64, F * 2 // 3 // 64 * 64)}
+    moe = {"kind": "moe", "expert": {"ff": F // 4}, "router": {"experts": 8, "top": 2, "groups": {"count": 4, "keep": 2}}}
+    attention = {"heads": H, "kv_heads": H, "dim": hd, "vdim": hd, "scale": hd ** -0.5, "mask": {"size": gpt2_cfg["n_positions"] // 2, "keep_first": 4},
+                 "rot": {"dims": hd, "base": 10000.0, "scaling": {"factor": 4.0}}}
+    layers = []
+    for i in range(L):
+        if i % 3 == 0:
+            layers.append({"type": "delta", "mixer": {"heads": H, "kv_heads": H // 2 if H % 2 == 0 else H, "dim": hd, "vdim": hd, "conv": 4}, "mlp": dense})
+        elif i % 3 == 1:
+            layers.append({"type": "gla", "mixer": {"heads": H, "dim": hd, "vdim": hd, "tau": 16.0, "decay_rank": 16}, "mlp": moe})
+        else:
+            layers.append({"type": "attention", "mixer": dict(attention, **({"kv_from": i - 3} if i % 6 == 5 else {})), "mlp": dense})
+    return {"architecture": "Lolulorn", "vocab": gpt2_cfg["vocab_size"], "width": d, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-5},
+            "max_positions": gpt2_cfg["n_positions"], "layers": json.loads(json.dumps(layers))}
+
+
+def _lolulorn_layer_weights(entry, d, experts=None):
+    """Matrix elements of a layer that a token's products read (2 flops an element a token), with `experts` experts in place of a token's own."""
+    m, mlp = entry["mixer"], entry.get("mlp")
+    n = 0
+    if mlp and mlp["kind"] == "dense":
+        n += 3 * mlp["ff"] * d
+    elif mlp:
+        n += mlp["router"]["experts"] * d + (experts or mlp["router"]["top"]) * 3 * mlp["expert"]["ff"] * d
+    H, D, V = m["heads"], m["dim"], m["vdim"]
+    n += d * H * V
+    if entry["type"] == "attention":
+        n += H * D * d + (0 if "kv_from" in m else m["kv_heads"] * (D + V) * d)
+    elif entry["type"] == "delta":
+        n += (2 * m["kv_heads"] * D + 2 * H * V + 2 * H) * d
+    else:
+        n += (2 * H * D + 2 * H * V + m["decay_rank"]) * d + H * D * m["decay_rank"]
+    return n
+
+
+def lolulorn_step_bytes(cfg, batch):
+    """The bytes a decode step has to read: every matrix a token of the batch can take (min(batch * top, experts) experts), the head, the
+    cached keys and values inside each request's window, and the 32-bit state of the recurrent layers (read and written) a request."""
+    def step_bytes(contexts, steps, elt):
+        d, V = cfg["width"], cfg["vocab"]
+        total = V * d * elt
+        for entry in cfg["layers"]:
+            m, mlp = entry["mixer"], entry.get("mlp")
+            r = mlp["router"] if mlp and mlp["kind"] == "moe" else None
+            total += _lolulorn_layer_weights(entry, d, min(len(contexts) * r["top"], r["experts"]) if r else None) * elt
+            if entry["type"] == "attention":
+                reach = m["mask"]["size"] + m["mask"]["keep_first"]
+                seen = sum(sum(min(c + s + 1, reach) for s in range(steps)) for c in contexts) / max(steps, 1)
+                total += seen * m["kv_heads"] * (m["dim"] + m["vdim"]) * elt
+            else:
+                total += len(contexts) * 2 * m["heads"] * m["dim"] * m["vdim"] * 4
+                if entry["type"] == "delta":
+                    total += len(contexts) * m["conv"] * (2 * m["kv_heads"] * m["dim"] + m["heads"] * m["vdim"]) * 4
+        return total
+    return step_bytes
+
+
+def lolulorn_prefill_flops(cfg, prompt_lens, logit_rows):
+    d, V, n = cfg["width"], cfg["vocab"], sum(prompt_lens)
+    flops = 2.0 * logit_rows * d * V
+    for entry in cfg["layers"]:
+        m = entry["mixer"]
+        flops += 2.0 * n * _lolulorn_layer_weights(entry, d)
+        if entry["type"] == "attention":
+            reach = m["mask"]["size"] + m["mask"]["keep_first"]
+            flops += 2.0 * sum(min(i + 1, reach) for t in prompt_lens for i in range(t)) * m["heads"] * (m["dim"] + m["vdim"])
+        else:
+            flops += n * m["heads"] * m["dim"] * m["vdim"] * (8.0 if entry["type"] == "delta" else 5.0)  # (the recurrence token by token)
+    return flops
+
+
 DESIGNS = {"bokulix": (lambda gpt2, size: bokulix_config(gpt2, BOKULIX_SHAPES[size]), bokulix_step_bytes, bokulix_prefill_flops),
            "mofulix": (lambda gpt2, size: mofulix_config(gpt2), mofulix_step_bytes, mofulix_prefill_flops),
            "dopilorn": (lambda gpt2, size: dopilorn_config(gpt2), dopilorn_step_bytes, dopilorn_prefill_flops),
-           "larulorn": (lambda gpt2, size: larulorn_config(gpt2), larulorn_step_bytes, larulorn_prefill_flops)}
-BESIDE = {"dopilorn": "mofulix", "larulorn": "mofulix"}  # the engine's closest model, where that is not GPT-2
+           "larulorn": (lambda gpt2, size: larulorn_config(gpt2), larulorn_step_bytes, larulorn_prefill_flops),
+           "lolulorn": (lambda gpt2, size: lolulorn_config(gpt2), lolulorn_step_bytes, lolulorn_prefill_flops)}
+BESIDE = {"dopilorn": "mofulix", "larulorn": "mofulix", "lolulorn": "larulorn"}  # the engine's closest model, where that is not GPT-2
 
 
 def design_run(args):
@@ -724,9 +805,9 @@ def main():
     ap.add_argument("--link-floor", action="store_true", help="measure what one dependent kernel of a replayed graph costs at least")
     ap.add_argument("--phases", action="store_true", help="device milliseconds per phase of the forward pass (embed, attention, dense_ffn, lm_head) a decode step "
                     "and a prefill of 2,048 tokens, as the reference's command line prints them (tools/liyab_cli.cpp:198-211); steps run kernel by kernel, without graphs")
-    ap.add_argument("--design", default="", choices=["", "bokulix", "mofulix", "dopilorn", "larulorn"],
+    ap.add_argument("--design", default="", choices=["", "bokulix", "mofulix", "dopilorn", "larulorn", "lolulorn"],
                     help="bokulix, mofulix: that design beside GPT-2 at equal layer sizes (prefill and decode, both with their rooflines); "
-                         "dopilorn, larulorn: beside Mofulix, the engine's closest model")
+                         "dopilorn, larulorn: beside Mofulix, lolulorn: beside Larulorn, the engine's closest model")
     ap.add_argument("--design-only", action="store_true", help="with --design: skip the GPT-2 run (for profiling)")
     ap.add_argument("--design-sizes", default="small,medium,xl", help="the sizes --design runs (of small, medium, xl)")
     args = ap.parse_args()
