@@ -15,7 +15,7 @@
 //   A step with long portions (seg_tokens > 0) runs in segments of that many tokens side by side, in three launches. The
 //   recurrence is linear in S, S_t = A_t S_(t-1) + k_t v_t^T with A_t = diag(w_t) - (a_t * u_t) u_t^T, so a segment's end is
 //   P S_start + Z: every segment but a request's last walks twice side by side, from a zero state for Z and, without the outer
-//   products, from the unit matrix for P (the product of its A_t); delta_combine_kernel (delta_segments.h) strings a request's segments
+//   products, from the unit matrix for P (the product of its A_t); combine_segments (delta_segments.h) strings a request's segments
 //   together and leaves each the state it starts from; then every segment walks from that state and writes its outputs.
 // liyab_head_norm_gate: out = o / sqrt(mean(o^2 over the head) + eps) * weight * sigmoid(gate) (silu: * gate * sigmoid(gate)), rounded
 //   once; a weight an entry of the row, or one of a head's width for all heads (shared_w).
@@ -384,7 +384,7 @@ extern "C" int liyab_delta_scan(float* out, const float* r, const float* k, cons
         p.phase = 1;
         walk(p, static_cast<int64_t>(max_segs) * 2, false);
         const DeltaSegments segs{state, state_stride, n_slots, seq_starts, positions, state_slots, n_seqs, H, D, D, seg_tokens};
-        delta_combine_kernel<<<dim3(n_seqs, H, n_cb), 256, 0, stream>>>(segs, seg_state, seg_trans, seg_start);
+        combine_segments(segs, seg_state, seg_trans, seg_start, stream);
         p.phase = 3;
         walk(p, max_segs, true);
         return check_launch("delta_scan");

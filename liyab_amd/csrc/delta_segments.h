@@ -146,4 +146,105 @@ delta_combine_kernel(DeltaSegments a, const float* __restrict__ seg_z, const flo
     }
 }
 
+// The same for D up to 64 on the matrix cores in 32-bit floats (v_mfma_f32_16x16x4_f32): a workgroup a (request, head, 16 columns),
+// its wave w rows 16 w .. 16 w + 15. What the chain over segments waits for is the trip of each segment's P and Z from memory, not the
+// arithmetic: a wave's operand of P goes straight into registers, kCombDepth segments ahead, and only S passes through LDS. In step q of
+// the product the four groups of 16 lanes hold rows 16 g + q of S (g the group), so that a lane's entries of P are 16 in a row.
+constexpr int kCombDepth = 4;
+typedef __attribute__((ext_vector_type(4))) float comb_f32x4;
+
+template <bool WHOLE>  // WHOLE: D = 64, P in pieces of four floats; otherwise entries past the matrix are read from inside and taken as zeros
+static __global__ void __launch_bounds__(256)
+delta_combine_mfma_kernel(DeltaSegments a, const float* __restrict__ seg_z, const float* __restrict__ seg_p, float* __restrict__ seg_start) {
+    constexpr int kGroup = 16 * 16 + 16;  // floats of 16 rows of S, the next group's rows in other banks
+    __shared__ float Sl[2][4 * kGroup];
+    const int s = blockIdx.x, h = blockIdx.y, cb = blockIdx.z, tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave;
+    const int D = WHOLE ? 64 : a.D, V = a.V, H = a.H;
+    int g0 = 0;
+    for (int q = 0; q < s; ++q) g0 += (a.seq_starts[q + 1] - a.seq_starts[q] + a.seg_tokens - 1) / a.seg_tokens;
+    const int begin = a.seq_starts[s];
+    const int n_seg = (a.seq_starts[s + 1] - begin + a.seg_tokens - 1) / a.seg_tokens;
+    if (n_seg <= 0) return;
+    const int slot = a.state_slots[s];
+    const bool from_slot = slot >= 0 && slot < a.n_slots && a.positions[begin] != 0;
+    const int li = lane % 16, grp = lane / 16, j = cb * kDeltaCols + li, jc = min(j, V - 1);
+    const int64_t DD = static_cast<int64_t>(D) * D, DV = static_cast<int64_t>(D) * V;
+    const float* S0 = a.state + static_cast<int64_t>(from_slot ? slot : 0) * a.state_stride + h * DV;
+    const int row_p = min(16 * wave + li, D - 1);      // this lane's row of P, columns 16 grp ..
+    const bool row_in = 16 * wave + li < D;
+    // a lane's part of the result: rows 16 wave + 4 grp + r, column j
+    const int row_s = 16 * wave + 4 * grp;
+    float p[kCombDepth][16], z[kCombDepth][4];
+    auto fetch = [&](int g, float (&pp)[16], float (&zz)[4]) {
+        const int64_t at = static_cast<int64_t>(g0 + min(g, n_seg - 1)) * H + h;  // (past the last one: read again, not used)
+        const float* P = seg_p + at * DD + static_cast<int64_t>(row_p) * D;
+        const float* Z = seg_z + at * DV;
+        if constexpr (WHOLE) {
+#pragma unroll
+            for (int q4 = 0; q4 < 4; ++q4) {
+                const comb_f32x4 v = *reinterpret_cast<const comb_f32x4*>(P + 16 * grp + 4 * q4);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) pp[4 * q4 + e] = v[e];
+            }
+        } else {
+#pragma unroll
+            for (int q = 0; q < 16; ++q) {
+                const float v = P[min(16 * grp + q, D - 1)];
+                pp[q] = row_in && 16 * grp + q < D ? v : 0.0f;
+            }
+        }
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const float v = Z[static_cast<int64_t>(min(row_s + r, D - 1)) * V + jc];
+            zz[r] = row_s + r < D && j < V ? v : 0.0f;
+        }
+    };
+#pragma unroll
+    for (int u = 0; u < kCombDepth; ++u) fetch(u, p[u], z[u]);
+    float S[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+        const float v = S0[static_cast<int64_t>(min(row_s + r, D - 1)) * V + jc];
+        S[r] = from_slot && row_s + r < D && j < V ? v : 0.0f;
+    }
+    for (int gb = 0; gb < n_seg; gb += kCombDepth) {
+#pragma unroll
+        for (int u = 0; u < kCombDepth; ++u) {
+            const int g = gb + u;
+            if (g >= n_seg) break;  // (the same for the whole workgroup)
+            float* out = seg_start + (static_cast<int64_t>(g0 + g) * H + h) * DV;
+            if (j < V) {
+#pragma unroll
+                for (int r = 0; r < 4; ++r)
+                    if (row_s + r < D) out[static_cast<int64_t>(row_s + r) * V + j] = S[r];
+            }
+            if (g + 1 >= n_seg) break;
+            float* buf = Sl[g & 1];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) buf[wave * kGroup + (4 * grp + r) * 16 + li] = S[r];
+            lds_barrier();  // (one a segment: the buffer written two segments ago has been read by then)
+            float b[16];
+#pragma unroll
+            for (int q = 0; q < 16; ++q) b[q] = buf[grp * kGroup + q * 16 + li];
+            comb_f32x4 acc0 = {z[u][0], z[u][1], z[u][2], z[u][3]}, acc1 = {0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+            for (int q = 0; q < 16; q += 2) {
+                acc0 = __builtin_amdgcn_mfma_f32_16x16x4f32(p[u][q], b[q], acc0, 0, 0, 0);
+                acc1 = __builtin_amdgcn_mfma_f32_16x16x4f32(p[u][q + 1], b[q + 1], acc1, 0, 0, 0);
+            }
+#pragma unroll
+            for (int r = 0; r < 4; ++r) S[r] = acc0[r] + acc1[r];
+            fetch(g + kCombDepth, p[u], z[u]);
+        }
+    }
+}
+
+// Leaves in seg_start [segments][H][D][V] the state each segment of a step starts from, given every segment's Z and P.
+inline void combine_segments(const DeltaSegments& a, const float* seg_z, const float* seg_p, float* seg_start, hipStream_t stream) {
+    const dim3 grid(a.n_seqs, a.H, (a.V + kDeltaCols - 1) / kDeltaCols);
+    if (a.D == 64) delta_combine_mfma_kernel<true><<<grid, 256, 0, stream>>>(a, seg_z, seg_p, seg_start);
+    else if (a.D < 64) delta_combine_mfma_kernel<false><<<grid, 256, 0, stream>>>(a, seg_z, seg_p, seg_start);
+    else delta_combine_kernel<<<grid, 256, 0, stream>>>(a, seg_z, seg_p, seg_start);
+}
+
 }  // namespace liyab

@@ -9,7 +9,7 @@
 // new row goes to a place nobody reads in that step, so the kernel that reads the ring can write it.
 //
 // liyab_gated_delta_prepare: every token's vectors as the recurrence wants them, float [n, 2 G D + H V + 2 H] = [q | k | v | g | beta];
-//   a wave a (token, head of q, k or v).
+//   a wave a (block of tokens, head of q, k or v).
 // liyab_gated_delta_scan: a workgroup a (request, head, 64 columns) walks the request's rows of the step in order: four lanes side by
 //   side share a column, each with a quarter of its rows in registers; the sums over a column's rows (S^T k and S^T q) come through the
 //   lanes' own data path; tokens' vectors go through LDS a chunk at a time, the next chunk fetched while this one is computed. The last
@@ -45,53 +45,88 @@ struct GdPrepareArgs {
     int n, H, G, D, V;
 };
 
+// A wave takes kGdTokens consecutive rows of the step for one head's channels: a channel's weights are read once, and a row once for
+// all the tokens whose taps it is. What lies before a request's first row of the step (its ring, or nothing) is the exception.
+// TAPS: the number of taps, or 0 for any number (each row then reads its own taps).
+constexpr int kGdTokens = 8;
+
+template <int TAPS>
 __global__ void __launch_bounds__(256)
 gated_delta_prepare_kernel(GdPrepareArgs a) {
-    const int units = 2 * a.G + a.H;
-    const int item = blockIdx.x * 4 + threadIdx.x / kWave, lane = threadIdx.x % kWave;
-    if (item >= a.n * units) return;
-    const int t = item / units, unit = item % units;
+    const int units = 2 * a.G + a.H, taps = TAPS > 0 ? TAPS : a.taps;
+    const int lane = threadIdx.x % kWave;
+    const int item = __builtin_amdgcn_readfirstlane(blockIdx.x * 4 + threadIdx.x / kWave);
+    if (item >= (a.n + kGdTokens - 1) / kGdTokens * units) return;
+    const int t0 = item / units * kGdTokens, unit = item % units;
     const int GD = a.G * a.D, C = 2 * GD + a.H * a.V;
     const bool is_v = unit >= 2 * a.G;
     const int width = is_v ? a.V : a.D;
     const int c0 = is_v ? 2 * GD + (unit - 2 * a.G) * a.V : unit * a.D;
-    const int s = a.tok_seq[t], p = a.positions[t], begin = a.seq_starts[s], slot = a.state_slots[s];
-    const bool slot_ok = slot >= 0 && slot < a.n_slots;
-    const float* ring = a.ring + static_cast<int64_t>(slot_ok ? slot : 0) * a.state_stride;  // (not followed with one tap)
-    float x[kGdMax / kWave];
-    float ss = 0.0f;
+    const int64_t pld = C + 2 * a.H;
+    constexpr int NQ = kGdMax / kWave, BACK = TAPS > 0 ? TAPS - 1 : 0, ROWS = kGdTokens + BACK;
+    float x[kGdTokens][NQ];
 #pragma unroll
-    for (int q = 0; q < kGdMax / kWave; ++q) {
-        const int i = lane + q * kWave;
-        x[q] = 0.0f;
-        if (i < width) {
-            const int c = c0 + i;
+    for (int tt = 0; tt < kGdTokens; ++tt)
+#pragma unroll
+        for (int q = 0; q < NQ; ++q) x[tt][q] = 0.0f;
+#pragma unroll
+    for (int q = 0; q < NQ; ++q) {
+        if (q * kWave >= width) break;  // (the same for the whole wave)
+        const int i = lane + q * kWave, c = c0 + min(i, width - 1);
+        float rows[ROWS], w[TAPS > 0 ? TAPS : 1];
+        if (TAPS > 0) {
+#pragma unroll
+            for (int r = 0; r < ROWS; ++r) rows[r] = a.src[static_cast<int64_t>(min(max(t0 - BACK + r, 0), a.n - 1)) * a.ld + c];
+#pragma unroll
+            for (int jt = 0; jt < TAPS; ++jt) w[jt] = a.cw[static_cast<int64_t>(jt) * C + c];
+        }
+#pragma unroll
+        for (int tt = 0; tt < kGdTokens; ++tt) {
+            const int t = min(t0 + tt, a.n - 1);
+            const int s = a.tok_seq[t], p = a.positions[t], begin = a.seq_starts[s];
             float acc = 0.0f;
-            for (int j = 0; j < a.taps; ++j) {
-                const int back = a.taps - 1 - j;
-                if (p - back < 0) continue;
-                float v;
-                if (t - back >= begin) v = a.src[static_cast<int64_t>(t - back) * a.ld + c];
-                else v = slot_ok ? ring[static_cast<int64_t>((p - back) % a.taps) * C + c] : 0.0f;
-                acc = fmaf(a.cw[static_cast<int64_t>(j) * C + c], v, acc);
+            if (TAPS > 0 && t - BACK >= begin && p >= BACK) {  // (the same for the whole wave, as everything but the channel)
+#pragma unroll
+                for (int jt = 0; jt < TAPS; ++jt) acc = fmaf(w[jt], rows[tt + jt], acc);
+            } else {
+                const int slot = a.state_slots[s];
+                const bool slot_ok = slot >= 0 && slot < a.n_slots;
+                const float* ring = a.ring + static_cast<int64_t>(slot_ok ? slot : 0) * a.state_stride;  // (not followed with one tap)
+                for (int jt = 0; jt < taps; ++jt) {
+                    const int back = taps - 1 - jt;
+                    if (p - back < 0) continue;
+                    float v = 0.0f;
+                    if (t - back >= begin) v = a.src[static_cast<int64_t>(t - back) * a.ld + c];
+                    else if (slot_ok) v = ring[static_cast<int64_t>((p - back) % taps) * C + c];
+                    acc = fmaf(a.cw[static_cast<int64_t>(jt) * C + c], v, acc);
+                }
             }
-            x[q] = acc * gd_sigmoid(acc);
-            ss = fmaf(x[q], x[q], ss);
+            x[tt][q] = i < width ? acc * gd_sigmoid(acc) : 0.0f;
         }
     }
-    float f = 1.0f;
-    if (!is_v) f = 1.0f / sqrtf(wave_sum(ss) + a.key_eps) * (unit < a.G ? a.q_scale : 1.0f);
-    float* o = a.prep + static_cast<int64_t>(t) * (C + 2 * a.H);
 #pragma unroll
-    for (int q = 0; q < kGdMax / kWave; ++q) {
-        const int i = lane + q * kWave;
-        if (i < width) o[c0 + i] = x[q] * f;
+    for (int tt = 0; tt < kGdTokens; ++tt) {
+        if (t0 + tt >= a.n) break;
+        float f = 1.0f;
+        if (!is_v) {
+            float ss = 0.0f;
+#pragma unroll
+            for (int q = 0; q < NQ; ++q) ss = fmaf(x[tt][q], x[tt][q], ss);
+            f = 1.0f / sqrtf(wave_sum(ss) + a.key_eps) * (unit < a.G ? a.q_scale : 1.0f);
+        }
+        float* o = a.prep + static_cast<int64_t>(t0 + tt) * pld;
+#pragma unroll
+        for (int q = 0; q < NQ; ++q) {
+            const int i = lane + q * kWave;
+            if (i < width) o[c0 + i] = x[tt][q] * f;
+        }
     }
-    if (is_v && lane < 2) {
-        const int h = unit - 2 * a.G;
+    if (is_v && lane < 2 * kGdTokens && t0 + lane / 2 < a.n) {  // decay and rate of the head, a token two lanes
+        const int h = unit - 2 * a.G, t = t0 + lane / 2;
         const float* row = a.src + static_cast<int64_t>(t) * a.ld;
-        if (lane == 0) o[C + h] = expf(-expf(a.a_log[h]) * gd_softplus(row[a.a_off + h] + a.dt_bias[h]));
-        else o[C + a.H + h] = gd_sigmoid(row[a.b_off + h]);
+        float* o = a.prep + static_cast<int64_t>(t) * pld + C + h;
+        if (lane % 2 == 0) o[0] = expf(-expf(a.a_log[h]) * gd_softplus(row[a.a_off + h] + a.dt_bias[h]));
+        else o[a.H] = gd_sigmoid(row[a.b_off + h]);
     }
 }
 
@@ -259,7 +294,7 @@ struct GdSingleArgs {
     int H, G, D, V;
 };
 
-template <typename OutT, int REG>
+template <typename OutT, int REG, int TAPS>
 __global__ void __launch_bounds__(kDeltaWaves * kWave)
 gated_delta_single_kernel(GdSingleArgs a) {
     constexpr int DP = 4 * REG, COLS = kDeltaWaves * kDeltaCols;
@@ -267,8 +302,8 @@ gated_delta_single_kernel(GdSingleArgs a) {
     __shared__ float v_s[kGdMax], o_s[kGdMax], gb_s[2], red[kDeltaWaves];
     const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave;
     const int h = blockIdx.x % a.H, s = blockIdx.x / a.H;
-    const int t = a.seq_starts[s];
-    if (a.seq_starts[s + 1] - t != 1) return;  // (the host sends steps of single tokens only)
+    const int t = s;  // (the host sends steps of single tokens only: as many rows as requests)
+    if (a.seq_starts[s] != s || a.seq_starts[s + 1] != s + 1) return;
     const int D = a.D, V = a.V, H = a.H, GD = a.G * D, C = 2 * GD + H * V;
     const int per_k = H / a.G, hk = h / per_k;
     const int p = a.positions[t], slot = a.state_slots[s];
@@ -292,7 +327,9 @@ gated_delta_single_kernel(GdSingleArgs a) {
         // a wave a vector: k, q, v
         const int width = wave == 2 ? V : D, pad = wave == 2 ? V : DP;
         const int c0 = wave == 0 ? GD + hk * D : wave == 1 ? hk * D : 2 * GD + h * V;
-        const bool writes = slot_ok && a.taps > 1 && (wave == 2 || h % per_k == 0);
+        const int taps = TAPS > 0 ? TAPS : a.taps;
+        const int here = p % taps;  // this row's place in the ring
+        const bool writes = slot_ok && taps > 1 && (wave == 2 || h % per_k == 0);
         float x[kGdMax / kWave];
         float ss = 0.0f;
 #pragma unroll
@@ -303,15 +340,28 @@ gated_delta_single_kernel(GdSingleArgs a) {
                 const int c = c0 + i;
                 const float now = row[c];
                 float acc = 0.0f;
-                for (int jt = 0; jt < a.taps - 1; ++jt) {
-                    const int back = a.taps - 1 - jt;
-                    const float before = ring[static_cast<int64_t>((p - back + a.taps) % a.taps) * C + c];
-                    acc = fmaf(a.cw[static_cast<int64_t>(jt) * C + c], slot_ok && p - back >= 0 ? before : 0.0f, acc);
+                auto place = [&](int back) { return here - back + (here < back ? taps : 0); };
+                if constexpr (TAPS > 0) {
+                    // all of a channel's inputs and weights are asked for together
+                    float before[TAPS], w[TAPS];
+#pragma unroll
+                    for (int jt = 0; jt < TAPS - 1; ++jt) before[jt] = ring[static_cast<int64_t>(place(TAPS - 1 - jt)) * C + c];
+#pragma unroll
+                    for (int jt = 0; jt < TAPS; ++jt) w[jt] = a.cw[static_cast<int64_t>(jt) * C + c];
+#pragma unroll
+                    for (int jt = 0; jt < TAPS - 1; ++jt) acc = fmaf(w[jt], slot_ok && p - (TAPS - 1 - jt) >= 0 ? before[jt] : 0.0f, acc);
+                    acc = fmaf(w[TAPS - 1], now, acc);
+                } else {
+                    for (int jt = 0; jt < taps - 1; ++jt) {
+                        const int back = taps - 1 - jt;
+                        const float before = ring[static_cast<int64_t>(place(back)) * C + c];
+                        acc = fmaf(a.cw[static_cast<int64_t>(jt) * C + c], slot_ok && p - back >= 0 ? before : 0.0f, acc);
+                    }
+                    acc = fmaf(a.cw[static_cast<int64_t>(taps - 1) * C + c], now, acc);
                 }
-                acc = fmaf(a.cw[static_cast<int64_t>(a.taps - 1) * C + c], now, acc);
                 x[q] = acc * gd_sigmoid(acc);
                 ss = fmaf(x[q], x[q], ss);
-                if (writes) ring[static_cast<int64_t>(p % a.taps) * C + c] = now;
+                if (writes) ring[static_cast<int64_t>(here) * C + c] = now;
             }
         }
         float f = 1.0f;
@@ -394,9 +444,13 @@ extern "C" int liyab_gated_delta_prepare(float* prep, const float* src, int64_t 
     if (n == 0) return 0;
     const GdPrepareArgs a{prep, src, ld, cw, taps, ring, state_stride, n_slots, a_log, dt_bias, b_off, a_off, key_eps, q_scale,
                           tok_seq, positions, seq_starts, state_slots, n, H, G, D, V};
-    const int64_t items = static_cast<int64_t>(n) * (2 * G + H);
+    const int64_t items = static_cast<int64_t>((n + kGdTokens - 1) / kGdTokens) * (2 * G + H);
     LIYAB_REQUIRE(items < (int64_t(1) << 31) - 4, "gated_delta_prepare: too many tokens");
-    gated_delta_prepare_kernel<<<static_cast<unsigned>((items + 3) / 4), 256, 0, stream>>>(a);
+    const unsigned grid = static_cast<unsigned>((items + 3) / 4);
+    if (taps == 4) gated_delta_prepare_kernel<4><<<grid, 256, 0, stream>>>(a);
+    else if (taps == 3) gated_delta_prepare_kernel<3><<<grid, 256, 0, stream>>>(a);
+    else if (taps == 2) gated_delta_prepare_kernel<2><<<grid, 256, 0, stream>>>(a);
+    else gated_delta_prepare_kernel<0><<<grid, 256, 0, stream>>>(a);
     return check_launch("gated_delta_prepare");
 }
 
@@ -429,7 +483,7 @@ extern "C" int liyab_gated_delta_scan(float* out, const float* prep, const float
         p.phase = 1;
         walk(p, max_segs, false);
         const DeltaSegments segs{state, state_stride, n_slots, seq_starts, positions, state_slots, n_seqs, H, D, V, seg_tokens};
-        delta_combine_kernel<<<dim3(n_seqs, H, (V + kDeltaCols - 1) / kDeltaCols), 256, 0, stream>>>(segs, seg_state, seg_trans, seg_start);
+        combine_segments(segs, seg_state, seg_trans, seg_start, stream);
         p.phase = 3;
         walk(p, max_segs, true);
         return check_launch("gated_delta_scan");
@@ -454,10 +508,15 @@ extern "C" int liyab_gated_delta_single(void* out, int out_dtype, const float* s
     constexpr int T = kDeltaWaves * kWave;
     auto run = [&](auto zero) {
         using O = decltype(zero);
-        if (D <= 32) gated_delta_single_kernel<O, 8><<<grid, T, 0, stream>>>(a);
-        else if (D <= 64) gated_delta_single_kernel<O, 16><<<grid, T, 0, stream>>>(a);
-        else if (D <= 128) gated_delta_single_kernel<O, 32><<<grid, T, 0, stream>>>(a);
-        else gated_delta_single_kernel<O, 64><<<grid, T, 0, stream>>>(a);
+        auto sized = [&](auto nt) {
+            constexpr int N = decltype(nt)::value;
+            if (D <= 32) gated_delta_single_kernel<O, 8, N><<<grid, T, 0, stream>>>(a);
+            else if (D <= 64) gated_delta_single_kernel<O, 16, N><<<grid, T, 0, stream>>>(a);
+            else if (D <= 128) gated_delta_single_kernel<O, 32, N><<<grid, T, 0, stream>>>(a);
+            else gated_delta_single_kernel<O, 64, N><<<grid, T, 0, stream>>>(a);
+        };
+        if (taps == 4) sized(std::integral_constant<int, 4>{});
+        else sized(std::integral_constant<int, 0>{});
     };
     if (out_dtype == kF32) run(float{});
     else run(bf16_t{});

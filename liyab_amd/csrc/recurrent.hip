@@ -516,8 +516,8 @@ gla_single_kernel(GlaSingleArgs a) {
     __shared__ float red[4];
     const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave;
     const int h = blockIdx.x % a.H, s = blockIdx.x / a.H;
-    const int t = a.seq_starts[s];
-    if (a.seq_starts[s + 1] - t != 1) return;  // (the host sends steps of single tokens only)
+    const int t = s;  // (the host sends steps of single tokens only: as many rows as requests)
+    if (a.seq_starts[s] != s || a.seq_starts[s + 1] != s + 1) return;
     const int R = a.R, C = a.C;
     const int slot = a.state_slots[s];
     const bool slot_ok = slot >= 0 && slot < a.n_slots;
@@ -538,9 +538,19 @@ gla_single_kernel(GlaSingleArgs a) {
         const bool in = i < R;
         const int64_t at = static_cast<int64_t>(t) * a.ld + h * R + (in ? i : 0);
         float z = a.bias[h * R + (in ? i : 0)];
-        for (int r = 0; r < a.rank; ++r)
-            z = fmaf(a.w2t[static_cast<int64_t>(r) * a.H * R + h * R + (in ? i : 0)], a.low[static_cast<int64_t>(t) * a.ldl + r], z);
         const float k = a.k[at], q = a.q[at];
+        constexpr int kAhead = 16;  // weights asked for together
+        for (int r0 = 0; r0 < a.rank; r0 += kAhead) {
+            float w[kAhead], l[kAhead];
+#pragma unroll
+            for (int e = 0; e < kAhead; ++e) {
+                const int r = min(r0 + e, a.rank - 1);
+                w[e] = a.w2t[static_cast<int64_t>(r) * a.H * R + h * R + (in ? i : 0)];
+                l[e] = a.low[static_cast<int64_t>(t) * a.ldl + r];
+            }
+#pragma unroll
+            for (int e = 0; e < kAhead; ++e) z = r0 + e < a.rank ? fmaf(w[e], l[e], z) : z;
+        }
         vec[i] = in ? gla_decay_of(z, a.inv_tau) : 0.0f;
         vec[RP + i] = in ? k : 0.0f;
         vec[2 * RP + i] = in ? q * a.q_scale : 0.0f;
