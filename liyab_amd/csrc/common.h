@@ -72,6 +72,14 @@ __device__ __forceinline__ void lds_barrier() {
     asm volatile("" ::: "memory");
 }
 
+// Loaded values as the compiler has to hold them: what follows may not be drawn into the loads. Without it a choice such as
+// `inside ? loaded : 0` turns into a branch around the load, and each load is waited for before the next one is asked for.
+template <int N>
+__device__ __forceinline__ void settle_loads(float (&v)[N]) {
+#pragma unroll
+    for (int i = 0; i < N; ++i) asm volatile("" : "+v"(v[i]));
+}
+
 // Sums and maxima over the 64 lanes of a wave, the same bits in every lane. Within a row of 16
 // lanes the partners come through the lanes' own data path (DPP: neighbours in a quad, the other
 // pair of the quad, the other quad of eight, the other eight of the row: a few cycles each);

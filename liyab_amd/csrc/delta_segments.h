@@ -188,25 +188,22 @@ delta_combine_mfma_kernel(DeltaSegments a, const float* __restrict__ seg_z, cons
             }
         } else {
 #pragma unroll
-            for (int q = 0; q < 16; ++q) {
-                const float v = P[min(16 * grp + q, D - 1)];
-                pp[q] = row_in && 16 * grp + q < D ? v : 0.0f;
-            }
+            for (int q = 0; q < 16; ++q) pp[q] = P[min(16 * grp + q, D - 1)];
         }
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            const float v = Z[static_cast<int64_t>(min(row_s + r, D - 1)) * V + jc];
-            zz[r] = row_s + r < D && j < V ? v : 0.0f;
-        }
+        for (int r = 0; r < 4; ++r) zz[r] = Z[static_cast<int64_t>(min(row_s + r, D - 1)) * V + jc];
     };
+    // (entries past the matrix are made zeros where they are used: a choice beside a load would wait for that load alone)
+    auto row_or_zero = [&](float v, int r) { return WHOLE || row_s + r < D ? v : 0.0f; };
+    auto p_or_zero = [&](float v, int q) { return WHOLE || (row_in && 16 * grp + q < D) ? v : 0.0f; };
 #pragma unroll
     for (int u = 0; u < kCombDepth; ++u) fetch(u, p[u], z[u]);
     float S[4];
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-        const float v = S0[static_cast<int64_t>(min(row_s + r, D - 1)) * V + jc];
-        S[r] = from_slot && row_s + r < D && j < V ? v : 0.0f;
-    }
+    for (int r = 0; r < 4; ++r) S[r] = S0[static_cast<int64_t>(min(row_s + r, D - 1)) * V + jc];
+    settle_loads(S);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) S[r] = from_slot && row_s + r < D ? S[r] : 0.0f;  // (columns past the last one meet no other and are not kept)
     for (int gb = 0; gb < n_seg; gb += kCombDepth) {
 #pragma unroll
         for (int u = 0; u < kCombDepth; ++u) {
@@ -226,11 +223,11 @@ delta_combine_mfma_kernel(DeltaSegments a, const float* __restrict__ seg_z, cons
             float b[16];
 #pragma unroll
             for (int q = 0; q < 16; ++q) b[q] = buf[grp * kGroup + q * 16 + li];
-            comb_f32x4 acc0 = {z[u][0], z[u][1], z[u][2], z[u][3]}, acc1 = {0.0f, 0.0f, 0.0f, 0.0f};
+            comb_f32x4 acc0 = {row_or_zero(z[u][0], 0), row_or_zero(z[u][1], 1), row_or_zero(z[u][2], 2), row_or_zero(z[u][3], 3)}, acc1 = {0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll
             for (int q = 0; q < 16; q += 2) {
-                acc0 = __builtin_amdgcn_mfma_f32_16x16x4f32(p[u][q], b[q], acc0, 0, 0, 0);
-                acc1 = __builtin_amdgcn_mfma_f32_16x16x4f32(p[u][q + 1], b[q + 1], acc1, 0, 0, 0);
+                acc0 = __builtin_amdgcn_mfma_f32_16x16x4f32(p_or_zero(p[u][q], q), b[q], acc0, 0, 0, 0);
+                acc1 = __builtin_amdgcn_mfma_f32_16x16x4f32(p_or_zero(p[u][q + 1], q + 1), b[q + 1], acc1, 0, 0, 0);
             }
 #pragma unroll
             for (int r = 0; r < 4; ++r) S[r] = acc0[r] + acc1[r];

@@ -300,13 +300,13 @@ gated_delta_single_kernel(GdSingleArgs a) {
     constexpr int DP = 4 * REG, COLS = kDeltaWaves * kDeltaCols;
     __shared__ __attribute__((aligned(16))) float k_s[DP], q_s[DP];
     __shared__ float v_s[kGdMax], o_s[kGdMax], gb_s[2], red[kDeltaWaves];
-    const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave;
+    const int tid = threadIdx.x, lane = tid % kWave, wave = __builtin_amdgcn_readfirstlane(tid / kWave);
     const int h = blockIdx.x % a.H, s = blockIdx.x / a.H;
     const int t = s;  // (the host sends steps of single tokens only: as many rows as requests)
+    const int p = a.positions[t], slot = a.state_slots[s];
     if (a.seq_starts[s] != s || a.seq_starts[s + 1] != s + 1) return;
     const int D = a.D, V = a.V, H = a.H, GD = a.G * D, C = 2 * GD + H * V;
     const int per_k = H / a.G, hk = h / per_k;
-    const int p = a.positions[t], slot = a.state_slots[s];
     const bool slot_ok = slot >= 0 && slot < a.n_slots;
     const bool old = slot_ok && p > 0;
     float* base = a.state + static_cast<int64_t>(slot_ok ? slot : 0) * a.state_stride;
@@ -315,14 +315,18 @@ gated_delta_single_kernel(GdSingleArgs a) {
     const float* row = a.src + static_cast<int64_t>(t) * a.ld;
     const int rb = lane % kDeltaSplit, i0 = rb * REG, jl = wave * kDeltaCols + lane / kDeltaSplit;
     float S[REG];
-    auto load = [&](int j) {
+    auto load = [&](int j) {  // places outside the matrix read one inside it, and are zeros after settle()
 #pragma unroll
-        for (int ii = 0; ii < REG; ++ii) {
-            const float val = Sg[static_cast<int64_t>(min(i0 + ii, D - 1)) * V + min(j, V - 1)];
-            S[ii] = (i0 + ii < D && j < V && old) ? val : 0.0f;
-        }
+        for (int ii = 0; ii < REG; ++ii) S[ii] = Sg[static_cast<int64_t>(min(i0 + ii, D - 1)) * V + min(j, V - 1)];
     };
-    load(jl);  // the first block of columns is on its way while the vectors are made
+    auto settle = [&](int j) {
+        settle_loads(S);
+#pragma unroll
+        for (int ii = 0; ii < REG; ++ii) S[ii] = (i0 + ii < D && j < V && old) ? S[ii] : 0.0f;
+    };
+    // The gate's logits and the norm's weights, which the last lines need, are asked for first, then what the vectors are made of, then
+    // the first block of columns: it is on its way while the vectors are made.
+    const float z = row[a.g_off + h * V + min(tid, V - 1)], norm_w = a.norm_w[min(tid, V - 1)];
     if (wave < 3) {
         // a wave a vector: k, q, v
         const int width = wave == 2 ? V : D, pad = wave == 2 ? V : DP;
@@ -330,39 +334,43 @@ gated_delta_single_kernel(GdSingleArgs a) {
         const int taps = TAPS > 0 ? TAPS : a.taps;
         const int here = p % taps;  // this row's place in the ring
         const bool writes = slot_ok && taps > 1 && (wave == 2 || h % per_k == 0);
-        float x[kGdMax / kWave];
+        auto place = [&](int back) { return here - back + (here < back ? taps : 0); };
+        constexpr int NQ = kGdMax / kWave;
+        float x[NQ];
+#pragma unroll
+        for (int q = 0; q < NQ; ++q) x[q] = 0.0f;
         float ss = 0.0f;
 #pragma unroll
-        for (int q = 0; q < kGdMax / kWave; ++q) {
-            const int i = lane + q * kWave;
-            x[q] = 0.0f;
-            if (i < width) {
-                const int c = c0 + i;
-                const float now = row[c];
-                float acc = 0.0f;
-                auto place = [&](int back) { return here - back + (here < back ? taps : 0); };
-                if constexpr (TAPS > 0) {
-                    // all of a channel's inputs and weights are asked for together
-                    float before[TAPS], w[TAPS];
+        for (int q = 0; q < NQ; ++q) {
+            if (q * kWave >= width) break;  // (the same for the whole wave)
+            const int i = lane + q * kWave, c = c0 + min(i, width - 1);
+            const float now = row[c];
+            float acc = 0.0f;
+            if constexpr (TAPS > 0) {
+                // all of a channel's inputs and weights are asked for together
+                float before[TAPS], w[TAPS];  // (the last input is this row's)
+                before[TAPS - 1] = now;
 #pragma unroll
-                    for (int jt = 0; jt < TAPS - 1; ++jt) before[jt] = ring[static_cast<int64_t>(place(TAPS - 1 - jt)) * C + c];
+                for (int jt = 0; jt < TAPS - 1; ++jt) before[jt] = ring[static_cast<int64_t>(place(TAPS - 1 - jt)) * C + c];
 #pragma unroll
-                    for (int jt = 0; jt < TAPS; ++jt) w[jt] = a.cw[static_cast<int64_t>(jt) * C + c];
+                for (int jt = 0; jt < TAPS; ++jt) w[jt] = a.cw[static_cast<int64_t>(jt) * C + c];
+                if (q == 0) load(jl);
+                settle_loads(before);
+                settle_loads(w);
 #pragma unroll
-                    for (int jt = 0; jt < TAPS - 1; ++jt) acc = fmaf(w[jt], slot_ok && p - (TAPS - 1 - jt) >= 0 ? before[jt] : 0.0f, acc);
-                    acc = fmaf(w[TAPS - 1], now, acc);
-                } else {
-                    for (int jt = 0; jt < taps - 1; ++jt) {
-                        const int back = taps - 1 - jt;
-                        const float before = ring[static_cast<int64_t>(place(back)) * C + c];
-                        acc = fmaf(a.cw[static_cast<int64_t>(jt) * C + c], slot_ok && p - back >= 0 ? before : 0.0f, acc);
-                    }
-                    acc = fmaf(a.cw[static_cast<int64_t>(taps - 1) * C + c], now, acc);
+                for (int jt = 0; jt < TAPS; ++jt) acc = fmaf(w[jt], (slot_ok && p - (TAPS - 1 - jt) >= 0) || jt == TAPS - 1 ? before[jt] : 0.0f, acc);
+            } else {
+                if (q == 0) load(jl);
+                for (int jt = 0; jt < taps - 1; ++jt) {
+                    const int back = taps - 1 - jt;
+                    const float before = ring[static_cast<int64_t>(place(back)) * C + c];
+                    acc = fmaf(a.cw[static_cast<int64_t>(jt) * C + c], slot_ok && p - back >= 0 ? before : 0.0f, acc);
                 }
-                x[q] = acc * gd_sigmoid(acc);
-                ss = fmaf(x[q], x[q], ss);
-                if (writes) ring[static_cast<int64_t>(here) * C + c] = now;
+                acc = fmaf(a.cw[static_cast<int64_t>(taps - 1) * C + c], now, acc);
             }
+            x[q] = i < width ? acc * gd_sigmoid(acc) : 0.0f;
+            ss = fmaf(x[q], x[q], ss);
+            if (writes && i < width) ring[static_cast<int64_t>(here) * C + c] = now;
         }
         float f = 1.0f;
         if (wave < 2) f = 1.0f / sqrtf(wave_sum(ss) + a.key_eps) * (wave == 1 ? a.q_scale : 1.0f);
@@ -372,16 +380,21 @@ gated_delta_single_kernel(GdSingleArgs a) {
             const int i = lane + q * kWave;
             if (i < pad) dst[i] = x[q] * f;  // (zeros behind a key's or query's last entry)
         }
-    } else if (lane == 0) {
-        gb_s[0] = expf(-expf(a.a_log[h]) * gd_softplus(row[a.a_off + h] + a.dt_bias[h]));
-        gb_s[1] = gd_sigmoid(row[a.b_off + h]);
+    } else {
+        const float decay_in = row[a.a_off + h], rate_in = row[a.b_off + h], a_log = a.a_log[h], dt_bias = a.dt_bias[h];
+        load(jl);
+        if (lane == 0) {
+            gb_s[0] = expf(-expf(a_log) * gd_softplus(decay_in + dt_bias));
+            gb_s[1] = gd_sigmoid(rate_in);
+        }
     }
-    __syncthreads();
+    lds_barrier();  // (the state's columns may stay on their way, the ring's new row too)
     const float g = gb_s[0], beta = gb_s[1];
     float ss = 0.0f;
     for (int c0 = 0; c0 < V; c0 += COLS) {
         const int j = c0 + jl;
         if (c0 > 0) load(j);
+        settle(j);
         f32x4_t seen4 = {0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll
         for (int q4 = 0; q4 < REG / 4; ++q4) {
@@ -414,12 +427,9 @@ gated_delta_single_kernel(GdSingleArgs a) {
     }
     ss = wave_sum(ss);
     if (lane == 0) red[wave] = ss;
-    __syncthreads();
+    lds_barrier();
     const float rinv = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / static_cast<float>(V) + a.eps);
-    if (tid < V) {
-        const float z = row[a.g_off + h * V + tid];
-        static_cast<OutT*>(a.out)[(static_cast<int64_t>(t) * H + h) * V + tid] = from_float<OutT>(o_s[tid] * rinv * a.norm_w[tid] * z * gd_sigmoid(z));
-    }
+    if (tid < V) static_cast<OutT*>(a.out)[(static_cast<int64_t>(t) * H + h) * V + tid] = from_float<OutT>(o_s[tid] * rinv * norm_w * z * gd_sigmoid(z));
 }
 
 }  // namespace liyab
