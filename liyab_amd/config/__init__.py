@@ -30,3 +30,4 @@ from .mofulix import MofulixConfig  # noqa: F401  (registers itself)
 from .dopilorn import DopilornConfig  # noqa: F401  (registers itself)
 from .larulorn import LarulornConfig  # noqa: F401  (registers itself)
 from .lolulorn import LolulornConfig  # noqa: F401  (registers itself)
+from .lafanex import LafanexConfig  # noqa: F401  (registers itself)

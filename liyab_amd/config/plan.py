@@ -135,19 +135,28 @@ class RoutedFFNSpec:
     weights are the chosen scores divided by their sum. `shared_inner` > 0: one more expert of the same form
     and that inner width runs for every token with weight one (tensors shared_up, shared_down, and shared_gate
     if gated). `scores` "logistic": s = sigmoid(z); the choice goes by s + correction (tensor `correction`, optional), with `groups` a
-    group's score is the sum of its two largest such values, and the weights are the chosen s as they are."""
+    group's score is the sum of its two largest such values, and the weights are the chosen s as they are. `scores` "softmax_all": the same with
+    s = softmax(z) over all outputs and weights `scale` * s. `identity` (with these two): the router has that many outputs more, behind the
+    experts'; one that is chosen gives the unit's input itself, times its weight. Activation "clamped_glu" (gated): g = min(gate h, limit), u = clamp(up
+    h, -limit, limit), down(g * sigmoid(slope * g) * (u + shift)) with `clamp` = (limit, slope, shift), the shared expert's `shared_clamp`.
+    `shared_weighed`: the shared expert's result times sigmoid(w h), one number a token (tensor shared_weight [1, width])."""
 
     kind: str  # "routed_ffn"
     width: int
     inner: int
     n_experts: int
     top: int
-    activation: str  # "silu" | "relu2"
+    activation: str  # "silu" | "relu2" | "clamped_glu"
     tensors: dict = field(default_factory=dict)  # router, router_bias, and per expert e: ("gate", e), ("up", e), ("down", e)
     gated: bool = True
     groups: Optional[tuple] = None  # (count, keep)
     shared_inner: int = 0
-    scores: str = "softmax"  # | "logistic"
+    scores: str = "softmax"  # | "logistic" | "softmax_all"
+    identity: int = 0
+    scale: float = 1.0
+    clamp: Optional[tuple] = None  # (limit, slope, shift)
+    shared_clamp: Optional[tuple] = None
+    shared_weighed: bool = False
 
 
 @dataclass(frozen=True)
@@ -159,6 +168,17 @@ class CausalConvSpec:
     width: int
     taps: int
     tensors: dict = field(default_factory=dict)  # "weight" [width, taps]
+
+
+@dataclass(frozen=True)
+class StreamConnectionSpec:
+    """How a sublayer meets the residual stream where that is `streams` copies x_1 .. x_s (all the embedding's output at the start; the
+    final norm reads their sum): the sublayer's norm reads sum_s take[s] x_s, and with the sublayer's result y, x_t <- sum_s mix[s, t] x_s +
+    give[t] y, every stream from the old ones."""
+
+    kind: str  # "stream_connection"
+    streams: int
+    tensors: dict = field(default_factory=dict)  # "take" [streams], "give" [streams], "mix" [streams, streams] ([from, to])
 
 
 @dataclass(frozen=True)
@@ -201,7 +221,8 @@ class ScoredAttentionSpec:
     the three projections (`biased`), a learned logit a head that joins the softmax's denominator with no key and no value
     (`sink`), values shared between layers (`value_mix`: "first" = this layer's values, as projected, are kept for the later
     layers of the same step; "later" = v <- (1 - lam) v + lam v_first with the learned scalar `vmix`, and the mixed values are
-    what is cached). `qk_norm_rows`: a root-mean-square norm of a token's whole queries (and whole keys) before they are heads, a
+    what is cached). `qk_norm_weights` False: `qk_norm` without weights, which a turn of the pairs leaves as it is (it may stand before or
+    behind the rotary encoding). `sink_value`: a fixed logit in every head's denominator instead of a learned one. `qk_norm_rows`: a root-mean-square norm of a token's whole queries (and whole keys) before they are heads, a
     weight an entry (tensors q_norm, k_norm). With a `window`, positions below `keep_first` stay visible. `kv_shared`: the keys and
     values are another layer's, as its cache holds them (the run order's `cache_of`, writes_cache False); the layer has queries only."""
 
@@ -229,6 +250,8 @@ class ScoredAttentionSpec:
     qk_norm_rows: bool = False
     keep_first: int = 0
     kv_shared: bool = False
+    qk_norm_weights: bool = True
+    sink_value: Optional[float] = None
 
 
 @dataclass(frozen=True)
@@ -371,6 +394,22 @@ class GatedLinearAttentionSpec:
 
 
 @dataclass(frozen=True)
+class SelectiveScanSpec:
+    """A mixer with a state of its own for every channel and state number: [x | z] = Win h, `inner` wide each; x <- silu(conv(x) + bias) a
+    channel over time (`taps` inputs; the last ones are part of a request's state); [low | B | C] = Wx x, `dt_rank` and twice `n_state` wide; dt =
+    softplus(Wdt low + bias) a channel; S[c, n] <- exp(-dt_c exp(A_log[c, n])) S[c, n] + dt_c x_c B_n from S = 0; y_c = sum_n S[c, n] C_n + D_c x_c; the
+    output projection of y * silu(z)."""
+
+    kind: str  # "selective_scan"
+    width: int
+    inner: int
+    n_state: int
+    dt_rank: int
+    taps: int
+    tensors: dict = field(default_factory=dict)  # in, conv, conv_bias, x, dt, dt_bias, A_log, D, out
+
+
+@dataclass(frozen=True)
 class GatedFFNSpec:
     """A gated feed-forward, down(act(gate h) * (up h)), act "silu" or "gelu_tanh"."""
 
@@ -442,6 +481,8 @@ class LayerSpec:
     followed by a convolution over time of its own (`input_conv`, `ffn_conv`: h <- h + conv(h); optional).
     arrangement "sandwich": x += post_norm_mixer(mixer(norm_mixer(x))); x += post_norm_ffn(ffn(norm_ffn(x))): a norm before and
     a norm behind each sublayer.
+    arrangement "streams": "pre_norm" over several residual streams, each sublayer connected to them as `connect_mixer` and `connect_ffn` say
+    (None: one stream, a plain sum). `ModelPlan.streams` says how many there are.
     `entry`: what is done to the stream before the layer runs (a spec of the entry registry), or None.
     """
 
@@ -457,6 +498,8 @@ class LayerSpec:
     entry: Any = None
     post_norm_mixer: Any = None
     post_norm_ffn: Any = None
+    connect_mixer: Any = None
+    connect_ffn: Any = None
 
 
 @dataclass(frozen=True)
@@ -501,3 +544,5 @@ class ModelPlan:
     # prefixes that may stand before every tensor name in a file
     name_prefixes: Sequence[str] = ("",)
     eos_token_id: Optional[int] = None
+    # copies of the residual stream (every layer's arrangement is then "streams"); 0: one, as any other arrangement has it
+    streams: int = 0

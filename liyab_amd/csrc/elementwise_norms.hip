@@ -6,7 +6,7 @@
 //
 // liyab_glu_clamped: the inner rows of a gated feed-forward whose two halves are clamped before
 // they meet: g = min(G, limit), u = clamp(U, -limit, limit), y = g * sigmoid(slope * g) * (u + shift),
-// from one 32-bit product [G | U] a row.
+// from one 32-bit product [G | U] a row; with `gate`, a row's entries times sigmoid of its logit there (one number a row).
 //
 // liyab_glu: the inner rows of a plain gated feed-forward, y = act(G) * U with act = silu or the tanh form of gelu, from such a product.
 //
@@ -48,14 +48,16 @@ dyt_kernel(T* __restrict__ out, const float* __restrict__ x, const float* __rest
 
 template <typename T>
 __global__ void __launch_bounds__(EW_THREADS)
-glu_clamped_kernel(T* __restrict__ out, const float* __restrict__ gu, int64_t ld, int ff, float limit, float slope, float shift) {
+glu_clamped_kernel(T* __restrict__ out, const float* __restrict__ gu, int64_t ld, int ff, float limit, float slope, float shift,
+                   const float* __restrict__ gate, int64_t gate_stride) {
     const int t = blockIdx.y;
     const int i = blockIdx.x * EW_THREADS + threadIdx.x;
     if (i >= ff) return;
     const float* row = gu + static_cast<int64_t>(t) * ld;
     const float g = fminf(row[i], limit);
     const float u = fminf(fmaxf(row[ff + i], -limit), limit);
-    out[static_cast<int64_t>(t) * ff + i] = from_float<T>(g * logistic(slope * g) * (u + shift));
+    const float scale = gate != nullptr ? logistic(gate[t * gate_stride]) : 1.0f;
+    out[static_cast<int64_t>(t) * ff + i] = from_float<T>(g * logistic(slope * g) * (u + shift) * scale);
 }
 
 template <typename T>
@@ -148,14 +150,14 @@ extern "C" int liyab_dyt(void* out, int out_dtype, const float* x, const float* 
 }
 
 extern "C" int liyab_glu_clamped(void* out, int out_dtype, const float* gu, int64_t ld, int n, int ff, float limit, float slope, float shift,
-                                 hipStream_t stream) {
+                                 const float* gate, int64_t gate_stride, hipStream_t stream) {
     LIYAB_REQUIRE(out && gu, "glu_clamped: null pointer");
     LIYAB_REQUIRE(n >= 0 && n <= 65535 && ff > 0 && ld >= 2 * static_cast<int64_t>(ff), "glu_clamped: bad sizes");
     LIYAB_REQUIRE(limit > 0.0f, "glu_clamped: the limit must be positive");
     if (n == 0) return 0;
     dim3 grid((ff + EW_THREADS - 1) / EW_THREADS, n);
-    if (out_dtype == kF32) glu_clamped_kernel<float><<<grid, EW_THREADS, 0, stream>>>(static_cast<float*>(out), gu, ld, ff, limit, slope, shift);
-    else if (out_dtype == kBF16) glu_clamped_kernel<bf16_t><<<grid, EW_THREADS, 0, stream>>>(static_cast<bf16_t*>(out), gu, ld, ff, limit, slope, shift);
+    if (out_dtype == kF32) glu_clamped_kernel<float><<<grid, EW_THREADS, 0, stream>>>(static_cast<float*>(out), gu, ld, ff, limit, slope, shift, gate, gate_stride);
+    else if (out_dtype == kBF16) glu_clamped_kernel<bf16_t><<<grid, EW_THREADS, 0, stream>>>(static_cast<bf16_t*>(out), gu, ld, ff, limit, slope, shift, gate, gate_stride);
     else return fail(1, "glu_clamped: unknown dtype %d", out_dtype);
     return check_launch("glu_clamped");
 }

@@ -74,12 +74,12 @@ int liyab_latent_store(void* cache, int dtype, const void* src, int64_t src_stri
 int liyab_grouped_product(const void* a, int64_t lda, int a_div, int a_group_cols, const void* w0, const void* w1, int dtype, void* out,
                           int out_dtype, int64_t ldo, int out_group_cols, const int* rows_list, const int* tile_group, int n_tiles,
                           int block, int n_groups, const float* row_scale, const void* gate, int gate_dtype, int64_t gate_stride, int M, int N,
-                          int K, int act, int out_div, int out_extra, hipStream_t stream);
+                          int K, int act, int out_div, int out_extra, float limit, float slope, float shift, hipStream_t stream);
 int liyab_moe_route(const float* logits, int64_t ld, int n, int n_experts, int top, int* ids, float* weights, int mode, int n_groups, int keep,
-                    const float* correction, hipStream_t stream);
+                    const float* correction, float scale, int n_listed, int extra, hipStream_t stream);
 int liyab_moe_route_align(const float* logits, int64_t ld, int n, int n_experts, int top, int* ids, float* weights, int block,
                           int* rows_list, int* tile_group, int max_tiles, int mode, int n_groups, int keep, const float* correction,
-                          hipStream_t stream);
+                          float scale, int n_listed, int extra, hipStream_t stream);
 int liyab_moe_align(const int* ids, int n_entries, int n_experts, int block, int* rows_list, int* tile_group, int max_tiles,
                     hipStream_t stream);
 
@@ -96,7 +96,7 @@ int liyab_gate_rows(void* x, int dtype, int64_t ldx, const float* gate, int64_t 
 int liyab_dyt(void* out, int out_dtype, const float* x, const float* w, const float* b, const float* alpha, const int* rows, int n, int d,
               hipStream_t stream);
 int liyab_glu_clamped(void* out, int out_dtype, const float* gu, int64_t ld, int n, int ff, float limit, float slope, float shift,
-                      hipStream_t stream);
+                      const float* gate, int64_t gate_stride, hipStream_t stream);
 int liyab_glu(void* out, int out_dtype, const float* gu, int64_t ld, int n, int ff, int act, hipStream_t stream);
 int liyab_activate(void* out, int out_dtype, int64_t ldo, const float* in, int64_t ldi, int op, int n, int d, hipStream_t stream);
 int liyab_mean_norm_add(float* x, const float* a, const float* b, const float* wa, const float* wb, float eps, float weight, int n, int d,
@@ -125,7 +125,7 @@ int liyab_gla_single(void* out, int out_dtype, const float* q, const float* k, c
 int liyab_token_shift(void* out, int dtype, const void* h, const float* mu, int n_mix, const float* state, int64_t state_stride, int n_slots,
                       const int* tok_seq, const int* positions, const int* seq_starts, const int* state_slots, int n, int d,
                       hipStream_t stream);
-int liyab_conv_act(float* out, int64_t ldo, const float* in, int64_t ldi, const float* w, const float* bias, int taps, const float* state,
+int liyab_conv_act(void* out, int out_dtype, int64_t ldo, const float* in, int64_t ldi, const float* w, const float* bias, int taps, const float* state,
                    int64_t state_stride, int n_slots, const int* tok_seq, const int* positions, const int* seq_starts,
                    const int* state_slots, int n, int C, int act, hipStream_t stream);
 int liyab_gated_group_norm(void* out, int out_dtype, const float* y, int64_t ldy, const float* z, int64_t ldz, const float* w, float eps,
@@ -195,4 +195,15 @@ int liyab_lru_scan(void* out, int out_dtype, const float* z, int64_t ldz, const 
                    int64_t state_stride, int n_slots, const float* x, int64_t ldx, int taps, const int* seq_starts, const int* positions,
                    const int* state_slots, int n_seqs, int C, int blocks, int stretches, hipStream_t stream);
 
+int liyab_streams_update(float* x, const float* enter, const float* y, int n_sum, const int* ids, const float* weights, int n_ids, const void* h,
+                         const float* mix, const float* add, const float* in, const float* w, float eps, void* out, int out_dtype, const int* rows,
+                         int n, int S, int d, hipStream_t stream);
+int liyab_scan_steps(float* dt, const float* low, int64_t ldl, const void* w, int dtype, const float* bias, int n, int C, int rank, hipStream_t stream);
+int liyab_selective_scan(void* out, int dtype, const void* x, const float* dt, const float* bc, int64_t ldb, const float* z, int64_t ldz,
+                         const float* a2, const float* skip, float* state, int64_t state_stride, int n_slots, const float* raw, int64_t ldr, int places,
+                         const int* seq_starts, const int* positions, const int* state_slots, int n_seqs, int C, int N, int seg_tokens, int max_segs,
+                         float* seg_state, float* seg_dt, hipStream_t stream);
+int liyab_selective_single(void* out, int dtype, const void* x, const float* low, int64_t ldb, int rank, const void* wt, const float* bias, const float* z,
+                           int64_t ldz, const float* a2, const float* skip, float* state, int64_t state_stride, int n_slots, const float* raw, int64_t ldr,
+                           int places, const int* seq_starts, const int* positions, const int* state_slots, int n_seqs, int C, int N, hipStream_t stream);
 }  // extern "C"

@@ -9,6 +9,10 @@
 // mode 2: scores s = 1 / (1 + exp(-z)), the choice by c = s + correction (route_wave): a group's score is the sum of its two
 // largest c, only experts of the best groups, of those the `top` largest c; weights are the chosen s as they are. A wave routes a
 // token (its scores in LDS, an expert a lane), since every score costs an exponential.
+// mode 3: as mode 2 with scores s = softmax(z) over all outputs; weights are scale * s of the chosen ones.
+// Modes 2 and 3: outputs from `n_listed` on are identity experts, whose result is the token's own input: they get the id -1, so that no
+// list holds them, and whoever adds a token's rows up puts the input there. With `extra`, a token has one more entry behind its `top`: expert
+// n_listed, which every token takes, weighted sigmoid(z[E]) (a logit of its own behind the router's).
 //
 // liyab_moe_align: the entries listed by expert, each expert's stretch padded to whole tiles of
 // `block` places: rows_list [max_tiles * block] (an entry's number, -1 for an empty place) and
@@ -16,7 +20,7 @@
 // a bound that the step's sizes fix (entries / block + min(experts, entries), rounded up), so
 // that the products' grids do not depend on where the tokens went. One workgroup.
 //
-// liyab_moe_route_align: both in one launch, for steps of at most 1,024 tokens (mode 2: kWaveRouteTokens).
+// liyab_moe_route_align: both in one launch, for steps of at most 1,024 tokens (modes 2 and 3: kWaveRouteTokens).
 #include "common.h"
 #include "launchers.h"
 
@@ -117,10 +121,28 @@ constexpr int kWaveRouteTokens = 64;  // tokens a launch of one workgroup routes
 // What a wave's lanes wrote to LDS is there for its other lanes.
 __device__ __forceinline__ void wave_lds_order() { asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory"); }
 
-__device__ __forceinline__ void route_wave(const float* __restrict__ z, const float* __restrict__ correction, int E, int top, int n_groups, int keep,
-                                           int* __restrict__ ids, float* __restrict__ weights, float* c) {
-    const int lane = threadIdx.x % kWave;
-    for (int e = lane; e < E; e += kWave) c[e] = 1.0f / (1.0f + expf(-z[e])) + (correction != nullptr ? correction[e] : 0.0f);
+struct RouteArgs {
+    int mode, n_groups, keep;
+    const float* correction;
+    float scale;          // mode 3: on the weights
+    int n_listed, extra;  // modes 2 and 3: see the head of this file
+};
+
+__device__ __forceinline__ void route_wave(const float* __restrict__ z, const RouteArgs& ra, int E, int top, int* __restrict__ ids, float* __restrict__ weights,
+                                           float* c) {
+    const int lane = threadIdx.x % kWave, n_groups = ra.n_groups, keep = ra.keep;
+    const float* correction = ra.correction;
+    float largest = 0.0f, norm = 1.0f;  // mode 3: a score is exp(z - largest) * norm
+    if (ra.mode == 3) {
+        largest = -INFINITY;
+        for (int e = lane; e < E; e += kWave) largest = fmaxf(largest, z[e]);
+        largest = wave_max(largest);
+        float total = 0.0f;
+        for (int e = lane; e < E; e += kWave) total += expf(z[e] - largest);
+        norm = 1.0f / wave_sum(total);
+    }
+    auto score = [&](int e) { return ra.mode == 3 ? expf(z[e] - largest) * norm : 1.0f / (1.0f + expf(-z[e])); };
+    for (int e = lane; e < E; e += kWave) c[e] = score(e) + (correction != nullptr ? correction[e] : 0.0f);
     wave_lds_order();
     const int per = E / n_groups;
     uint64_t kept = ~uint64_t(0);
@@ -157,23 +179,26 @@ __device__ __forceinline__ void route_wave(const float* __restrict__ z, const fl
         wave_argmax(bv, bi);
         const int best = min(bi, E - 1);
         if (lane == 0) {
-            ids[k] = best;
-            weights[k] = 1.0f / (1.0f + expf(-z[best]));
+            ids[k] = best < ra.n_listed ? best : -1;
+            weights[k] = score(best) * ra.scale;
         }
         if (lane == best % kWave) c[best] = -INFINITY;
         wave_lds_order();
+    }
+    if (ra.extra && lane == 0) {
+        ids[top] = ra.n_listed;
+        weights[top] = 1.0f / (1.0f + expf(-z[E]));
     }
 }
 
 // a wave a token, four waves a workgroup
 __global__ void __launch_bounds__(256)
-moe_route_wave_kernel(const float* __restrict__ logits, int64_t ld, const float* __restrict__ correction, int n, int E, int top, int* __restrict__ ids,
-                      float* __restrict__ weights, int n_groups, int keep) {
+moe_route_wave_kernel(const float* __restrict__ logits, int64_t ld, RouteArgs ra, int n, int E, int top, int* __restrict__ ids, float* __restrict__ weights) {
     extern __shared__ int sh[];
     const int wave = threadIdx.x / kWave, t = blockIdx.x * 4 + wave;
     if (t >= n) return;
-    route_wave(logits + static_cast<int64_t>(t) * ld, correction, E, top, n_groups, keep, ids + static_cast<int64_t>(t) * top,
-               weights + static_cast<int64_t>(t) * top, reinterpret_cast<float*>(sh) + wave * E);
+    const int64_t at = static_cast<int64_t>(t) * (top + ra.extra);
+    route_wave(logits + static_cast<int64_t>(t) * ld, ra, E, top, ids + at, weights + at, reinterpret_cast<float*>(sh) + wave * E);
 }
 
 // mode 0: the largest logits, softmax over the chosen ones; mode 1: softmax over all, groups, weights by their sum
@@ -237,36 +262,40 @@ moe_align_kernel(const int* __restrict__ ids, int n_entries, int E, int block, i
 // Both in one launch for steps of at most 1,024 tokens: a thread routes a token, then the workgroup lists the entries.
 __global__ void __launch_bounds__(1024)
 moe_route_align_kernel(const float* __restrict__ logits, int64_t ld, int n, int E, int top, int* __restrict__ ids, float* __restrict__ weights,
-                       int block, int* __restrict__ rows_list, int* __restrict__ tile_group, int max_tiles, int mode, int n_groups, int keep,
-                       const float* __restrict__ correction) {
+                       int block, int* __restrict__ rows_list, int* __restrict__ tile_group, int max_tiles, RouteArgs ra) {
     extern __shared__ int sh[];
     const int t = threadIdx.x;
-    if (mode == 2) {  // a wave a token, sixteen at a time
+    if (ra.mode >= 2) {  // a wave a token, sixteen at a time
         const int wave = t / kWave;
-        for (int i = wave; i < n; i += 1024 / kWave)
-            route_wave(logits + static_cast<int64_t>(i) * ld, correction, E, top, n_groups, keep, ids + static_cast<int64_t>(i) * top,
-                       weights + static_cast<int64_t>(i) * top, reinterpret_cast<float*>(sh) + wave * E);
-    } else if (t < n) route_any(logits + static_cast<int64_t>(t) * ld, E, top, mode, n_groups, keep, ids + static_cast<int64_t>(t) * top, weights + static_cast<int64_t>(t) * top);
+        for (int i = wave; i < n; i += 1024 / kWave) {
+            const int64_t at = static_cast<int64_t>(i) * (top + ra.extra);
+            route_wave(logits + static_cast<int64_t>(i) * ld, ra, E, top, ids + at, weights + at, reinterpret_cast<float*>(sh) + wave * E);
+        }
+    } else if (t < n) route_any(logits + static_cast<int64_t>(t) * ld, E, top, ra.mode, ra.n_groups, ra.keep, ids + static_cast<int64_t>(t) * top, weights + static_cast<int64_t>(t) * top);
     __syncthreads();  // (the ids are read back by other threads of this workgroup)
-    align_entries(ids, n * top, E, block, rows_list, tile_group, max_tiles, sh);
+    align_entries(ids, n * (top + ra.extra), ra.n_listed + ra.extra, block, rows_list, tile_group, max_tiles, sh);
 }
 
 }  // namespace liyab
 
 using namespace liyab;
 
+// ids and weights: [n, top + extra]. n_listed, extra: see the head of this file (n_experts and 0 outside modes 2 and 3).
 extern "C" int liyab_moe_route(const float* logits, int64_t ld, int n, int n_experts, int top, int* ids, float* weights, int mode, int n_groups,
-                               int keep, const float* correction, hipStream_t stream) {
+                               int keep, const float* correction, float scale, int n_listed, int extra, hipStream_t stream) {
     LIYAB_REQUIRE(logits && ids && weights, "moe_route: null pointer");
-    LIYAB_REQUIRE(mode == 0 || ((mode == 1 || mode == 2) && n_groups >= 1 && n_groups <= kMaxGroups && n_experts % n_groups == 0 && keep >= 1 && keep <= n_groups &&
+    LIYAB_REQUIRE(mode == 0 || (mode >= 1 && mode <= 3 && n_groups >= 1 && n_groups <= kMaxGroups && n_experts % n_groups == 0 && keep >= 1 && keep <= n_groups &&
                                 top <= keep * (n_experts / n_groups)),
                   "moe_route: %d of %d groups of %d experts do not hold %d choices (at most %d groups)", keep, n_groups, n_experts, top, kMaxGroups);
     LIYAB_REQUIRE(n >= 0 && n_experts > 0 && top >= 1 && top <= n_experts && top <= kMaxTop && ld >= n_experts,
                   "moe_route: bad sizes n=%d experts=%d top=%d (at most %d choices a token)", n, n_experts, top, kMaxTop);
-    LIYAB_REQUIRE(mode != 2 || n_experts <= kMaxWaveExperts, "moe_route: %d experts; at most %d are taken in this mode", n_experts, kMaxWaveExperts);
+    LIYAB_REQUIRE(mode < 2 || n_experts <= kMaxWaveExperts, "moe_route: %d experts; at most %d are taken in this mode", n_experts, kMaxWaveExperts);
+    LIYAB_REQUIRE(n_listed >= 1 && n_listed <= n_experts && (extra == 0 || extra == 1) && (mode >= 2 || (n_listed == n_experts && extra == 0)) && ld >= n_experts + extra,
+                  "moe_route: %d listed of %d outputs, %d entries for every token do not go with this mode", n_listed, n_experts, extra);
     if (n == 0) return 0;
-    if (mode == 2) {
-        moe_route_wave_kernel<<<(n + 3) / 4, 256, 4 * n_experts * sizeof(float), stream>>>(logits, ld, correction, n, n_experts, top, ids, weights, n_groups, keep);
+    if (mode >= 2) {
+        const RouteArgs ra{mode, n_groups, keep, correction, scale, n_listed, extra};
+        moe_route_wave_kernel<<<(n + 3) / 4, 256, 4 * n_experts * sizeof(float), stream>>>(logits, ld, ra, n, n_experts, top, ids, weights);
         return check_launch("moe_route");
     }
     moe_route_kernel<<<(n + 255) / 256, 256, 0, stream>>>(logits, ld, n, n_experts, top, ids, weights, mode, n_groups, keep);
@@ -286,16 +315,17 @@ extern "C" int liyab_moe_align(const int* ids, int n_entries, int n_experts, int
 
 extern "C" int liyab_moe_route_align(const float* logits, int64_t ld, int n, int n_experts, int top, int* ids, float* weights, int block,
                                      int* rows_list, int* tile_group, int max_tiles, int mode, int n_groups, int keep, const float* correction,
-                                     hipStream_t stream) {
+                                     float scale, int n_listed, int extra, hipStream_t stream) {
     LIYAB_REQUIRE(n <= 1024, "moe_route_align: %d tokens; one workgroup routes at most 1,024 (moe_route and moe_align take more)", n);
-    if (const int rc = liyab_moe_route(logits, ld, 0, n_experts, top, ids, weights, mode, n_groups, keep, correction, stream)) return rc;                    // (the checks of both,
-    if (const int rc = liyab_moe_align(ids, 0, n_experts, block, rows_list, tile_group, max_tiles, stream)) return rc;    //  nothing launched)
-    LIYAB_REQUIRE(n >= 0 && static_cast<int64_t>(max_tiles) * block >= static_cast<int64_t>(n) * top + static_cast<int64_t>(n * top < n_experts ? n * top : n_experts) * (block - 1),
-                  "moe_route_align: %d tiles of %d places do not hold %d entries of %d experts", max_tiles, block, n * top, n_experts);
-    LIYAB_REQUIRE(mode != 2 || (n <= kWaveRouteTokens && n_experts <= 512), "moe_route_align: %d tokens of %d experts; mode 2 takes %d of 512 here", n, n_experts, kWaveRouteTokens);
+    if (const int rc = liyab_moe_route(logits, ld, 0, n_experts, top, ids, weights, mode, n_groups, keep, correction, scale, n_listed, extra, stream)) return rc;  // (the checks of both,
+    const int listed = n_listed + extra;
+    if (const int rc = liyab_moe_align(ids, 0, listed, block, rows_list, tile_group, max_tiles, stream)) return rc;    //  nothing launched)
+    LIYAB_REQUIRE(n >= 0 && static_cast<int64_t>(max_tiles) * block >= static_cast<int64_t>(n) * (top + extra) + static_cast<int64_t>(n * (top + extra) < listed ? n * (top + extra) : listed) * (block - 1),
+                  "moe_route_align: %d tiles of %d places do not hold %d entries of %d experts", max_tiles, block, n * (top + extra), listed);
+    LIYAB_REQUIRE(mode < 2 || (n <= kWaveRouteTokens && n_experts <= 512), "moe_route_align: %d tokens of %d experts; modes 2 and 3 take %d of 512 here", n, n_experts, kWaveRouteTokens);
     if (n == 0) return 0;
-    const size_t smem = sizeof(int) * (mode == 2 ? (1024 / kWave) * static_cast<size_t>(n_experts) + 1 : 2 * static_cast<size_t>(n_experts) + 1);  // (the scores; then the lists' counts)
-    moe_route_align_kernel<<<1, 1024, smem, stream>>>(logits, ld, n, n_experts, top, ids, weights, block, rows_list,
-                                                                                    tile_group, max_tiles, mode, n_groups, keep, correction);
+    const size_t smem = sizeof(int) * (mode >= 2 ? (1024 / kWave) * static_cast<size_t>(n_experts) + 4 : 2 * static_cast<size_t>(n_experts) + 1);  // (the scores; then the lists' counts)
+    const RouteArgs ra{mode, n_groups, keep, correction, scale, n_listed, extra};
+    moe_route_align_kernel<<<1, 1024, smem, stream>>>(logits, ld, n, n_experts, top, ids, weights, block, rows_list, tile_group, max_tiles, ra);
     return check_launch("moe_route_align");
 }

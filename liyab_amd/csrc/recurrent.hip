@@ -616,8 +616,9 @@ token_shift_kernel(T* __restrict__ out, const T* __restrict__ h, const float* __
     }
 }
 
+template <typename T>
 __global__ void __launch_bounds__(256)
-conv_act_kernel(float* __restrict__ out, int64_t ldo, const float* __restrict__ in, int64_t ldi, const float* __restrict__ w,
+conv_act_kernel(T* __restrict__ out, int64_t ldo, const float* __restrict__ in, int64_t ldi, const float* __restrict__ w,
                 const float* __restrict__ bias, int taps, const float* __restrict__ state, int64_t state_stride, int n_slots,
                 const int* __restrict__ tok_seq, const int* __restrict__ positions, const int* __restrict__ seq_starts,
                 const int* __restrict__ state_slots, int C, int act) {
@@ -639,7 +640,7 @@ conv_act_kernel(float* __restrict__ out, int64_t ldo, const float* __restrict__ 
         else x = slot_ok ? ring[static_cast<int64_t>(sp % (taps - 1)) * C + c] : 0.0f;
         acc = fmaf(w[static_cast<int64_t>(c) * taps + jt], x, acc);
     }
-    out[static_cast<int64_t>(t) * ldo + c] = act ? silu_f(acc) : acc;
+    out[static_cast<int64_t>(t) * ldo + c] = from_float<T>(act ? silu_f(acc) : acc);
 }
 
 template <typename T>
@@ -812,7 +813,7 @@ extern "C" int liyab_token_shift(void* out, int dtype, const void* h, const floa
     return check_launch("token_shift");
 }
 
-extern "C" int liyab_conv_act(float* out, int64_t ldo, const float* in, int64_t ldi, const float* w, const float* bias, int taps,
+extern "C" int liyab_conv_act(void* out, int out_dtype, int64_t ldo, const float* in, int64_t ldi, const float* w, const float* bias, int taps,
                               const float* state, int64_t state_stride, int n_slots, const int* tok_seq, const int* positions,
                               const int* seq_starts, const int* state_slots, int n, int C, int act, hipStream_t stream) {
     LIYAB_REQUIRE(out && in && w && tok_seq && positions && seq_starts && state_slots, "conv_act: null pointer");
@@ -821,8 +822,13 @@ extern "C" int liyab_conv_act(float* out, int64_t ldo, const float* in, int64_t 
                   "conv_act: %d taps need the last %d rows of a request in its slot", taps, taps - 1);
     if (n == 0) return 0;
     dim3 grid((C + 255) / 256, n);
-    conv_act_kernel<<<grid, 256, 0, stream>>>(out, ldo, in, ldi, w, bias, taps, state, state_stride, taps > 1 ? n_slots : 0, tok_seq, positions,
-                                              seq_starts, state_slots, C, act);
+    if (out_dtype == kF32)
+        conv_act_kernel<float><<<grid, 256, 0, stream>>>(static_cast<float*>(out), ldo, in, ldi, w, bias, taps, state, state_stride, taps > 1 ? n_slots : 0, tok_seq,
+                                                         positions, seq_starts, state_slots, C, act);
+    else if (out_dtype == kBF16)
+        conv_act_kernel<bf16_t><<<grid, 256, 0, stream>>>(static_cast<bf16_t*>(out), ldo, in, ldi, w, bias, taps, state, state_stride, taps > 1 ? n_slots : 0, tok_seq,
+                                                          positions, seq_starts, state_slots, C, act);
+    else return fail(1, "conv_act: unknown dtype %d", out_dtype);
     return check_launch("conv_act");
 }
 

@@ -133,6 +133,10 @@ static const Entry kEntries[] = {
     LIYAB_ENTRY(liyab_lru_conv),
     LIYAB_ENTRY(liyab_lru_coeffs),
     LIYAB_ENTRY(liyab_lru_scan),
+    LIYAB_ENTRY(liyab_streams_update),
+    LIYAB_ENTRY(liyab_scan_steps),
+    LIYAB_ENTRY(liyab_selective_scan),
+    LIYAB_ENTRY(liyab_selective_single),
 };
 constexpr int kNumEntries = static_cast<int>(sizeof(kEntries) / sizeof(kEntries[0]));
 

@@ -79,17 +79,17 @@ _SIGNATURES = {
     "liyab_keep_rows": [P, c_int, c_int, P, P, P, P, P, P, c_int, c_int, P],
     "liyab_latent_store": [P, c_int, P, c_int64, c_int, P, c_float, P, c_int, c_int, c_int, c_int, P],
     "liyab_grouped_product": [P, c_int64, c_int, c_int, P, P, c_int, P, c_int, c_int64, c_int, P, P, c_int, c_int, c_int, P, P, c_int, c_int64,
-                              c_int, c_int, c_int, c_int, c_int, c_int, P],
-    "liyab_moe_route": [P, c_int64, c_int, c_int, c_int, P, P, c_int, c_int, c_int, P, P],
+                              c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_float, P],
+    "liyab_moe_route": [P, c_int64, c_int, c_int, c_int, P, P, c_int, c_int, c_int, P, c_float, c_int, c_int, P],
     "liyab_moe_align": [P, c_int, c_int, c_int, P, P, c_int, P],
-    "liyab_moe_route_align": [P, c_int64, c_int, c_int, c_int, P, P, c_int, P, P, c_int, c_int, c_int, c_int, P, P],
+    "liyab_moe_route_align": [P, c_int64, c_int, c_int, c_int, P, P, c_int, P, P, c_int, c_int, c_int, c_int, P, c_float, c_int, c_int, P],
     "liyab_attention_decode_scored": [P, c_int64, P, c_int64, P, P, c_int, P, c_int, P, P, P, c_int, c_float, c_int, c_int, c_int,
                                       c_int, c_int, c_int, c_int, c_int, c_int, P, c_int, c_int, c_float, P, c_int, P, c_int, P],
     "liyab_attention_prefill_scored": [P, c_int64, P, c_int64, P, P, P, c_int, P, c_int, c_int, c_int, c_float, c_int, c_int,
                                        c_int, c_int, c_int, c_int, c_float, P, c_int, P, c_int, P],
     "liyab_gate_rows": [P, c_int, c_int64, P, c_int64, c_int, c_int, c_float, P],
     "liyab_dyt": [P, c_int, P, P, P, P, P, c_int, c_int, P],
-    "liyab_glu_clamped": [P, c_int, P, c_int64, c_int, c_int, c_float, c_float, c_float, P],
+    "liyab_glu_clamped": [P, c_int, P, c_int64, c_int, c_int, c_float, c_float, c_float, P, c_int64, P],
     "liyab_glu": [P, c_int, P, c_int64, c_int, c_int, c_int, P],
     "liyab_activate": [P, c_int, c_int64, P, c_int64, c_int, c_int, c_int, P],
     "liyab_mean_norm_add": [P, P, P, P, P, c_float, c_float, c_int, c_int, P],
@@ -103,7 +103,7 @@ _SIGNATURES = {
     "liyab_gla_single": [P, c_int, P, P, P, P, c_int64, P, c_int64, P, P, c_float, P, c_float, c_float, P, c_int64, c_int, P, P, P, c_int, c_int, c_int,
                          c_int, c_int, P],
     "liyab_token_shift": [P, c_int, P, P, c_int, P, c_int64, c_int, P, P, P, P, c_int, c_int, P],
-    "liyab_conv_act": [P, c_int64, P, c_int64, P, P, c_int, P, c_int64, c_int, P, P, P, P, c_int, c_int, c_int, P],
+    "liyab_conv_act": [P, c_int, c_int64, P, c_int64, P, P, c_int, P, c_int64, c_int, P, P, P, P, c_int, c_int, c_int, P],
     "liyab_gated_group_norm": [P, c_int, P, c_int64, P, c_int64, P, c_float, c_int, c_int, c_int, P],
     "liyab_qk_prepare": [P, c_int64, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, P, P, P, c_int, P, c_int, c_int, P, P, c_float, P,
                          c_int, c_float, c_int, P, c_int, c_int, c_float, P, P, P, P],
@@ -133,6 +133,12 @@ _SIGNATURES = {
     "liyab_lru_coeffs": [P, P, P, c_int64, P, P, P, P, c_float, c_int, c_int, c_int, P],
     "liyab_lru_scan": [P, c_int, P, c_int64, P, P, P, P, P, P, c_float, c_float, P, c_int64, P, c_int64, c_int, P, c_int64, c_int, P, P, P, c_int, c_int,
                        c_int, c_int, P],
+    "liyab_streams_update": [P, P, P, c_int, P, P, c_int, P, P, P, P, P, c_float, P, c_int, P, c_int, c_int, c_int, P],
+    "liyab_scan_steps": [P, P, c_int64, P, c_int, P, c_int, c_int, c_int, P],
+    "liyab_selective_scan": [P, c_int, P, P, P, c_int64, P, c_int64, P, P, P, c_int64, c_int, P, c_int64, c_int, P, P, P, c_int, c_int, c_int, c_int,
+                             c_int, P, P, P],
+    "liyab_selective_single": [P, c_int, P, P, c_int64, c_int, P, P, P, c_int64, P, P, P, c_int64, c_int, P, c_int64, c_int, P, P, P, c_int, c_int,
+                               c_int, P],
 }
 
 

@@ -1225,7 +1225,7 @@ def heads_product(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor, gate: Opt
                             and w.data_ptr() % 16 == 0) else GROUPED_ROWS
     _lib.call("liyab_grouped_product", a.data_ptr(), lda, 1, K, w.data_ptr(), None, dtype_code(a.dtype), out.data_ptr(),
               dtype_code(out.dtype), ldo, N, None, None, (n + block - 1) // block, block, H, None, _ptr(gate),
-              dtype_code(gate.dtype) if gate is not None else F32, gs, n, N, K, 0, 1, 0, _stream())
+              dtype_code(gate.dtype) if gate is not None else F32, gs, n, N, K, 0, 1, 0, 0.0, 0.0, 0.0, _stream())
 
 
 MOE_MAX_TOP = 64
@@ -1253,30 +1253,40 @@ MOE_WAVE_TOKENS = 64  # tokens such a choice and its lists take in one launch (k
 
 
 def moe_route(logits: torch.Tensor, top: int, ids: torch.Tensor, weights: torch.Tensor, rows_list: torch.Tensor,
-              tile_group: torch.Tensor, block: int = GROUPED_ROWS, groups: Optional[tuple] = None, logistic: bool = False,
-              correction: Optional[torch.Tensor] = None) -> None:
+              tile_group: torch.Tensor, block: int = GROUPED_ROWS, groups: Optional[tuple] = None, scores: str = "softmax",
+              correction: Optional[torch.Tensor] = None, scale: float = 1.0, identity: int = 0, extra: bool = False, n_lists: int = 0) -> None:
     """From float32 router logits [n, experts] (rows may be strided): ids int32 and weights float32 [n,
     top] (the experts with the largest logits, softmax over those alone), and the entries t * top + k
     listed by expert in tiles of `block` places: rows_list int32 [tiles * block] (-1: empty), tile_group
     int32 [tiles] (-1: unused), tiles = moe_tiles(n * top, experts, block). `groups` = (count, keep): the choice among groups
     of experts instead: softmax over all experts, the experts in `count` equal groups of neighbours, only those of the `keep`
-    groups with the largest member can be chosen, the weights the chosen scores divided by their sum. `logistic`: scores s = sigmoid(logit),
+    groups with the largest member can be chosen, the weights the chosen scores divided by their sum. `scores` "logistic": s = sigmoid(logit),
     the choice by s + correction (float32 [experts], or None); a group's score is then the sum of its two largest, and the weights are the
-    chosen s as they are."""
+    chosen s as they are. "softmax_all": the same with s = softmax(logits) over all outputs and weights scale * s. With either of these, the last
+    `identity` outputs are identity experts: an entry that takes one gets the id -1 and stands in no list; and `extra`: the logits have one
+    column more, and a token one more entry behind its `top`, of the expert behind the listed ones, weighted sigmoid(that logit). `n_lists`: the
+    experts that `tile_group` and `rows_list` are made for, where they are more than the router lists."""
     ld = _rows(logits, "logits")
     n, E = logits.shape
+    E -= 1 if extra else 0
+    logistic = scores in ("logistic", "softmax_all")  # the choice by corrected scores, a wave a token
+    if not logistic and scores != "softmax":
+        raise KernelError(f"moe_route: scores '{scores}'")
+    listed, rows = E - identity + (1 if extra else 0), top + (1 if extra else 0)
+    if identity < 0 or identity >= E or ((identity or extra or scale != 1.0) and not logistic) or (scale != 1.0 and scores != "softmax_all"):
+        raise KernelError("moe_route: identity experts, an entry for every token and a scale go with corrected scores")
     if logits.dtype != torch.float32:
         raise KernelError("moe_route: the logits must be float32")
     if not 1 <= top <= min(E, MOE_MAX_TOP):
         raise KernelError(f"moe_route: {top} of {E} experts a token (at most {MOE_MAX_TOP})")
     if block not in (GROUPED_ROWS, SKINNY_ROWS):
         raise KernelError(f"moe_route: tiles of {block} places ({GROUPED_ROWS} or {SKINNY_ROWS})")
-    tiles = moe_tiles(n * top, E, block)
-    _i32(ids, "ids", n * top)
+    tiles = moe_tiles(n * rows, max(listed, n_lists), block)
+    _i32(ids, "ids", n * rows)
     _i32(rows_list, "rows_list", tiles * block)
     _i32(tile_group, "tile_group", tiles)
     _dev(weights, "weights")
-    if weights.dtype != torch.float32 or weights.numel() < n * top or not weights.is_contiguous():
+    if weights.dtype != torch.float32 or weights.numel() < n * rows or not weights.is_contiguous():
         raise KernelError("moe_route: weights must be contiguous float32 [n, top]")
     mode, count, keep = 0, 1, 1
     if groups is not None:
@@ -1284,27 +1294,29 @@ def moe_route(logits: torch.Tensor, top: int, ids: torch.Tensor, weights: torch.
         if not (1 <= count <= MOE_MAX_GROUPS and E % count == 0 and 1 <= keep <= count and top <= keep * (E // count)):
             raise KernelError(f"moe_route: {keep} of {count} groups of {E} experts do not hold {top} choices (at most {MOE_MAX_GROUPS} groups)")
     if logistic:
-        mode = 2
+        mode = 2 if scores == "logistic" else 3
         if E > MOE_MAX_WAVE_EXPERTS:
-            raise KernelError(f"moe_route: {E} experts with logistic scores (at most {MOE_MAX_WAVE_EXPERTS})")
+            raise KernelError(f"moe_route: {E} experts with corrected scores (at most {MOE_MAX_WAVE_EXPERTS})")
         _f32vec(correction, "the choice's correction", E)
     elif correction is not None:
         raise KernelError("moe_route: a correction goes with logistic scores")
-    if n <= (1024 if mode != 2 else MOE_WAVE_TOKENS if E <= 512 else 0):  # one launch: the tokens are routed, then the workgroup lists the entries
+    more = (float(scale), E - identity, 1 if extra else 0)
+    if n <= (1024 if mode < 2 else MOE_WAVE_TOKENS if E <= 512 else 0):  # one launch: the tokens are routed, then the workgroup lists the entries
         _lib.call("liyab_moe_route_align", logits.data_ptr(), ld, n, E, top, ids.data_ptr(), weights.data_ptr(), block,
-                  rows_list.data_ptr(), tile_group.data_ptr(), tiles, mode, count, keep, _ptr(correction), _stream())
+                  rows_list.data_ptr(), tile_group.data_ptr(), tiles, mode, count, keep, _ptr(correction), *more, _stream())
         return
-    _lib.call("liyab_moe_route", logits.data_ptr(), ld, n, E, top, ids.data_ptr(), weights.data_ptr(), mode, count, keep, _ptr(correction), _stream())
-    _lib.call("liyab_moe_align", ids.data_ptr(), n * top, E, block, rows_list.data_ptr(), tile_group.data_ptr(), tiles, _stream())
+    _lib.call("liyab_moe_route", logits.data_ptr(), ld, n, E, top, ids.data_ptr(), weights.data_ptr(), mode, count, keep, _ptr(correction), *more, _stream())
+    _lib.call("liyab_moe_align", ids.data_ptr(), n * rows, listed, block, rows_list.data_ptr(), tile_group.data_ptr(), tiles, _stream())
 
 
 def moe_product(out: torch.Tensor, a: torch.Tensor, w0: torch.Tensor, w1: Optional[torch.Tensor], rows_list: torch.Tensor,
                 tile_group: torch.Tensor, *, a_div: int = 1, row_scale: Optional[torch.Tensor] = None, block: int = GROUPED_ROWS,
-                act: str = "none", out_div: int = 1, out_extra: int = 0) -> None:
+                act: str = "none", out_div: int = 1, out_extra: int = 0, clamp: Optional[tuple] = None) -> None:
     """For every listed entry e of expert g: out[e] = f(a[e // a_div] . w0[g]^T, a[e // a_div] . w1[g]^T) *
     row_scale[e], f(u, v) = silu(u) * v with two matrices and u with one. a [*, K] and out [entries, N]
     contiguous, w0 / w1 [experts, N, K] in a's dtype; rows_list and tile_group as `moe_route` leaves them for
-    tiles of `block` places. `act` = "relu2" (one matrix): f(u) = relu(u)^2. `out_extra`: rows of `out` left free behind each
+    tiles of `block` places. `act` = "relu2" (one matrix): f(u) = relu(u)^2. `clamp` = (limit, slope, shift) (two
+    matrices): f(u, v) = g * sigmoid(slope * g) * (w + shift) with g = min(u, limit), w = clamp(v, -limit, limit). `out_extra`: rows of `out` left free behind each
     `out_div` rows (a token's entries), which another product fills: entry e then lies at row e + (e // out_div) * out_extra."""
     _dev(w0, "w0")
     if w0.dim() != 3 or not w0.is_contiguous() or w0.dtype != a.dtype:
@@ -1313,7 +1325,7 @@ def moe_product(out: torch.Tensor, a: torch.Tensor, w0: torch.Tensor, w1: Option
     if w1 is not None and (tuple(w1.shape) != (E, N, K) or not w1.is_contiguous() or w1.dtype != a.dtype):
         raise KernelError("moe_product: w1 must match w0")
     lda, ldo = _rows(a, "a"), _rows(out, "out")
-    if act not in ("none", "relu2") or (act != "none" and w1 is not None) or out_extra < 0 or out_div < 1 or (out_extra and out.shape[0] % (out_div + out_extra)):
+    if act not in ("none", "relu2") or (act != "none" and w1 is not None) or (clamp is not None and (w1 is None or not clamp[0] > 0)) or out_extra < 0 or out_div < 1 or (out_extra and out.shape[0] % (out_div + out_extra)):
         raise KernelError(f"moe_product: activation '{act}' / {out_extra} free rows a token are not taken here")
     entries = out.shape[0] // (out_div + out_extra) * out_div if out_extra else out.shape[0]
     if a.shape[1] != K or out.shape[1] != N or a_div < 1 or a.shape[0] * a_div < entries:
@@ -1331,7 +1343,8 @@ def moe_product(out: torch.Tensor, a: torch.Tensor, w0: torch.Tensor, w1: Option
             raise KernelError("moe_product: row_scale must be contiguous float32 [entries]")
     _lib.call("liyab_grouped_product", a.data_ptr(), lda, a_div, 0, w0.data_ptr(), _ptr(w1), dtype_code(a.dtype), out.data_ptr(),
               dtype_code(out.dtype), ldo, 0, rows_list.data_ptr(), tile_group.data_ptr(), tiles, block, E, _ptr(row_scale), None, F32, 0,
-              entries, N, K, 1 if act == "relu2" else 0, int(out_div), int(out_extra), _stream())
+              entries, N, K, 2 if clamp is not None else 1 if act == "relu2" else 0, int(out_div), int(out_extra),
+              *(float(v) for v in (clamp or (0.0, 0.0, 0.0))), _stream())
 
 
 # -- norms without statistics, clamped gated activations, two sublayers' results joined ------------
@@ -1354,15 +1367,23 @@ def dyt(out: torch.Tensor, x: torch.Tensor, weight: Optional[torch.Tensor], bias
     _lib.call("liyab_dyt", out.data_ptr(), dtype_code(out.dtype), x.data_ptr(), _ptr(weight), _ptr(bias), alpha.data_ptr(), _ptr(rows), n, d, _stream())
 
 
-def glu_clamped(out: torch.Tensor, gu: torch.Tensor, limit: float, slope: float, shift: float) -> None:
+def glu_clamped(out: torch.Tensor, gu: torch.Tensor, limit: float, slope: float, shift: float, row_gate: Optional[torch.Tensor] = None) -> None:
     """out = g * sigmoid(slope * g) * (u + shift) with g = min(G, limit), u = clamp(U, -limit, limit); gu float32
-    [n, 2 * ff] = [G | U], out contiguous [n, ff] float32 or bfloat16."""
+    [n, 2 * ff] = [G | U], out contiguous [n, ff] float32 or bfloat16. `row_gate` (float32 [n, 1], a column of wider rows): a row's entries
+    times the sigmoid of its number there."""
     _dev(out, "out")
     ld = _rows(gu, "gu")
     n, ff = out.shape
     if gu.dtype != torch.float32 or tuple(gu.shape) != (n, 2 * ff) or not out.is_contiguous():
         raise KernelError(f"glu_clamped: needs float32 [n, {2 * ff}] and a contiguous out [n, {ff}], got {tuple(gu.shape)} {gu.dtype}")
-    _lib.call("liyab_glu_clamped", out.data_ptr(), dtype_code(out.dtype), gu.data_ptr(), ld, n, ff, float(limit), float(slope), float(shift), _stream())
+    gs = 0
+    if row_gate is not None:
+        _dev(row_gate, "row_gate")
+        if row_gate.dtype != torch.float32 or tuple(row_gate.shape) != (n, 1):
+            raise KernelError(f"glu_clamped: the rows' gate must be float32 [{n}, 1]")
+        gs = row_gate.stride(0)
+    _lib.call("liyab_glu_clamped", out.data_ptr(), dtype_code(out.dtype), gu.data_ptr(), ld, n, ff, float(limit), float(slope), float(shift), _ptr(row_gate), gs,
+              _stream())
 
 
 GLU_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
@@ -1497,13 +1518,13 @@ def wkv_scan(out: torch.Tensor, proj: torch.Tensor, w0: torch.Tensor, u: torch.T
 
 def conv_act(out: torch.Tensor, x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], state: Optional[torch.Tensor],
              ring_off: int, ctx, act: bool = True) -> None:
-    """(`act` False: without the silu.) out[t, c] = silu(bias[c] + sum_j weight[c, j] * x[t - taps + 1 + j, c]) over each request's own rows in time; x, out float32
-    rows (columns of wider rows are fine), weight float32 [C, taps]; the rows before a request's first row of the step come from
+    """(`act` False: without the silu.) out[t, c] = silu(bias[c] + sum_j weight[c, j] * x[t - taps + 1 + j, c]) over each request's own rows in time; x float32
+    rows, out float32 or bfloat16 rows (columns of wider rows are fine), weight float32 [C, taps]; the rows before a request's first row of the step come from
     state[slot, ring_off + (position % (taps - 1)) * C + c], zeros before position 0."""
     ldo, ldi = _rows(out, "out"), _rows(x, "x")
     n, C = x.shape
-    if x.dtype != torch.float32 or out.dtype != torch.float32 or tuple(out.shape) != (n, C) or ctx.n_tokens != n:
-        raise KernelError("conv_act: x and out must be the step's float32 rows of one shape")
+    if x.dtype != torch.float32 or tuple(out.shape) != (n, C) or ctx.n_tokens != n:
+        raise KernelError("conv_act: x must be the step's float32 rows and out rows of their shape")
     _dev(weight, "weight")
     if weight.dtype != torch.float32 or weight.dim() != 2 or weight.shape[0] != C or not weight.is_contiguous():
         raise KernelError(f"conv_act: the weight must be contiguous float32 [{C}, taps]")
@@ -1516,7 +1537,7 @@ def conv_act(out: torch.Tensor, x: torch.Tensor, weight: torch.Tensor, bias: Opt
             raise KernelError("conv_act: the ring does not lie in the slot")
         slots, base = state.shape[0], state.data_ptr() + 4 * ring_off
     _step_lists(ctx, n)
-    _lib.call("liyab_conv_act", out.data_ptr(), ldo, x.data_ptr(), ldi, weight.data_ptr(), _ptr(bias), taps, base, stride, slots,
+    _lib.call("liyab_conv_act", out.data_ptr(), dtype_code(out.dtype), ldo, x.data_ptr(), ldi, weight.data_ptr(), _ptr(bias), taps, base, stride, slots,
               ctx.tok_seq.data_ptr(), ctx.positions.data_ptr(), ctx.seq_starts.data_ptr(), ctx.state_slots.data_ptr(), n, C, 1 if act else 0,
               _stream())
 
@@ -2149,3 +2170,121 @@ def lru_scan(out: torch.Tensor, z: torch.Tensor, u: torch.Tensor, y: torch.Tenso
     _lib.call("liyab_lru_scan", out.data_ptr(), dtype_code(out.dtype), z.data_ptr(), ldz, u.data_ptr(), _ptr(decay), _ptr(gated), br.data_ptr(), bi.data_ptr(),
               lam.data_ptr(), float(rate), float(out_scale), y.data_ptr(), ldy, state.data_ptr(), stride, state.shape[0], x.data_ptr(), ldx, int(taps),
               ctx.seq_starts.data_ptr(), ctx.positions.data_ptr(), ctx.state_slots.data_ptr(), ctx.n_seqs, C, int(blocks), 1 if stretches else 0, _stream())
+
+
+# -- several residual streams -----------------------------------------------------------------------------
+MAX_STREAMS = 8  # csrc/streams.hip: ST_MAX_STREAMS
+
+
+class IdentityEntries:
+    """Which of the rows a routed feed-forward leaves a token stand for an identity expert: `ids` and `weights` [n * n_ids] as the router
+    leaves them (id -1: the entry's result is its weight times the row of `h` that the feed-forward read, and its own row is not written)."""
+
+    def __init__(self, ids: torch.Tensor, weights: torch.Tensor, n_ids: int, h: torch.Tensor):
+        self.ids, self.weights, self.n_ids, self.h = ids, weights, int(n_ids), h
+
+
+def streams_update(x: torch.Tensor, *, enter: Optional[torch.Tensor] = None, y: Optional[torch.Tensor] = None, n_sum: int = 1,
+                   identity: Optional[IdentityEntries] = None, mix: Optional[torch.Tensor] = None, add: Optional[torch.Tensor] = None, next_norm=None,
+                   out: Optional[torch.Tensor] = None, rows: Optional[torch.Tensor] = None) -> None:
+    """x float32 [n, streams, d]: x_t <- sum_s mix[s, t] x_s + add[t] s for every token, s the sum of its `n_sum` rows of y (float32 [n *
+    n_sum, d]; `identity` says which of them stand for identity experts); mix float32 [streams, streams] ([from, to]; None: each stream stays),
+    add float32 [streams] (None: ones). `enter` (float32 [n, d]) sets all streams to its rows first; without y nothing is added. `next_norm` =
+    (combination float32 [streams] or None for ones, weight float32 [d] or None, eps): `out` [n, d] gets u / sqrt(mean(u^2) + eps) * weight with u = sum_s
+    combination[s] x_s of the new streams. `rows`: out [len(rows), d] of those rows of x, which stays as it is."""
+    _dev(x, "x")
+    n, S, d = x.shape
+    if x.dtype != torch.float32 or not x.is_contiguous() or not 1 <= S <= MAX_STREAMS:
+        raise KernelError(f"streams_update: x must be contiguous float32 [n, up to {MAX_STREAMS} streams, d], got {tuple(x.shape)} {x.dtype}")
+    if enter is not None:
+        _dev(enter, "enter")
+        if enter.dtype != torch.float32 or tuple(enter.shape) != (n, d) or not enter.is_contiguous() or (S > 1 and enter.data_ptr() == x.data_ptr()):
+            raise KernelError(f"streams_update: the entering rows must be contiguous float32 [{n}, {d}] of their own")
+    if y is not None:
+        _dev(y, "y")
+        if y.dtype != torch.float32 or not y.is_contiguous() or n_sum < 1 or y.numel() != n * n_sum * d:
+            raise KernelError(f"streams_update: y must be contiguous float32 with {n_sum} rows of {d} a token, got {tuple(y.shape)} {y.dtype}")
+    _f32vec(mix, "mix", S * S)
+    _f32vec(add, "add", S)
+    take, weight, eps = next_norm if next_norm is not None else (None, None, 0.0)
+    code, count = F32, n
+    if out is not None:
+        _dev(out, "out")
+        count = n if rows is None else out.shape[0]
+        if next_norm is None or tuple(out.shape) != (count, d) or not out.is_contiguous():
+            raise KernelError(f"streams_update: out must be contiguous [{count}, {d}] and needs a norm")
+        _f32vec(take, "the next sublayer's combination", S)
+        _f32vec(weight, "the next norm's weight", d)
+        code = dtype_code(out.dtype)
+        if rows is not None:
+            _i32(rows, "rows", count)
+    ids = weights = h = None
+    n_ids = 0
+    if identity is not None:
+        ids, weights, n_ids, h = identity.ids, identity.weights, identity.n_ids, identity.h
+        _i32(ids, "ids", n * n_ids)
+        _f32vec(weights, "weights", n * n_ids)
+        _dev(h, "h")
+        if out is None:
+            code = dtype_code(h.dtype)
+        if dtype_code(h.dtype) != code or tuple(h.shape) != (n, d) or not h.is_contiguous() or not 1 <= n_ids <= n_sum:
+            raise KernelError(f"streams_update: identity entries need the rows [{n}, {d}] that were routed, in the next rows' dtype")
+    _lib.call("liyab_streams_update", x.data_ptr(), _ptr(enter), _ptr(y), int(n_sum), _ptr(ids), _ptr(weights), n_ids, _ptr(h), _ptr(mix), _ptr(add), _ptr(take),
+              _ptr(weight), float(eps), _ptr(out), code, _ptr(rows), count, S, d, _stream())
+
+
+# -- a selective scan: a state of its own for every channel and state number ------------------------------
+SELECTIVE_MAX_STATES = 128  # csrc/selective_scan.hip: kMaxScanStates
+SELECTIVE_SEGMENTS_FROM = 48  # the longest portion a step may hold from which its walks run in segments side by side
+SELECTIVE_WAVES = 1024  # waves that segments of 64 tokens should make before they are taken; shorter ones below
+
+
+def selective_segments(n: int, n_seqs: int, channels: int):
+    """(tokens a segment, the most segments) of a step's walks, (0, 0): each portion by one wave a 64 channels. From the step's rows and
+    requests alone, as its grids, so that a captured graph holds for every step of its shape."""
+    if n - n_seqs + 1 < SELECTIVE_SEGMENTS_FROM:
+        return 0, 0
+    tokens = 64 if -(-n // 64) * -(-channels // 64) >= SELECTIVE_WAVES else 32
+    return tokens, -(-n // tokens) + n_seqs
+
+
+def selective_scan(out: torch.Tensor, x: torch.Tensor, low: torch.Tensor, z: torch.Tensor, dt_weight: torch.Tensor, dt_weight_t: torch.Tensor, dt_bias: torch.Tensor,
+                   a2: torch.Tensor, skip: torch.Tensor, state: StateSlice, raw: torch.Tensor, taps: int, ctx) -> None:
+    """S[c, n] <- exp2(dt_c a2[n, c]) S[c, n] + dt_c x_c B_n, out_c = (sum_n S[c, n] C_n + skip_c x_c) silu(z_c) along each request's rows of the step, with
+    dt = softplus(low . dt_weight^T + dt_bias). x, out contiguous [n, C] in the compute dtype; low float32 rows [n, rank + 2 N] = [low | B | C]; z float32 rows
+    [n, C]; dt_weight [C, rank] and once more as dt_weight_t [rank, C] in the compute dtype; a2 float32 [N, C] = A log2(e). `state`: S [N, C] and behind it the last
+    taps - 1 rows of `raw` (float32 rows [n, C]), position p at ring place p % (taps - 1). S starts from zero at position 0."""
+    _dev(out, "out")
+    _dev(x, "x")
+    n, C = x.shape
+    N, rank = a2.shape[0], dt_weight.shape[1]
+    ldb, ldz, ldr = _rows(low, "low"), _rows(z, "z"), _rows(raw, "raw")
+    if tuple(out.shape) != (n, C) or out.dtype != x.dtype or not out.is_contiguous() or not x.is_contiguous() or ctx.n_tokens != n:
+        raise KernelError("selective_scan: x and out must be the step's contiguous rows of one shape and dtype")
+    if any(t.dtype != torch.float32 for t in (low, z, raw)) or tuple(low.shape) != (n, rank + 2 * N) or tuple(z.shape) != (n, C) or tuple(raw.shape) != (n, C):
+        raise KernelError(f"selective_scan: low [{n}, {rank + 2 * N}], z and raw [{n}, {C}] must be float32 rows")
+    for w, shape in ((dt_weight, (C, rank)), (dt_weight_t, (rank, C))):
+        _dev(w, "dt_weight")
+        if w.dtype != x.dtype or tuple(w.shape) != shape or not w.is_contiguous():
+            raise KernelError(f"selective_scan: the step sizes' weights must be contiguous {shape} in x's dtype, got {tuple(w.shape)} {w.dtype}")
+    if not 1 <= N <= SELECTIVE_MAX_STATES or taps < 1 or state.size != (N + taps - 1) * C:
+        raise KernelError(f"selective_scan: {N} states (up to {SELECTIVE_MAX_STATES}), {taps} taps, a slot of {state.size} floats")
+    _f32vec(dt_bias, "dt_bias", C)
+    _f32vec(a2, "a2", N * C)
+    _f32vec(skip, "skip", C)
+    _step_lists(ctx, n)
+    code, lists = dtype_code(x.dtype), (ctx.seq_starts.data_ptr(), ctx.positions.data_ptr(), ctx.state_slots.data_ptr(), ctx.n_seqs)
+    kept = (state.data_ptr(), state.stride, state.n_slots, raw.data_ptr(), ldr, taps - 1)
+    if single_token_step(ctx):
+        _lib.call("liyab_selective_single", out.data_ptr(), code, x.data_ptr(), low.data_ptr(), ldb, rank, dt_weight_t.data_ptr(), dt_bias.data_ptr(), z.data_ptr(), ldz,
+                  a2.data_ptr(), skip.data_ptr(), *kept, *lists, C, N, _stream())
+        return
+    dt = ctx.workspace.get("selective_dt", (n, C), torch.float32)
+    _lib.call("liyab_scan_steps", dt.data_ptr(), low.data_ptr(), ldb, dt_weight.data_ptr(), code, dt_bias.data_ptr(), n, C, rank, _stream())
+    tokens, most = selective_segments(n, ctx.n_seqs, C)
+    ends = sums = None
+    if tokens:
+        ends = ctx.workspace.get("selective_ends", (most, N, C), torch.float32)
+        sums = ctx.workspace.get("selective_sums", (most, C), torch.float32)
+    _lib.call("liyab_selective_scan", out.data_ptr(), code, x.data_ptr(), dt.data_ptr(), low.data_ptr() + 4 * rank, ldb, z.data_ptr(), ldz, a2.data_ptr(), skip.data_ptr(),
+              *kept, *lists, C, N, tokens, most, _ptr(ends), _ptr(sums), _stream())

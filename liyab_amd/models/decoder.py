@@ -130,7 +130,7 @@ class DecoderModel:
             # sublayer's input, gates on the results): built here, handed over by name where the plan has them
             extras = {}
             for name, family in (("input_conv", "conv"), ("ffn_conv", "conv"), ("gate_mixer", "gate"), ("gate_ffn", "gate"),
-                                 ("post_norm_mixer", "norm"), ("post_norm_ffn", "norm")):
+                                 ("post_norm_mixer", "norm"), ("post_norm_ffn", "norm"), ("connect_mixer", "connection"), ("connect_ffn", "connection")):
                 extra = getattr(spec, name, None)
                 if extra is not None:
                     extras[name] = build_part(family, extra, store, dtype)
@@ -138,6 +138,12 @@ class DecoderModel:
         # what is done to the stream ahead of a layer (where a repeated stretch of layers begins a pass), by the layer's number
         self.entries = {i: build_part("entry", spec.entry, store, dtype) for i, spec in enumerate(plan.layers) if getattr(spec, "entry", None) is not None}
         self.keeps_embedding = any(getattr(e, "needs_embedding", False) for e in self.entries.values())
+        # several residual streams [n, streams, width]: every block works on all of them, the first one sets them to the embedding's output
+        # (`enter`, which also takes its first norm), and the final norm reads their sum
+        self.streams = int(getattr(plan, "streams", 0) or 0)
+        if self.streams:
+            if self.entries or plan.final_norm is None or any(not hasattr(b, "enter") for b in self.blocks):
+                raise ValueError("several residual streams need blocks that take them (arrangement 'streams'), a final norm, and nothing between the layers")
         self.final_norm = build_part("norm", plan.final_norm, store, dtype) if plan.final_norm is not None else None
         self.head = build_part("head", plan.head, store, dtype)
         self.order = list(plan.order)
@@ -147,6 +153,8 @@ class DecoderModel:
             for i in range(len(self.blocks) - 1):
                 if hasattr(self.blocks[i], "chain_norm") and (i + 1) not in self.entries:
                     self.blocks[i].chain_norm(self.blocks[i + 1])
+        if self.streams:
+            self.blocks[self.order[0].layer].input_normed = True  # (by `enter`)
         # the parts' step planners, one of each name (every attention layer shares attention's)
         self.step_planners = []
         for block in self.blocks:
@@ -222,6 +230,10 @@ class DecoderModel:
             # the embedding's output as later layers' entries read it: rounded once to the compute dtype
             embedded = ctx.workspace.get("embedding_out", (ctx.n_tokens, self.width), self.dtype)
             ops.gather_rows(embedded, x)
+        if self.streams:
+            embedded, x = x, (ctx.workspace.get("residual_streams", (ctx.n_tokens, self.streams, self.width), torch.float32) if self.streams > 1
+                              else x.view(ctx.n_tokens, 1, self.width))
+            self.blocks[self.order[0].layer].enter(x, embedded, ctx)
         pending = None  # the stream as a SplitStream while a layer has left it split (x is then stale)
         recorded = {}  # this step's lists of launches, by the kind of layer and the state it found the stream in
         for e in self.order:

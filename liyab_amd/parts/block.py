@@ -4,11 +4,12 @@ from __future__ import annotations
 
 import torch
 
+from ..errors import Unsupported
 from ..kernels import ops
 from .base import SplitStream, StepContext, settled
 from .linear import linear
 from .norms import as_tensor
-from .registry import register_block
+from .registry import register_block, register_connection
 
 
 class PreNormBlock:
@@ -118,6 +119,11 @@ class ParallelBlock:
 register_block("parallel", ParallelBlock)
 
 
+def _refuse_identity(ffn) -> None:
+    if getattr(ffn, "identity", 0):
+        raise Unsupported("a feed-forward with identity experts behind a norm of its result: the rows' update does not read its entries")
+
+
 class PostNormGatedBlock:
     """x += norm_mixer(g1 * mixer(conv(x))); x += norm_ffn(g2 * ffn(x)): the sublayers read the stream
     itself, and the norms stand on their results. g = sigmoid(W x + b) from the stream as the sublayer
@@ -143,6 +149,7 @@ class PostNormGatedBlock:
         for part, what in ((mixer, "mixer"), (ffn, "feed-forward")):
             if part is not None and "out" not in part.forward.__code__.co_varnames:
                 raise ValueError(f"a post-norm block needs a {what} that can leave its result to the block (forward(..., out=))")
+        _refuse_identity(ffn)
         for norm in (norm_mixer, norm_ffn if ffn is not None else norm_mixer):
             if not getattr(norm, "root_mean_square", False) and not getattr(norm, "centred", False):
                 raise ValueError("a post-norm block's row update applies a root-mean-square norm or a layer norm (kinds 'rmsnorm', 'layernorm')")
@@ -251,6 +258,7 @@ class SandwichBlock:
         for part, what in ((mixer, "mixer"), (ffn, "feed-forward")):
             if part is not None and "out" not in part.forward.__code__.co_varnames:
                 raise ValueError(f"a sandwich block needs a {what} that can leave its result to the block (forward(..., out=))")
+        _refuse_identity(ffn)
         for norm in (post_norm_mixer, post_norm_ffn if ffn is not None else post_norm_mixer):
             if norm is None or not getattr(norm, "root_mean_square", False):
                 raise ValueError("a sandwich block's row update applies a root-mean-square norm behind each sublayer (kind 'rmsnorm')")
@@ -371,3 +379,97 @@ class ParallelPairBlock:
 
 
 register_block("parallel_pair", ParallelPairBlock)
+
+
+class StreamConnection:
+    """What ties a sublayer to several residual streams (see StreamConnectionSpec): three small 32-bit tensors that the rows' update
+    reads on the device."""
+
+    replayable = True
+    takes_padding_rows = True
+
+    def __init__(self, spec, store, dtype: torch.dtype):
+        S, t = int(spec.streams), spec.tensors
+        if not 1 <= S <= ops.MAX_STREAMS:
+            raise Unsupported(f"{S} residual streams are not supported (up to {ops.MAX_STREAMS})")
+        self.streams = S
+        self.take = store.fetch(t["take"], (S,), "vector")
+        self.give = store.fetch(t["give"], (S,), "vector")
+        self.mix = store.fetch(t["mix"], (S, S), "vector")
+
+
+register_connection("stream_connection", StreamConnection)
+
+
+class StreamsBlock:
+    """y = mixer(norm_mixer(sum_s take[s] x_s)); x_t <- sum_s mix[s, t] x_s + give[t] y; then the feed-forward in the same way with a
+    connection of its own: a sequential pre-norm layer over several residual streams, or, without connections, over one. The sublayers leave their 32-bit results
+    to the block (`forward(..., out=)`; a feed-forward may leave several rows a token and identity entries), and one kernel a sublayer adds a
+    token's rows up, mixes the streams and takes the next sublayer's norm of them, also the following layer's first (`chain_norm`)."""
+
+    replayable = True
+    takes_padding_rows = True
+    takes_pending = False
+
+    def __init__(self, spec, mixer, ffn, norm_mixer, norm_ffn, connect_mixer=None, connect_ffn=None):
+        self.mixer, self.ffn, self.norm_mixer, self.norm_ffn = mixer, ffn, norm_mixer, norm_ffn if ffn is not None else None
+        self.connect_mixer, self.connect_ffn = connect_mixer, connect_ffn if ffn is not None else None
+        self.mixer_phase = getattr(getattr(spec, "mixer", None), "kind", "mixer")
+        self.ffn_phase = getattr(getattr(spec, "ffn", None), "kind", "ffn")
+        self.next_norm, self.input_normed = None, False
+        for part, what in ((mixer, "mixer"), (ffn, "feed-forward")):
+            if part is not None and "out" not in part.forward.__code__.co_varnames:
+                raise ValueError(f"a block of several streams needs a {what} that can leave its result to the block (forward(..., out=))")
+        for norm in [norm_mixer] + ([norm_ffn] if ffn is not None else []):
+            if norm is None or not getattr(norm, "root_mean_square", False):
+                raise ValueError("a block of several streams takes a root-mean-square norm before each sublayer (kind 'rmsnorm')")
+        if ffn is not None and (connect_mixer is None) != (connect_ffn is None):
+            raise ValueError("a block's sublayers are both connected to the streams, or neither is")
+
+    @staticmethod
+    def _reads(connection, norm):
+        return connection.take if connection is not None else None, norm.weight, norm.eps
+
+    def chain_norm(self, following) -> bool:
+        """Called once, when the model is built, for a block that runs right before `following` in every pass: this block's last
+        update of the rows then also takes `following`'s first norm of them. True if the two were chained."""
+        if not isinstance(following, StreamsBlock) or following.norm_mixer.dtype != self.norm_mixer.dtype:
+            return False
+        self.next_norm = list(self._reads(following.connect_mixer, following.norm_mixer))
+        following.input_normed = True
+        return True
+
+    def enter(self, x: torch.Tensor, embedded: torch.Tensor, ctx: StepContext) -> None:
+        """Sets all streams of `x` to the embedding's output and takes the first sublayer's norm of them, for the first block of a model."""
+        n, _, d = x.shape
+        ops.streams_update(x, enter=embedded, next_norm=self._reads(self.connect_mixer, self.norm_mixer), out=ctx.workspace.get("block_in", (n, d), self.norm_mixer.dtype))
+
+    def _update(self, x, y, ctx, connection, following, **rows) -> torch.Tensor:
+        """The streams with the sublayer's result; what the following sublayer reads, or None where nobody is known to follow."""
+        n, _, d = x.shape
+        h = ctx.workspace.get("block_in", (n, d), self.norm_mixer.dtype) if following is not None else None
+        mix, give = (connection.mix, connection.give) if connection is not None else (None, None)
+        ops.streams_update(x, y=y, mix=mix, add=give, next_norm=following, out=h, **rows)
+        return h
+
+    def forward(self, x: torch.Tensor, ctx: StepContext, cache, state, writes_cache: bool = True):
+        ws, (n, _, d) = ctx.workspace, x.shape
+        if ctx.phases is not None:
+            ctx.phases.mark(self.mixer_phase)
+        h = ws.get("block_in", (n, d), self.norm_mixer.dtype)
+        if not self.input_normed:
+            ops.streams_update(x, next_norm=self._reads(self.connect_mixer, self.norm_mixer), out=h)
+        y = ws.get("sublayer_out", (n, d), torch.float32)
+        self.mixer.forward(h, ctx, cache, state, None, writes_cache=writes_cache, out=y)
+        h = self._update(x, y, ctx, self.connect_mixer, self._reads(self.connect_ffn, self.norm_ffn) if self.ffn is not None else self.next_norm)
+        if self.ffn is not None:
+            if ctx.phases is not None:
+                ctx.phases.mark(self.ffn_phase)
+            k = int(getattr(self.ffn, "rows_a_token", 1))
+            y = ws.get("sublayer_rows", (n * k, d), torch.float32) if k > 1 else y
+            identity = self.ffn.forward(h, ctx, None, out=y)
+            self._update(x, y, ctx, self.connect_ffn, self.next_norm, n_sum=k, identity=identity)
+        return None
+
+
+register_block("streams", StreamsBlock)

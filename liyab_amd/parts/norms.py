@@ -90,7 +90,8 @@ class RMSNorm:
     scaling 32-bit. `rows` gathers (the final norm runs on the wanted rows only). Behind a sublayer,
     a block applies it through the fused residual update (`ops.gated_norm_add`), which reads
     `weight` and `eps` from here. A spec with a `weight_offset` stores its weight around zero: what
-    multiplies is weight + offset, added once at load in 32 bits."""
+    multiplies is weight + offset, added once at load in 32 bits. Rows of several residual streams [n, streams, width] are
+    summed over the streams first."""
 
     replayable = True
     takes_padding_rows = True
@@ -109,9 +110,12 @@ class RMSNorm:
 
     def forward(self, x: torch.Tensor, ctx: StepContext, rows: Optional[torch.Tensor] = None,
                 n_rows: Optional[int] = None, name: str = "normed") -> torch.Tensor:
-        n = x.shape[-2] if rows is None else (n_rows if n_rows is not None else rows.numel())
+        n = x.shape[0] if rows is None else (n_rows if n_rows is not None else rows.numel())
         out = ctx.workspace.get(name, (n, self.width), self.dtype)
-        ops.rmsnorm(out, x, self.weight, self.eps, rows=rows)
+        if x.dim() == 3:
+            ops.streams_update(x, next_norm=(None, self.weight, self.eps), out=out, rows=rows)
+        else:
+            ops.rmsnorm(out, x, self.weight, self.eps, rows=rows)
         return out
 
 

@@ -132,6 +132,11 @@ class ScoredAttention:
                                      lambda: torch.cat([bias, torch.zeros(H * V, dtype=torch.float32, device=bias.device)]).contiguous())
             self.in_bias = bias
         self.sinks = store.fetch(t["sink"], (H,), "vector") if getattr(spec, "sink", False) else None
+        fixed = getattr(spec, "sink_value", None)
+        if fixed is not None:
+            if self.sinks is not None:
+                raise ValueError("scored attention: a sink is learned or fixed, not both")
+            self.sinks = store.derived(("sink_value", float(fixed), H), lambda: torch.full((H,), float(fixed), dtype=torch.float32, device=self.in_weight.device))
         # values shared between layers of a step: the first such layer keeps its values as projected, the later ones mix theirs
         # with those at a learned rate (one float, read on the device); both find the rows under one name in the step's workspace
         self.value_mix = getattr(spec, "value_mix", "") or ""
@@ -149,8 +154,14 @@ class ScoredAttention:
             self.out_weight = store.derived(("padded_heads", t["out"].name, P), lambda: torch.nn.functional.pad(w.view(d, H, V), (0, P - V)).reshape(d, H * P).contiguous())
         per_q, per_k = (H * D, G * D) if self.norm_rows else (D, D)
         normed = spec.qk_norm or self.norm_rows
-        self.q_norm = store.fetch(t["q_norm"], (per_q,), "vector") if normed else None
-        self.k_norm = store.fetch(t["k_norm"], (per_k,), "vector") if normed and not self.kv_shared else None
+        if spec.qk_norm and not getattr(spec, "qk_norm_weights", True):
+            # (heads brought to unit root mean square as they are: a weight of ones)
+            if spec.rotary is not None and spec.rotary.ramp is not None:
+                raise Unsupported("scored attention: norms without weights beside a rotary encoding that is no turn alone")
+            self.q_norm, self.k_norm = (store.derived(("ones", D, c), lambda: torch.ones(D, dtype=torch.float32, device=self.in_weight.device)) for c in "qk")
+        else:
+            self.q_norm = store.fetch(t["q_norm"], (per_q,), "vector") if normed else None
+            self.k_norm = store.fetch(t["k_norm"], (per_k,), "vector") if normed and not self.kv_shared else None
         self.rot_dims, self.freqs, self.rot_halves, self.rot_mag = 0, None, False, 1.0
         if spec.rotary is not None:
             rot = spec.rotary

@@ -469,7 +469,7 @@ def _choice(z, correction, top, groups):
     w = torch.empty(n * top, dtype=torch.float32, device=DEV)
     rows = torch.empty(tiles * ops.GROUPED_ROWS, dtype=torch.int32, device=DEV)
     tile_group = torch.empty(tiles, dtype=torch.int32, device=DEV)
-    ops.moe_route(z.to(DEV).contiguous(), top, ids, w, rows, tile_group, groups=groups, logistic=True,
+    ops.moe_route(z.to(DEV).contiguous(), top, ids, w, rows, tile_group, groups=groups, scores="logistic",
                   correction=correction.to(DEV) if correction is not None else None)
     listed = rows[rows >= 0].cpu().numpy()
     assert sorted(listed.tolist()) == list(range(n * top))  # every entry is listed once, in a tile of its expert
