@@ -6,7 +6,7 @@
     python bench.py --workload medium16|xl64         # the continuous-batching and the batch-64 workloads of the larger sizes
     python bench.py --link-floor                     # what one dependent kernel of a replayed graph costs at least
     python bench.py --product 4096,4096,16384,8,15   # one product in tiles of 128 x 128 and of 256 x 256
-    python bench.py --design bokulix|mofulix|dopilorn|larulorn|lolulorn [--design-sizes small,medium,xl] [--layers L] [--phases]   # that design beside GPT-2 (dopilorn, larulorn: beside Mofulix; lolulorn: beside Larulorn) at equal sizes
+    python bench.py --design bokulix|mofulix|dopilorn|larulorn|lolulorn|lafanex [--design-sizes small,medium,xl] [--layers L] [--phases]   # that design beside GPT-2 (dopilorn, larulorn: beside Mofulix; lolulorn, lafanex: beside Larulorn) at equal sizes
 
 The default run has GPT-2 small's layer sizes (12 layers, width 768, 12 heads
 of 64, feed-forward 3072, vocabulary 50257, 1024 positions) with random
@@ -722,12 +722,81 @@ def lolulorn_prefill_flops(cfg, prompt_lens, logit_rows):
     return flops
 
 
+# The Lafanex of each size has GPT-2's width, layers, vocabulary and head count, and two residual streams; its layers take turns as attention
+# (as many key heads as query heads, whole heads turned) over a gated feed-forward two thirds as wide as GPT-2's, a selective scan twice as wide as the
+# model (16 states a channel, a rank of a sixteenth of the width, four taps) over the same feed-forward, and attention again over eight gated experts of a
+# quarter of GPT-2's inner width and two identity experts, two a token, beside a shared expert of that width. It stands beside Larulorn, the engine's
+# closest design: attention with sinks and a recurrence a channel, a norm before each sublayer, experts beside a shared one.
+def lafanex_config(gpt2_cfg):
+    d, H, F, L = gpt2_cfg["n_embd"], gpt2_cfg["n_head"], gpt2_cfg["n_inner"], gpt2_cfg["n_layer"]
+    hd = d // H
+    dense = {"kind": "dense", "ff": max(64, F * 2 // 3 // 64 * 64)}
+    expert = {"ff": F // 4, "limit": 7.0}
+    moe = {"kind": "moe", "expert": expert, "router": {"experts": 8, "top": 2, "identity": 2, "scale": 2.5}, "shared": expert}
+    attention = {"heads": H, "kv_heads": H, "dim": hd, "vdim": hd, "scale": hd ** -0.5, "rot": {"dims": hd, "base": 10000.0}}
+    kinds = [{"type": "attention", "mixer": attention, "mlp": dense},
+             {"type": "mamba1", "mixer": {"inner": 2 * d, "state": 16, "dt_rank": max(8, d // 16), "conv": 4}, "mlp": dense},
+             {"type": "attention", "mixer": attention, "mlp": moe}]
+    return {"architecture": "Lafanex", "vocab": gpt2_cfg["vocab_size"], "width": d, "streams": 2, "norm": {"eps": 1e-5}, "max_positions": gpt2_cfg["n_positions"],
+            "layers": [json.loads(json.dumps(kinds[i % 3])) for i in range(L)]}
+
+
+def _lafanex_layer_weights(entry, d, experts=None):
+    """Matrix elements of a layer that a token's products read (2 flops an element a token), with `experts` experts in place of a token's own
+    (an identity expert, which has none, taken as one with)."""
+    m, mlp = entry["mixer"], entry.get("mlp")
+    n = 0
+    if mlp and mlp["kind"] == "dense":
+        n += 3 * mlp["ff"] * d
+    elif mlp:
+        r = mlp["router"]
+        n += (r["experts"] + r["identity"] + 1) * d + (experts or r["top"]) * 3 * mlp["expert"]["ff"] * d + 3 * mlp["shared"]["ff"] * d
+    if entry["type"] == "attention":
+        return n + (m["heads"] * m["dim"] + m["kv_heads"] * (m["dim"] + m["vdim"])) * d + d * m["heads"] * m["vdim"]
+    W = m["inner"]
+    return n + 3 * W * d + (2 * m["dt_rank"] + 2 * m["state"]) * W
+
+
+def lafanex_step_bytes(cfg, batch):
+    """The bytes a decode step has to read: every matrix a token of the batch can take (min(batch * top, experts) experts), the head, the
+    cached keys and values, and the 32-bit state of the recurrent layers (read and written) a request."""
+    def step_bytes(contexts, steps, elt):
+        d, V = cfg["width"], cfg["vocab"]
+        total = V * d * elt
+        seen = sum(sum(c + s + 1 for s in range(steps)) for c in contexts) / max(steps, 1)
+        for entry in cfg["layers"]:
+            m, mlp = entry["mixer"], entry.get("mlp")
+            r = mlp["router"] if mlp and mlp["kind"] == "moe" else None
+            total += _lafanex_layer_weights(entry, d, min(len(contexts) * r["top"], r["experts"]) if r else None) * elt
+            if entry["type"] == "attention":
+                total += seen * m["kv_heads"] * (m["dim"] + m["vdim"]) * elt
+            else:
+                total += len(contexts) * 4 * m["inner"] * (2 * m["state"] + m["conv"]) + 4 * m["inner"] * m["state"]
+        return total
+    return step_bytes
+
+
+def lafanex_prefill_flops(cfg, prompt_lens, logit_rows):
+    d, V, n = cfg["width"], cfg["vocab"], sum(prompt_lens)
+    flops = 2.0 * logit_rows * d * V
+    pairs = sum(t * (t + 1) / 2 for t in prompt_lens)
+    for entry in cfg["layers"]:
+        m = entry["mixer"]
+        flops += 2.0 * n * _lafanex_layer_weights(entry, d)
+        if entry["type"] == "attention":
+            flops += 2.0 * pairs * m["heads"] * (m["dim"] + m["vdim"])
+        else:
+            flops += n * m["inner"] * m["state"] * 7.0  # (the recurrence token by token)
+    return flops
+
+
 DESIGNS = {"bokulix": (lambda gpt2, size: bokulix_config(gpt2, BOKULIX_SHAPES[size]), bokulix_step_bytes, bokulix_prefill_flops),
            "mofulix": (lambda gpt2, size: mofulix_config(gpt2), mofulix_step_bytes, mofulix_prefill_flops),
            "dopilorn": (lambda gpt2, size: dopilorn_config(gpt2), dopilorn_step_bytes, dopilorn_prefill_flops),
            "larulorn": (lambda gpt2, size: larulorn_config(gpt2), larulorn_step_bytes, larulorn_prefill_flops),
-           "lolulorn": (lambda gpt2, size: lolulorn_config(gpt2), lolulorn_step_bytes, lolulorn_prefill_flops)}
-BESIDE = {"dopilorn": "mofulix", "larulorn": "mofulix", "lolulorn": "larulorn"}  # the engine's closest model, where that is not GPT-2
+           "lolulorn": (lambda gpt2, size: lolulorn_config(gpt2), lolulorn_step_bytes, lolulorn_prefill_flops),
+           "lafanex": (lambda gpt2, size: lafanex_config(gpt2), lafanex_step_bytes, lafanex_prefill_flops)}
+BESIDE = {"dopilorn": "mofulix", "larulorn": "mofulix", "lolulorn": "larulorn", "lafanex": "larulorn"}  # the engine's closest model, where that is not GPT-2
 
 
 def design_run(args):
@@ -805,9 +874,9 @@ def main():
     ap.add_argument("--link-floor", action="store_true", help="measure what one dependent kernel of a replayed graph costs at least")
     ap.add_argument("--phases", action="store_true", help="device milliseconds per phase of the forward pass (embed, attention, dense_ffn, lm_head) a decode step "
                     "and a prefill of 2,048 tokens, as the reference's command line prints them (tools/liyab_cli.cpp:198-211); steps run kernel by kernel, without graphs")
-    ap.add_argument("--design", default="", choices=["", "bokulix", "mofulix", "dopilorn", "larulorn", "lolulorn"],
+    ap.add_argument("--design", default="", choices=["", "bokulix", "mofulix", "dopilorn", "larulorn", "lolulorn", "lafanex"],
                     help="bokulix, mofulix: that design beside GPT-2 at equal layer sizes (prefill and decode, both with their rooflines); "
-                         "dopilorn, larulorn: beside Mofulix, lolulorn: beside Larulorn, the engine's closest model")
+                         "dopilorn, larulorn: beside Mofulix, lolulorn, lafanex: beside Larulorn, the engine's closest model")
     ap.add_argument("--design-only", action="store_true", help="with --design: skip the GPT-2 run (for profiling)")
     ap.add_argument("--design-sizes", default="small,medium,xl", help="the sizes --design runs (of small, medium, xl)")
     args = ap.parse_args()

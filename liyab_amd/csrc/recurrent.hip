@@ -643,6 +643,71 @@ conv_act_kernel(T* __restrict__ out, int64_t ldo, const float* __restrict__ in, 
     out[static_cast<int64_t>(t) * ldo + c] = from_float<T>(act ? silu_f(acc) : acc);
 }
 
+// The same for steps of many rows: a thread four channels side by side and CONV_TOKENS rows one after the other, which keeps the rows before a
+// row in registers and reads each once; only a row near its request's start looks into the ring (a branch the whole workgroup takes together).
+constexpr int CONV_TOKENS = 8;
+template <typename T, int TAPS>
+__global__ void __launch_bounds__(128)
+conv_act_rows_kernel(T* __restrict__ out, int64_t ldo, const float* __restrict__ in, int64_t ldi, const float* __restrict__ w,
+                     const float* __restrict__ bias, const float* __restrict__ state, int64_t state_stride, int n_slots,
+                     const int* __restrict__ tok_seq, const int* __restrict__ positions, const int* __restrict__ seq_starts,
+                     const int* __restrict__ state_slots, int n, int C, int act) {
+    const int c = (blockIdx.x * 128 + threadIdx.x) * 4;
+    if (c >= C) return;
+    const int t0 = blockIdx.y * CONV_TOKENS, t1 = min(t0 + CONV_TOKENS, n);
+    float wt[4][TAPS];
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) wt[e][j] = w[static_cast<int64_t>(c + e) * TAPS + j];
+    const f32x4_t b0 = bias != nullptr ? *reinterpret_cast<const f32x4_t*>(bias + c) : f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
+    // rows t0 - TAPS + 1 .. t1 - 1 of the step (one before the first: the first once more, never used)
+    f32x4_t x[CONV_TOKENS + TAPS - 1];
+#pragma unroll
+    for (int j = 0; j < CONV_TOKENS + TAPS - 1; ++j)
+        x[j] = *reinterpret_cast<const f32x4_t*>(in + static_cast<int64_t>(min(max(t0 - (TAPS - 1) + j, 0), n - 1)) * ldi + c);
+#pragma unroll
+    for (int k = 0; k < CONV_TOKENS; ++k) {
+        const int t = t0 + k;
+        if (t >= t1) break;
+        const int s = tok_seq[t], p = positions[t];
+        const int begin = seq_starts[s];
+        f32x4_t rows[TAPS];
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) rows[j] = x[k + j];
+        if (p < TAPS - 1 || t - (TAPS - 1) < begin) {
+            const int slot = state_slots[s];
+            const bool slot_ok = slot >= 0 && slot < n_slots;
+            const float* ring = state + static_cast<int64_t>(slot_ok ? slot : 0) * state_stride;
+#pragma unroll
+            for (int j = 0; j < TAPS - 1; ++j) {
+                const int back = TAPS - 1 - j, sp = p - back;
+                if (sp < 0) rows[j] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
+                else if (t - back < begin)
+                    rows[j] = slot_ok ? *reinterpret_cast<const f32x4_t*>(ring + static_cast<int64_t>(sp % (TAPS > 1 ? TAPS - 1 : 1)) * C + c) : f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
+            }
+        }
+        float v[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            float acc = b0[e];
+#pragma unroll
+            for (int j = 0; j < TAPS; ++j) acc = fmaf(wt[e][j], rows[j][e], acc);
+            v[e] = act ? silu_f(acc) : acc;
+        }
+        store4<T>(out + static_cast<int64_t>(t) * ldo + c, v);
+    }
+}
+
+template <typename T, typename... A>
+bool launch_conv_rows(int taps, dim3 grid, hipStream_t stream, A... args) {
+    if (taps == 2) conv_act_rows_kernel<T, 2><<<grid, 128, 0, stream>>>(args...);
+    else if (taps == 3) conv_act_rows_kernel<T, 3><<<grid, 128, 0, stream>>>(args...);
+    else if (taps == 4) conv_act_rows_kernel<T, 4><<<grid, 128, 0, stream>>>(args...);
+    else return false;
+    return true;
+}
+
 template <typename T>
 __global__ void __launch_bounds__(256)
 gated_group_norm_kernel(T* __restrict__ out, const float* __restrict__ y, int64_t ldy, const float* __restrict__ z, int64_t ldz,
@@ -821,6 +886,15 @@ extern "C" int liyab_conv_act(void* out, int out_dtype, int64_t ldo, const float
     LIYAB_REQUIRE(taps == 1 || (state != nullptr && n_slots > 0 && state_stride >= static_cast<int64_t>(taps - 1) * C),
                   "conv_act: %d taps need the last %d rows of a request in its slot", taps, taps - 1);
     if (n == 0) return 0;
+    const auto aligned = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+    if (n >= 64 && C % 4 == 0 && ldi % 4 == 0 && ldo % 4 == 0 && state_stride % 4 == 0 && aligned(in) && aligned(out) && aligned(bias) && aligned(state)) {
+        const dim3 rows((C / 4 + 127) / 128, (n + CONV_TOKENS - 1) / CONV_TOKENS);
+        const bool took = out_dtype == kF32
+            ? launch_conv_rows<float>(taps, rows, stream, static_cast<float*>(out), ldo, in, ldi, w, bias, state, state_stride, n_slots, tok_seq, positions, seq_starts, state_slots, n, C, act)
+            : out_dtype == kBF16 && launch_conv_rows<bf16_t>(taps, rows, stream, static_cast<bf16_t*>(out), ldo, in, ldi, w, bias, state, state_stride, n_slots, tok_seq, positions, seq_starts,
+                                                             state_slots, n, C, act);
+        if (took) return check_launch("conv_act");
+    }
     dim3 grid((C + 255) / 256, n);
     if (out_dtype == kF32)
         conv_act_kernel<float><<<grid, 256, 0, stream>>>(static_cast<float*>(out), ldo, in, ldi, w, bias, taps, state, state_stride, taps > 1 ? n_slots : 0, tok_seq,

@@ -28,6 +28,20 @@ constexpr float kLog2e = 1.4426950408889634f;
 
 __device__ __forceinline__ float ss_exp2(float v) { return __builtin_amdgcn_exp2f(v); }
 __device__ __forceinline__ float ss_softplus(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
+// The same for results that end in 16 bits: ln(1 + e), e = exp(-|z|) in (0, 1], as its series where e is small (1 + e rounds its digits away), by the
+// logarithm instruction elsewhere; within some units of 32-bit precision of the above.
+__device__ __forceinline__ float ss_softplus_fast(float z) {
+    const float e = ss_exp2(-fabsf(z) * kLog2e);
+    float s = fmaf(e, -0.125f, 1.0f / 7.0f);
+    s = fmaf(s, e, -1.0f / 6.0f);
+    s = fmaf(s, e, 0.2f);
+    s = fmaf(s, e, -0.25f);
+    s = fmaf(s, e, 1.0f / 3.0f);
+    s = fmaf(s, e, -0.5f);
+    s = fmaf(s, e, 1.0f) * e;
+    const float l = __builtin_amdgcn_logf(1.0f + e) * 0.6931471805599453f;
+    return fmaxf(z, 0.0f) + (e < 0.125f ? s : l);
+}
 __device__ __forceinline__ float ss_silu(float z) { return z / (1.0f + expf(-z)); }
 
 typedef __attribute__((ext_vector_type(8))) __bf16 ss_bf16x8;
@@ -85,7 +99,7 @@ scan_steps_mfma_kernel(float* __restrict__ dt, const float* __restrict__ low, in
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
         const int t = t0 + 8 * (r / 4) + 4 * (lane / 32) + r % 4;
-        if (t < n) dt[static_cast<int64_t>(t) * C + c] = ss_softplus(acc[r] + b);
+        if (t < n) dt[static_cast<int64_t>(t) * C + c] = ss_softplus_fast(acc[r] + b);
     }
 }
 
@@ -325,6 +339,18 @@ selective_single_kernel(SelectiveArgs a, const T* __restrict__ wt, const float* 
     const bool from_slot = slot_ok && pos > 0;
     const float* row = a.bc + t * a.ldb;  // [low | B | C]
     const float x = to_float<T>(static_cast<const T*>(a.x)[t * a.C + cc]);
+    // this wave's quarter of the states: the first four are asked for before anything is computed
+    const int nq = (a.N + 3) / 4, n0 = wave * nq, n1 = min(a.N, n0 + nq);
+    float S[4], A2[4];
+    auto states = [&](int i0) {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int64_t at = static_cast<int64_t>(min(i0 + j, a.N - 1)) * a.C + cc;
+            A2[j] = a.a2[at];
+            S[j] = base[at];
+        }
+    };
+    states(n0);
     // this wave's quarter of the rank; weights [rank, C], a row's channels side by side
     const int kq = (rank + 3) / 4, k1 = min(rank, (wave + 1) * kq);
     float acc = 0.0f;
@@ -342,16 +368,9 @@ selective_single_kernel(SelectiveArgs a, const T* __restrict__ wt, const float* 
     if (wave == 0) steps[lane] = ss_softplus((part[0][lane] + part[1][lane]) + (part[2][lane] + part[3][lane]) + bias[cc]);
     __syncthreads();
     const float dt = steps[lane], dx = dt * x;
-    const int nq = (a.N + 3) / 4, n0 = wave * nq, n1 = min(a.N, n0 + nq);
     float y = 0.0f;
-    for (int i0 = n0; i0 < n1; i0 += 4) {  // four states are asked for together
-        float S[4], A2[4];
-#pragma unroll
-        for (int j = 0; j < 4; ++j) {
-            const int64_t at = static_cast<int64_t>(min(i0 + j, n1 - 1)) * a.C + cc;
-            A2[j] = a.a2[at];
-            S[j] = base[at];
-        }
+    for (int i0 = n0; i0 < n1; i0 += 4) {
+        if (i0 > n0) states(i0);
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const int i = i0 + j;
