@@ -118,6 +118,134 @@ qk_prepare_kernel(const float* __restrict__ src, int64_t ld, int q_off, int k_of
     }
 }
 
+struct PrepareArgs {
+    const float* src;
+    int64_t ld;
+    int q_off, k_off, v_off, H, G, dk, dv, dk_out, dv_out;
+    void *q_out, *kc, *vc;
+    const int* slots;
+    int page_size, num_pages;
+    const float *q_norm, *k_norm;
+    float eps;
+    const double* freqs;
+    int rot_dims;
+    float temp_coef;
+    int temp_every;
+    const int* positions;
+    int rot_halves;
+    float rot_mag;
+    float* v_keep;
+    const float *v_first, *v_lam;
+};
+
+// The same for sizes in fours: a workgroup a token (or, in steps of few tokens, several, gridDim.y), the token's cosines and sines once for
+// all heads, L lanes a head with four of its entries each; the next head's entries are on their way while one is worked on. How a
+// row's bits come about does not depend on the grid.
+constexpr int QH_MAX_PAIRS = 128;
+template <typename T, int L>
+__global__ void __launch_bounds__(AS_THREADS)
+qk_prepare_heads_kernel(PrepareArgs a) {
+    __shared__ float turn_c[QH_MAX_PAIRS], turn_s[QH_MAX_PAIRS];
+    const int t = blockIdx.x, tid = threadIdx.x, l = tid % L;
+    constexpr int kSide = AS_THREADS / L;  // heads side by side
+    const int items = a.H + 2 * a.G, step = kSide * gridDim.y;
+    const float* row = a.src + static_cast<int64_t>(t) * a.ld;
+    const f32x4_t zero = {0.0f, 0.0f, 0.0f, 0.0f};
+    const int e = 4 * l;  // this lane's entries of a head
+    auto load = [&](int hh) {
+        const bool is_v = hh >= a.H + a.G;
+        const int width = is_v ? a.dv : a.dk, head = hh < a.H ? hh : hh < a.H + a.G ? hh - a.H : hh - a.H - a.G;
+        const int off = (hh < a.H ? a.q_off : is_v ? a.v_off : a.k_off) + head * width;
+        const f32x4_t v = *reinterpret_cast<const f32x4_t*>(row + off + min(e, width - 4));
+        return e < width ? v : zero;
+    };
+    int hh = blockIdx.y * kSide + tid / L;
+    f32x4_t next = load(min(hh, items - 1));
+    const int p = a.positions[t];
+    const int64_t slot = a.slots[t];
+    const bool stored = slot >= 0 && slot < static_cast<int64_t>(a.num_pages) * a.page_size;
+    for (int i = tid; i < a.rot_dims / 2; i += AS_THREADS) {
+        const float angle = turn_angle(p, a.freqs[i]);
+        turn_c[i] = cosf(angle) * a.rot_mag;
+        turn_s[i] = sinf(angle) * a.rot_mag;
+    }
+    const float temp = a.temp_every > 0 ? 1.0f + a.temp_coef * logf(static_cast<float>((p + 1) / a.temp_every) + 1.0f) : 1.0f;
+    __syncthreads();
+    for (; hh < items; hh += step) {
+        f32x4_t x = next;
+        next = load(min(hh + step, items - 1));
+        if (hh >= a.H + a.G) {
+            const int head = hh - a.H - a.G;
+            const int64_t at = (static_cast<int64_t>(t) * a.G + head) * a.dv + e;
+            if (e < a.dv) {
+                if (a.v_keep != nullptr) *reinterpret_cast<f32x4_t*>(a.v_keep + at) = x;
+                if (a.v_first != nullptr) {
+                    const float lam = a.v_lam[0];
+                    const f32x4_t f = *reinterpret_cast<const f32x4_t*>(a.v_first + at);
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) x[j] = (1.0f - lam) * x[j] + lam * f[j];
+                }
+            }
+            if (!stored || e >= a.dv_out) continue;
+            const float v[4] = {x[0], x[1], x[2], x[3]};
+            store4<T>(static_cast<T*>(a.vc) + (((slot / a.page_size) * a.G + head) * a.page_size + slot % a.page_size) * a.dv_out + e, v);
+            continue;
+        }
+        const bool is_q = hh < a.H;
+        const int head = is_q ? hh : hh - a.H;
+        const float* nw = is_q ? a.q_norm : a.k_norm;
+        float v[4] = {x[0], x[1], x[2], x[3]};
+        if (nw != nullptr) {
+            float ss = fmaf(v[3], v[3], fmaf(v[2], v[2], fmaf(v[1], v[1], v[0] * v[0])));
+            if constexpr (L == 64) ss = wave_sum(ss);
+            else ss = group_sum<L>(ss);
+            const float factor = 1.0f / sqrtf(ss / static_cast<float>(a.dk) + a.eps);
+            const f32x4_t w = *reinterpret_cast<const f32x4_t*>(nw + min(e, a.dk - 4));
+#pragma unroll
+            for (int j = 0; j < 4; ++j) v[j] *= factor * w[j];
+        }
+        if (a.rot_halves) {
+            // pairs (i, i + half), half a multiple of four: the partners are another lane's four entries
+            const int half = a.rot_dims / 2;
+            const bool first = e < half, turned = e < a.rot_dims;
+            const int partner = turned ? (first ? l + half / 4 : l - half / 4) : l;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const float o = __shfl(v[j], partner, L);
+                const int i = min(first ? e + j : e - half + j, QH_MAX_PAIRS - 1);
+                if (turned) v[j] = first ? v[j] * turn_c[i] - o * turn_s[i] : v[j] * turn_c[i] + o * turn_s[i];
+            }
+        } else {
+#pragma unroll
+            for (int j = 0; j < 4; j += 2) {
+                if (e + j + 1 < a.rot_dims) {
+                    const float c = turn_c[(e + j) / 2], s = turn_s[(e + j) / 2], u = v[j];
+                    v[j] = u * c - v[j + 1] * s;
+                    v[j + 1] = v[j + 1] * c + u * s;
+                }
+            }
+        }
+        if (is_q && a.temp_every > 0)
+#pragma unroll
+            for (int j = 0; j < 4; ++j) v[j] *= temp;
+        if (e >= a.dk_out || (!is_q && !stored)) continue;
+        T* dst = is_q ? static_cast<T*>(a.q_out) + (static_cast<int64_t>(t) * a.H + head) * a.dk_out
+                      : static_cast<T*>(a.kc) + (((slot / a.page_size) * a.G + head) * a.page_size + slot % a.page_size) * a.dk_out;
+        store4<T>(dst + e, v);
+    }
+}
+
+template <typename T>
+void launch_prepare_heads(const PrepareArgs& a, int n, hipStream_t stream) {
+    const int lanes = (a.dk_out > a.dv_out ? a.dk_out : a.dv_out) / 4, items = a.H + 2 * a.G;
+    const int L = lanes <= 8 ? 8 : lanes <= 16 ? 16 : lanes <= 32 ? 32 : 64, side = AS_THREADS / L;
+    const dim3 grid(n, n >= 256 ? 1 : (items + side - 1) / side);
+    if (L == 8) qk_prepare_heads_kernel<T, 8><<<grid, AS_THREADS, 0, stream>>>(a);
+    else if (L == 16) qk_prepare_heads_kernel<T, 16><<<grid, AS_THREADS, 0, stream>>>(a);
+    else if (L == 32) qk_prepare_heads_kernel<T, 32><<<grid, AS_THREADS, 0, stream>>>(a);
+    else qk_prepare_heads_kernel<T, 64><<<grid, AS_THREADS, 0, stream>>>(a);
+}
+
 constexpr int QR_MAX_PAIRS = 256;  // turned pairs of a head (heads of up to 512)
 
 template <typename T>
@@ -305,6 +433,16 @@ extern "C" int liyab_qk_prepare(const float* src, int64_t ld, int q_off, int k_o
     LIYAB_REQUIRE(temp_every >= 0, "qk_prepare: bad query factor");
     LIYAB_REQUIRE((v_first == nullptr) == (v_lam == nullptr) && !(v_keep != nullptr && v_first != nullptr), "qk_prepare: values are kept, or mixed with kept ones and a rate");
     if (n == 0) return 0;
+    const auto aligned = [](const void* p, uintptr_t to) { return (reinterpret_cast<uintptr_t>(p) & (to - 1)) == 0; };
+    if ((ld | q_off | k_off | v_off | dk | dv | dk_out | dv_out) % 4 == 0 && dk_out <= 256 && dv_out <= 256 && (!rot_halves || rot_dims % 8 == 0) && aligned(src, 16) &&
+        aligned(q_out, 16) && aligned(kc, 16) && aligned(vc, 16) && aligned(q_norm, 16) && aligned(k_norm, 16) && aligned(v_keep, 16) && aligned(v_first, 16) &&
+        (dtype == kF32 || dtype == kBF16)) {
+        const PrepareArgs a{src, ld, q_off, k_off, v_off, H, G, dk, dv, dk_out, dv_out, q_out, kc, vc, slots, page_size, num_pages, q_norm, k_norm, eps, freqs, rot_dims,
+                            temp_coef, temp_every, positions, rot_halves, rot_mag, v_keep, v_first, v_lam};
+        if (dtype == kF32) launch_prepare_heads<float>(a, n, stream);
+        else launch_prepare_heads<bf16_t>(a, n, stream);
+        return check_launch("qk_prepare");
+    }
     dim3 grid(n, H + 2 * G);
     const double* fr = rot_dims > 0 ? freqs : nullptr;
     if (dtype == kF32)
