@@ -198,7 +198,8 @@ int liyab_lru_scan(void* out, int out_dtype, const float* z, int64_t ldz, const 
 int liyab_streams_update(float* x, const float* enter, const float* y, int n_sum, const int* ids, const float* weights, int n_ids, const void* h,
                          const float* mix, const float* add, const float* in, const float* w, float eps, void* out, int out_dtype, const int* rows,
                          int n, int S, int d, hipStream_t stream);
-int liyab_scan_steps(float* dt, const float* low, int64_t ldl, const void* w, int dtype, const float* bias, int n, int C, int rank, hipStream_t stream);
+int liyab_scan_steps(float* dt, const float* low, int64_t ldl, const void* w, int ldw, int dtype, const float* bias, int n, int C, int rank,
+                     hipStream_t stream);
 int liyab_selective_scan(void* out, int dtype, const void* x, const float* dt, const float* bc, int64_t ldb, const float* z, int64_t ldz,
                          const float* a2, const float* skip, float* state, int64_t state_stride, int n_slots, const float* raw, int64_t ldr, int places,
                          const int* seq_starts, const int* positions, const int* state_slots, int n_seqs, int C, int N, int seg_tokens, int max_segs,

@@ -191,6 +191,37 @@ __device__ __forceinline__ void route_wave(const float* __restrict__ z, const Ro
     }
 }
 
+// The same for one group of at most 64 outputs: an output a lane, its score in a register; zl is the lane's logit, and with `extra` lane 0 knows the
+// token's own one. No trip through LDS.
+__device__ __forceinline__ void route_wave_lane(float zl, float own, const RouteArgs& ra, int E, int top, int* __restrict__ ids, float* __restrict__ weights) {
+    const int lane = threadIdx.x % kWave;
+    const bool real = lane < E;
+    float s;
+    if (ra.mode == 3) {
+        const float v = real ? expf(zl - wave_max(real ? zl : -INFINITY)) : 0.0f;
+        s = v * (1.0f / wave_sum(v));
+    } else {
+        s = 1.0f / (1.0f + expf(-zl));
+    }
+    float c = real ? s + (ra.correction != nullptr ? ra.correction[lane] : 0.0f) : -INFINITY;
+    for (int k = 0; k < top; ++k) {
+        float bv = c;
+        int bi = real ? lane : kWave + lane;
+        wave_argmax(bv, bi);
+        const int best = min(bi, E - 1);
+        if (lane == best) {
+            ids[k] = best < ra.n_listed ? best : -1;
+            weights[k] = s * ra.scale;
+            c = -INFINITY;
+        }
+    }
+    if (ra.extra && lane == 0) {
+        ids[top] = ra.n_listed;
+        weights[top] = 1.0f / (1.0f + expf(-own));
+    }
+}
+__device__ __forceinline__ bool routes_in_lanes(const RouteArgs& ra, int E) { return E <= kWave && ra.keep == ra.n_groups; }
+
 // a wave a token, four waves a workgroup
 __global__ void __launch_bounds__(256)
 moe_route_wave_kernel(const float* __restrict__ logits, int64_t ld, RouteArgs ra, int n, int E, int top, int* __restrict__ ids, float* __restrict__ weights) {
@@ -198,6 +229,11 @@ moe_route_wave_kernel(const float* __restrict__ logits, int64_t ld, RouteArgs ra
     const int wave = threadIdx.x / kWave, t = blockIdx.x * 4 + wave;
     if (t >= n) return;
     const int64_t at = static_cast<int64_t>(t) * (top + ra.extra);
+    if (routes_in_lanes(ra, E)) {
+        const float* z = logits + static_cast<int64_t>(t) * ld;
+        route_wave_lane(z[min(static_cast<int>(threadIdx.x) % kWave, E - 1)], z[ra.extra ? E : 0], ra, E, top, ids + at, weights + at);
+        return;
+    }
     route_wave(logits + static_cast<int64_t>(t) * ld, ra, E, top, ids + at, weights + at, reinterpret_cast<float*>(sh) + wave * E);
 }
 
@@ -267,7 +303,22 @@ moe_route_align_kernel(const float* __restrict__ logits, int64_t ld, int n, int 
     const int t = threadIdx.x;
     if (ra.mode >= 2) {  // a wave a token, sixteen at a time
         const int wave = t / kWave;
-        for (int i = wave; i < n; i += 1024 / kWave) {
+        if (routes_in_lanes(ra, E)) {
+            constexpr int kEach = kWaveRouteTokens / (1024 / kWave);  // tokens a wave: all their logits are asked for together
+            float zl[kEach], own[kEach];
+#pragma unroll
+            for (int j = 0; j < kEach; ++j) {
+                const float* z = logits + static_cast<int64_t>(min(wave + j * (1024 / kWave), n - 1)) * ld;
+                zl[j] = z[min(t % kWave, E - 1)];
+                own[j] = z[ra.extra ? E : 0];
+            }
+#pragma unroll
+            for (int j = 0; j < kEach; ++j) {
+                const int i = wave + j * (1024 / kWave);
+                const int64_t at = static_cast<int64_t>(i) * (top + ra.extra);
+                if (i < n) route_wave_lane(zl[j], own[j], ra, E, top, ids + at, weights + at);
+            }
+        } else for (int i = wave; i < n; i += 1024 / kWave) {
             const int64_t at = static_cast<int64_t>(i) * (top + ra.extra);
             route_wave(logits + static_cast<int64_t>(i) * ld, ra, E, top, ids + at, weights + at, reinterpret_cast<float*>(sh) + wave * E);
         }

@@ -666,12 +666,19 @@ conv_act_rows_kernel(T* __restrict__ out, int64_t ldo, const float* __restrict__
 #pragma unroll
     for (int j = 0; j < CONV_TOKENS + TAPS - 1; ++j)
         x[j] = *reinterpret_cast<const f32x4_t*>(in + static_cast<int64_t>(min(max(t0 - (TAPS - 1) + j, 0), n - 1)) * ldi + c);
+    int seq[CONV_TOKENS], pos[CONV_TOKENS], start[CONV_TOKENS];  // (all asked for together)
+#pragma unroll
+    for (int k = 0; k < CONV_TOKENS; ++k) {
+        seq[k] = tok_seq[min(t0 + k, n - 1)];
+        pos[k] = positions[min(t0 + k, n - 1)];
+    }
+#pragma unroll
+    for (int k = 0; k < CONV_TOKENS; ++k) start[k] = seq_starts[seq[k]];
 #pragma unroll
     for (int k = 0; k < CONV_TOKENS; ++k) {
         const int t = t0 + k;
         if (t >= t1) break;
-        const int s = tok_seq[t], p = positions[t];
-        const int begin = seq_starts[s];
+        const int s = seq[k], p = pos[k], begin = start[k];
         f32x4_t rows[TAPS];
 #pragma unroll
         for (int j = 0; j < TAPS; ++j) rows[j] = x[k + j];

@@ -9,8 +9,8 @@
 //   registers; a token's B and C are staged through LDS sixteen tokens at a time, x, dt and z are asked for eight tokens ahead. phase 0: a request's whole portion
 //   by one wave. Long portions in segments side by side instead, in three launches: phase 1, every segment from zero for its end
 //   state and the sum of its dt (the product of a segment's decays is exp(A sum dt)); phase 2, the segments of a
-//   request strung together, which leaves each the state it starts from; phase 3, every segment again from that state, with
-//   outputs. The grids follow from the step's rows and requests alone.
+//   request strung together, which leaves the true state behind each; phase 3, every segment again from the state behind the one before it (a
+//   request's first one from its slot), with outputs. The grids follow from the step's rows and requests alone.
 // liyab_selective_single: a step of single tokens, step sizes included, in one kernel: four waves a (request, 64 channels), each with a
 //   quarter of the rank and a quarter of the states.
 //
@@ -48,46 +48,30 @@ typedef __attribute__((ext_vector_type(8))) __bf16 ss_bf16x8;
 typedef __attribute__((ext_vector_type(16))) float ss_floatx16;
 typedef __attribute__((ext_vector_type(4))) uint32_t ss_u32x4;
 
-// a wave 32 tokens x 32 channels, straight from global memory; A: lane's row li, k 8 (lane / 32) .. + 7 of each 16
-template <bool VEC>
+// a wave 32 tokens x 32 channels, straight from global memory in pieces of eight k; A: lane's row li, k 8 (lane / 32) .. + 7 of each 16. The
+// weights' rows are ldw long, a multiple of 8, zeros behind the rank; what low holds behind its rank is read and masked.
 __global__ void __launch_bounds__(256)
-scan_steps_mfma_kernel(float* __restrict__ dt, const float* __restrict__ low, int64_t ldl, const bf16_t* __restrict__ w, const float* __restrict__ bias,
+scan_steps_mfma_kernel(float* __restrict__ dt, const float* __restrict__ low, int64_t ldl, const bf16_t* __restrict__ w, int ldw, const float* __restrict__ bias,
                        int n, int C, int rank) {
     const int lane = threadIdx.x % 64, wave = threadIdx.x / 64;
     const int li = lane % 32, lk = (lane / 32) * 8;
     const int t0 = (blockIdx.y * 4 + wave) * 32, c0 = blockIdx.x * 32;
     if (t0 >= n) return;
     const float* lrow = low + static_cast<int64_t>(min(t0 + li, n - 1)) * ldl;
-    const bf16_t* wrow = w + static_cast<int64_t>(min(c0 + li, C - 1)) * rank;
+    const bf16_t* wrow = w + static_cast<int64_t>(min(c0 + li, C - 1)) * ldw;
     ss_floatx16 acc;
 #pragma unroll
     for (int r = 0; r < 16; ++r) acc[r] = 0.0f;
     for (int k0 = 0; k0 < rank; k0 += 16) {
-        float v[8];
         union { ss_bf16x8 v; ss_u32x4 u; bf16_t e[8]; } fw, hi, lo;
-        if constexpr (VEC) {  // (rank a multiple of 8: a piece lies inside the row or past it)
-            const int k = min(k0 + lk, rank - 8);
-            const bool in = k0 + lk < rank;
-            const f32x4_t a = *reinterpret_cast<const f32x4_t*>(lrow + k), b = *reinterpret_cast<const f32x4_t*>(lrow + k + 4);
-            fw.u = *reinterpret_cast<const ss_u32x4*>(wrow + k);
-#pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                v[e] = in ? a[e] : 0.0f;
-                v[4 + e] = in ? b[e] : 0.0f;
-            }
-        } else {
-#pragma unroll
-            for (int e = 0; e < 8; ++e) {
-                const int k = min(k0 + lk + e, rank - 1);
-                const float x = lrow[k];
-                fw.e[e] = wrow[k];
-                v[e] = k0 + lk + e < rank ? x : 0.0f;
-            }
-        }
+        const int k = min(k0 + lk, ldw - 8);  // (a piece past the last one: the last one, masked)
+        const f32x4_t a = *reinterpret_cast<const f32x4_t*>(lrow + k), b = *reinterpret_cast<const f32x4_t*>(lrow + k + 4);
+        fw.u = *reinterpret_cast<const ss_u32x4*>(wrow + k);
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
-            hi.e[e] = float_to_bf16(v[e]);
-            lo.e[e] = float_to_bf16(v[e] - bf16_to_float(hi.e[e]));
+            const float v = k0 + lk + e < rank ? (e < 4 ? a[e] : b[e - 4]) : 0.0f;
+            hi.e[e] = float_to_bf16(v);
+            lo.e[e] = float_to_bf16(v - bf16_to_float(hi.e[e]));
         }
         acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(hi.v, fw.v, acc, 0, 0, 0);
         acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(lo.v, fw.v, acc, 0, 0, 0);
@@ -104,12 +88,12 @@ scan_steps_mfma_kernel(float* __restrict__ dt, const float* __restrict__ low, in
 }
 
 __global__ void __launch_bounds__(256)
-scan_steps_plain_kernel(float* __restrict__ dt, const float* __restrict__ low, int64_t ldl, const float* __restrict__ w, const float* __restrict__ bias,
-                        int C, int rank) {
+scan_steps_plain_kernel(float* __restrict__ dt, const float* __restrict__ low, int64_t ldl, const float* __restrict__ w, int ldw,
+                        const float* __restrict__ bias, int C, int rank) {
     const int t = blockIdx.y, c = blockIdx.x * 256 + threadIdx.x;
     if (c >= C) return;
     const float* lrow = low + static_cast<int64_t>(t) * ldl;
-    const float* wrow = w + static_cast<int64_t>(c) * rank;
+    const float* wrow = w + static_cast<int64_t>(c) * ldw;
     float acc = 0.0f;
     for (int k = 0; k < rank; ++k) acc = fmaf(lrow[k], wrow[k], acc);
     dt[static_cast<int64_t>(t) * C + c] = ss_softplus(acc + bias[c]);
@@ -216,6 +200,35 @@ __device__ __forceinline__ float ss_walk(const SelectiveArgs& a, float (&S)[NREG
     return sum_dt;
 }
 
+// Segment g of a step in the order of its requests, found by a wave: its request s, the request's rows, and which of the request's segments it is; a lane
+// a request, the running sum over the lanes. False past the last segment.
+__device__ __forceinline__ bool ss_find(const int* __restrict__ seq_starts, int n_seqs, int seg_tokens, int g, int& s, int& begin, int& end, int& local) {
+    const int lane = threadIdx.x % kWave;
+    int before = 0;
+    for (int base = 0; base < n_seqs; base += kWave) {
+        const int i = min(base + lane, n_seqs - 1);
+        const int b = seq_starts[i], e = seq_starts[i + 1];
+        const int count = base + lane < n_seqs ? (e - b + seg_tokens - 1) / seg_tokens : 0;
+        int sum = count;
+#pragma unroll
+        for (int o = 1; o < kWave; o *= 2) {
+            const int v = __shfl_up(sum, o, kWave);
+            if (lane >= o) sum += v;
+        }
+        const uint64_t past = __ballot(before + sum > g);
+        if (past != 0) {
+            const int l = __builtin_ctzll(past);
+            s = base + l;
+            begin = __builtin_amdgcn_readlane(b, l);
+            end = __builtin_amdgcn_readlane(e, l);
+            local = g - before - (__builtin_amdgcn_readlane(sum, l) - __builtin_amdgcn_readlane(count, l));
+            return true;
+        }
+        before += __builtin_amdgcn_readlane(sum, kWave - 1);
+    }
+    return false;
+}
+
 template <typename T, int NREG, int PHASE>
 __global__ void __launch_bounds__(64)
 selective_scan_kernel(SelectiveArgs a) {
@@ -232,30 +245,19 @@ selective_scan_kernel(SelectiveArgs a) {
         end = t1 = a.seq_starts[s + 1];
         if (end <= begin) return;
     } else {
-        // segment blockIdx.y in the order of the requests: which request's, and which of its segments (a workgroup past the last exits)
-        int g = blockIdx.y;
-        begin = end = 0;
-        bool found = false;
-        for (s = 0; s < a.n_seqs; ++s) {
-            begin = a.seq_starts[s];
-            end = a.seq_starts[s + 1];
-            const int n_seg = (end - begin + a.seg_tokens - 1) / a.seg_tokens;
-            if (g < n_seg) {
-                t0 = begin + g * a.seg_tokens;
-                t1 = min(t0 + a.seg_tokens, end);
-                last = g == n_seg - 1;
-                found = true;
-                break;
-            }
-            g -= n_seg;
-        }
-        if (!found || (PHASE == 1 && last)) return;  // (nobody needs the end state of a request's last segment from zero)
+        int g;
+        if (!ss_find(a.seq_starts, a.n_seqs, a.seg_tokens, blockIdx.y, s, begin, end, g)) return;  // a workgroup past the last segment
+        t0 = begin + g * a.seg_tokens;
+        t1 = min(t0 + a.seg_tokens, end);
+        last = t1 == end;
+        if (PHASE == 1 && last) return;  // (nobody needs the end state of a request's last segment from zero)
     }
     const int slot = a.state_slots[s];
     const bool slot_ok = slot >= 0 && slot < a.n_slots;
     float* base = a.state + static_cast<int64_t>(slot_ok ? slot : 0) * a.state_stride;
     float* seg = a.seg_state + static_cast<int64_t>(blockIdx.y) * a.N * a.C;  // (read or written in phases 1 and 3 only)
-    const bool from_slot = PHASE == 0 && slot_ok && a.positions[begin] > 0;
+    const bool first = PHASE != 1 && t0 == begin;  // starts from the request's own state
+    const bool from_slot = first && slot_ok && a.positions[begin] > 0;
     float S[NREG], A2[NREG];
 #pragma unroll
     for (int i = 0; i < NREG; ++i) {
@@ -263,8 +265,8 @@ selective_scan_kernel(SelectiveArgs a) {
         A2[i] = a.a2[static_cast<int64_t>(min(i, a.N - 1)) * a.C + cc];
         S[i] = 0.0f;
     }
-    if (PHASE == 3 || from_slot) {
-        const float* src = PHASE == 3 ? seg : base;
+    if ((PHASE == 3 && !first) || from_slot) {
+        const float* src = first ? base : seg - static_cast<int64_t>(a.N) * a.C;  // (the segment before holds the state behind it)
 #pragma unroll
         for (int i = 0; i < NREG; ++i) S[i] = src[static_cast<int64_t>(min(i, a.N - 1)) * a.C + cc];
     }
@@ -283,39 +285,41 @@ selective_scan_kernel(SelectiveArgs a) {
     }
 }
 
-// phase 2: a thread a (channel, state) of a request strings its segments together; eight segments' ends are asked for together
+// phase 2: a thread a (channel, state) of a request strings its segments together, where it has more than one; eight segments' ends are asked for together
 __global__ void __launch_bounds__(256)
 selective_combine_kernel(SelectiveArgs a) {
+    const int s = blockIdx.y, begin = a.seq_starts[s];
+    const int n_seg = (a.seq_starts[s + 1] - begin + a.seg_tokens - 1) / a.seg_tokens;
+    if (n_seg <= 1) return;  // (its only segment starts from the slot)
+    // the segments of the requests before this one, a lane a request
+    int g0 = 0;
+    for (int i = threadIdx.x % kWave; i < s; i += kWave) g0 += (a.seq_starts[i + 1] - a.seq_starts[i] + a.seg_tokens - 1) / a.seg_tokens;
+#pragma unroll
+    for (int o = 1; o < kWave; o *= 2) g0 += __shfl_xor(g0, o, kWave);
     const int64_t e = static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x;
     const int64_t NC = static_cast<int64_t>(a.N) * a.C;
     if (e >= NC) return;
-    int g0 = 0, n_seg = 0;
-    for (int s = 0; s <= static_cast<int>(blockIdx.y); ++s) {
-        g0 += n_seg;
-        n_seg = (a.seq_starts[s + 1] - a.seq_starts[s] + a.seg_tokens - 1) / a.seg_tokens;
-    }
-    if (n_seg == 0) return;
-    const int s = blockIdx.y, slot = a.state_slots[s], c = static_cast<int>(e % a.C);
+    const int slot = a.state_slots[s], c = static_cast<int>(e % a.C);
     const bool slot_ok = slot >= 0 && slot < a.n_slots;
-    float S = (slot_ok && a.positions[a.seq_starts[s]] > 0) ? a.state[static_cast<int64_t>(slot) * a.state_stride + e] : 0.0f;
+    float S = (slot_ok && a.positions[begin] > 0) ? a.state[static_cast<int64_t>(slot) * a.state_stride + e] : 0.0f;
     const float a2 = a.a2[e];
     float* st = a.seg_state + g0 * NC + e;
     const float* sd = a.seg_dt + static_cast<int64_t>(g0) * a.C + c;
-    for (int g = 0; g < n_seg; g += 8) {
+    for (int g = 0; g < n_seg - 1; g += 8) {
         float end[8], sum[8];
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
-            const int64_t gg = min(g + j, n_seg - 1);
-            end[j] = st[gg * NC];  // (the last segment's is not written and not used)
+            const int64_t gg = min(g + j, n_seg - 2);  // (the last segment's end is not written and not used)
+            end[j] = st[gg * NC];
             sum[j] = sd[gg * a.C];
         }
         settle_loads(end);
         settle_loads(sum);
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
-            if (g + j < n_seg) {
+            if (g + j < n_seg - 1) {
+                S = fmaf(ss_exp2(sum[j] * a2), S, end[j]);
                 st[(g + j) * NC] = S;
-                if (g + j < n_seg - 1) S = fmaf(ss_exp2(sum[j] * a2), S, end[j]);
             }
         }
     }
@@ -414,21 +418,20 @@ using namespace liyab;
 
 constexpr int kMaxScanStates = 128;
 
-// dt: float [n, C]; low: float rows [n, ldl], `rank` of them read; w [C, rank] in `dtype`; bias: float [C].
-extern "C" int liyab_scan_steps(float* dt, const float* low, int64_t ldl, const void* w, int dtype, const float* bias, int n, int C, int rank,
+// dt: float [n, C]; low: float rows [n, ldl], `rank` of them used; w: rows of ldw in `dtype`, the first `rank` of [C, ldw] used, for bfloat16 zeros behind them
+// and ldw a multiple of 8 that ldl (a multiple of 4) holds; bias: float [C].
+extern "C" int liyab_scan_steps(float* dt, const float* low, int64_t ldl, const void* w, int ldw, int dtype, const float* bias, int n, int C, int rank,
                                 hipStream_t stream) {
     LIYAB_REQUIRE(dt && low && w && bias, "scan_steps: null pointer");
-    LIYAB_REQUIRE(n >= 0 && n <= 65535 && C > 0 && rank > 0 && ldl >= rank, "scan_steps: bad sizes n=%d C=%d rank=%d", n, C, rank);
+    LIYAB_REQUIRE(n >= 0 && n <= 65535 && C > 0 && rank > 0 && ldl >= rank && ldw >= rank, "scan_steps: bad sizes n=%d C=%d rank=%d", n, C, rank);
     LIYAB_REQUIRE(dtype == kF32 || dtype == kBF16, "scan_steps: unknown dtype %d", dtype);
+    LIYAB_REQUIRE(dtype == kF32 || (ldw % 8 == 0 && ldl % 4 == 0 && ldl >= ldw && (reinterpret_cast<uintptr_t>(low) & 15) == 0 && (reinterpret_cast<uintptr_t>(w) & 15) == 0),
+                  "scan_steps: rows of %lld floats and weights of %d a row are not taken in 16-byte pieces", static_cast<long long>(ldl), ldw);
     if (n == 0) return 0;
-    if (dtype == kF32) {
-        scan_steps_plain_kernel<<<dim3((C + 255) / 256, n), 256, 0, stream>>>(dt, low, ldl, static_cast<const float*>(w), bias, C, rank);
-    } else {
-        const dim3 grid((C + 31) / 32, (n + 127) / 128);
-        const bool vec = rank % 8 == 0 && ldl % 4 == 0 && (reinterpret_cast<uintptr_t>(low) & 15) == 0 && (reinterpret_cast<uintptr_t>(w) & 15) == 0;
-        if (vec) scan_steps_mfma_kernel<true><<<grid, 256, 0, stream>>>(dt, low, ldl, static_cast<const bf16_t*>(w), bias, n, C, rank);
-        else scan_steps_mfma_kernel<false><<<grid, 256, 0, stream>>>(dt, low, ldl, static_cast<const bf16_t*>(w), bias, n, C, rank);
-    }
+    if (dtype == kF32)
+        scan_steps_plain_kernel<<<dim3((C + 255) / 256, n), 256, 0, stream>>>(dt, low, ldl, static_cast<const float*>(w), ldw, bias, C, rank);
+    else
+        scan_steps_mfma_kernel<<<dim3((C + 31) / 32, (n + 127) / 128), 256, 0, stream>>>(dt, low, ldl, static_cast<const bf16_t*>(w), ldw, bias, n, C, rank);
     return check_launch("scan_steps");
 }
 

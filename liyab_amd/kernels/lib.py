@@ -134,7 +134,7 @@ _SIGNATURES = {
     "liyab_lru_scan": [P, c_int, P, c_int64, P, P, P, P, P, P, c_float, c_float, P, c_int64, P, c_int64, c_int, P, c_int64, c_int, P, P, P, c_int, c_int,
                        c_int, c_int, P],
     "liyab_streams_update": [P, P, P, c_int, P, P, c_int, P, P, P, P, P, c_float, P, c_int, P, c_int, c_int, c_int, P],
-    "liyab_scan_steps": [P, P, c_int64, P, c_int, P, c_int, c_int, c_int, P],
+    "liyab_scan_steps": [P, P, c_int64, P, c_int, c_int, P, c_int, c_int, c_int, P],
     "liyab_selective_scan": [P, c_int, P, P, P, c_int64, P, c_int64, P, P, P, c_int64, c_int, P, c_int64, c_int, P, P, P, c_int, c_int, c_int, c_int,
                              c_int, P, P, P],
     "liyab_selective_single": [P, c_int, P, P, c_int64, c_int, P, P, P, c_int64, P, P, P, c_int64, c_int, P, c_int64, c_int, P, P, P, c_int, c_int,

@@ -2254,22 +2254,23 @@ def selective_segments(n: int, n_seqs: int, channels: int):
 def selective_scan(out: torch.Tensor, x: torch.Tensor, low: torch.Tensor, z: torch.Tensor, dt_weight: torch.Tensor, dt_weight_t: torch.Tensor, dt_bias: torch.Tensor,
                    a2: torch.Tensor, skip: torch.Tensor, state: StateSlice, raw: torch.Tensor, taps: int, ctx) -> None:
     """S[c, n] <- exp2(dt_c a2[n, c]) S[c, n] + dt_c x_c B_n, out_c = (sum_n S[c, n] C_n + skip_c x_c) silu(z_c) along each request's rows of the step, with
-    dt = softplus(low . dt_weight^T + dt_bias). x, out contiguous [n, C] in the compute dtype; low float32 rows [n, rank + 2 N] = [low | B | C]; z float32 rows
-    [n, C]; dt_weight [C, rank] and once more as dt_weight_t [rank, C] in the compute dtype; a2 float32 [N, C] = A log2(e). `state`: S [N, C] and behind it the last
+    dt = softplus(low . dt_weight^T + dt_bias). x, out contiguous [n, C] in the compute dtype; low float32 rows [n, rank + 2 N] = [low | B | C], in bfloat16 runs
+    of a stride that is a multiple of 4 and as long as dt_weight's rows; z float32 rows [n, C]; dt_weight_t [rank, C] in the compute dtype, and once more as dt_weight
+    [C, >= rank], in bfloat16 rows of a multiple of 8 with zeros behind the rank; a2 float32 [N, C] = A log2(e). `state`: S [N, C] and behind it the last
     taps - 1 rows of `raw` (float32 rows [n, C]), position p at ring place p % (taps - 1). S starts from zero at position 0."""
     _dev(out, "out")
     _dev(x, "x")
     n, C = x.shape
-    N, rank = a2.shape[0], dt_weight.shape[1]
+    N, rank = a2.shape[0], dt_weight_t.shape[0]
     ldb, ldz, ldr = _rows(low, "low"), _rows(z, "z"), _rows(raw, "raw")
     if tuple(out.shape) != (n, C) or out.dtype != x.dtype or not out.is_contiguous() or not x.is_contiguous() or ctx.n_tokens != n:
         raise KernelError("selective_scan: x and out must be the step's contiguous rows of one shape and dtype")
     if any(t.dtype != torch.float32 for t in (low, z, raw)) or tuple(low.shape) != (n, rank + 2 * N) or tuple(z.shape) != (n, C) or tuple(raw.shape) != (n, C):
         raise KernelError(f"selective_scan: low [{n}, {rank + 2 * N}], z and raw [{n}, {C}] must be float32 rows")
-    for w, shape in ((dt_weight, (C, rank)), (dt_weight_t, (rank, C))):
+    for w, fits in ((dt_weight, dt_weight.shape[0] == C and dt_weight.shape[1] >= rank), (dt_weight_t, dt_weight_t.shape[1] == C)):
         _dev(w, "dt_weight")
-        if w.dtype != x.dtype or tuple(w.shape) != shape or not w.is_contiguous():
-            raise KernelError(f"selective_scan: the step sizes' weights must be contiguous {shape} in x's dtype, got {tuple(w.shape)} {w.dtype}")
+        if w.dtype != x.dtype or w.dim() != 2 or not fits or not w.is_contiguous():
+            raise KernelError(f"selective_scan: the step sizes' weights must be contiguous [{C}, >= {rank}] and [{rank}, {C}] in x's dtype, got {tuple(w.shape)} {w.dtype}")
     if not 1 <= N <= SELECTIVE_MAX_STATES or taps < 1 or state.size != (N + taps - 1) * C:
         raise KernelError(f"selective_scan: {N} states (up to {SELECTIVE_MAX_STATES}), {taps} taps, a slot of {state.size} floats")
     _f32vec(dt_bias, "dt_bias", C)
@@ -2283,7 +2284,7 @@ def selective_scan(out: torch.Tensor, x: torch.Tensor, low: torch.Tensor, z: tor
                   a2.data_ptr(), skip.data_ptr(), *kept, *lists, C, N, _stream())
         return
     dt = ctx.workspace.get("selective_dt", (n, C), torch.float32)
-    _lib.call("liyab_scan_steps", dt.data_ptr(), low.data_ptr(), ldb, dt_weight.data_ptr(), code, dt_bias.data_ptr(), n, C, rank, _stream())
+    _lib.call("liyab_scan_steps", dt.data_ptr(), low.data_ptr(), ldb, dt_weight.data_ptr(), dt_weight.shape[1], code, dt_bias.data_ptr(), n, C, rank, _stream())
     tokens, most = selective_segments(n, ctx.n_seqs, C)
     ends = sums = None
     if tokens:

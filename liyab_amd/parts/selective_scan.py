@@ -40,9 +40,11 @@ class SelectiveScan:
         self.conv = store.fetch(t["conv"], (W, self.taps), "vector")
         self.conv_bias = store.fetch(t["conv_bias"], (W,), "vector")
         self.x_weight = store.fetch(t["x"], (R + 2 * N, W), "matrix")
-        self.dt_weight = store.fetch(t["dt"], (W, R), "matrix")
-        # [rank, channels]: a row's channels side by side, as a step of single tokens reads them
-        self.dt_weight_t = store.derived(("rank_first", t["dt"].name), lambda: self.dt_weight.t().contiguous())
+        dt = store.fetch(t["dt"], (W, R), "matrix")
+        # [rank, channels]: a row's channels side by side, as a step of single tokens reads them; and rows of a multiple of eight
+        self.dt_weight_t = store.derived(("rank_first", t["dt"].name), lambda: dt.t().contiguous())
+        self.dt_weight = store.derived(("rows_of_eights", t["dt"].name), lambda: torch.nn.functional.pad(dt, (0, -R % 8)).contiguous())
+        self.low_stride = -(-max(R + 2 * N, self.dt_weight.shape[1]) // 4) * 4
         self.dt_bias = store.fetch(t["dt_bias"], (W,), "vector")
         a_log = store.fetch(t["A_log"], (W, N), "vector")
         # [states, channels], times log2(e): a decay is 2^(dt a)
@@ -71,7 +73,7 @@ class SelectiveScan:
         raw, z = proj[:, :W], proj[:, W:]
         x = ws.get("selective_x", (n, W), self.dtype)
         ops.conv_act(x, raw, self.conv, self.conv_bias, own.state, own.offset + N * W, ctx)
-        low = ws.get("selective_low", (n, self.rank + 2 * N), torch.float32)
+        low = ws.get("selective_low", (n, self.low_stride), torch.float32)[:, :self.rank + 2 * N]
         linear(x, self.x_weight, None, out=low)
         y = ws.get("selective_out", (n, W), self.dtype)
         # (the walk also keeps the step's last rows of x in the slot's ring: the convolution, which reads the ring, has run)

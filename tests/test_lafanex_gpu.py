@@ -421,19 +421,22 @@ def test_the_selective_scan_carries_a_token_far_and_forgets_at_once():
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("n,C,rank", [(1, 37, 3), (33, 64, 16), (130, 100, 5), (200, 96, 48), (65, 31, 8)])
+@pytest.mark.parametrize("n,C,rank", [(1, 37, 3), (33, 64, 16), (130, 100, 5), (200, 96, 48), (65, 31, 8), (70, 50, 100)])
 def test_step_sizes_keep_their_digits(dtype, n, C, rank):
     """softplus of the product with unrounded rows, down to step sizes a millionth of one: relative to each one's own size."""
     from liyab_amd.kernels import lib
 
     rng = np.random.default_rng(n)
-    low = rand(rng, n, rank + 6).to(DEV)
-    w = rand(rng, C, rank, scale=rank ** -0.5).to(getattr(torch, dtype)).to(DEV)
+    ldw = -(-rank // 8) * 8
+    low = rand(rng, n, ldw + 4).to(DEV)
+    low[:, rank:] = float("nan")  # (what lies behind the rank is not looked at)
+    w = torch.zeros(C, ldw, dtype=getattr(torch, dtype), device=DEV)
+    w[:, :rank] = rand(rng, C, rank, scale=rank ** -0.5)
     bias = torch.linspace(-14.0, 25.0, C, device=DEV)
     dt = torch.empty(n, C, device=DEV)
-    lib.call("liyab_scan_steps", dt.data_ptr(), low.data_ptr(), rank + 6, w.data_ptr(), 1 if dtype == "bfloat16" else 0, bias.data_ptr(), n, C, rank,
+    lib.call("liyab_scan_steps", dt.data_ptr(), low.data_ptr(), ldw + 4, w.data_ptr(), ldw, 1 if dtype == "bfloat16" else 0, bias.data_ptr(), n, C, rank,
              torch.cuda.current_stream().cuda_stream)
-    want = plain.softplus(f64(low)[:, :rank] @ f64(w).T + f64(bias))
+    want = plain.softplus(f64(low)[:, :rank] @ f64(w)[:, :rank].T + f64(bias))
     assert (np.abs(f64(dt) - want) / want).max() < (2e-5 if dtype == "float32" else 1e-4)
 
 
