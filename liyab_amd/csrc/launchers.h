@@ -127,7 +127,7 @@ int liyab_token_shift(void* out, int dtype, const void* h, const float* mu, int 
                       hipStream_t stream);
 int liyab_conv_act(void* out, int out_dtype, int64_t ldo, const float* in, int64_t ldi, const float* w, const float* bias, int taps, const float* state,
                    int64_t state_stride, int n_slots, const int* tok_seq, const int* positions, const int* seq_starts,
-                   const int* state_slots, int n, int C, int act, hipStream_t stream);
+                   const int* state_slots, int n, int C, int act, int portions, hipStream_t stream);
 int liyab_gated_group_norm(void* out, int out_dtype, const float* y, int64_t ldy, const float* z, int64_t ldz, const float* w, float eps,
                            int n, int inner, int groups, hipStream_t stream);
 int liyab_qk_prepare(const float* src, int64_t ld, int q_off, int k_off, int v_off, int H, int G, int dk, int dv, int dk_out, int dv_out,

@@ -885,16 +885,17 @@ extern "C" int liyab_token_shift(void* out, int dtype, const void* h, const floa
     return check_launch("token_shift");
 }
 
+// portions: whether the step holds more than single tokens (a hint: rows beside each other are then mostly one request's).
 extern "C" int liyab_conv_act(void* out, int out_dtype, int64_t ldo, const float* in, int64_t ldi, const float* w, const float* bias, int taps,
                               const float* state, int64_t state_stride, int n_slots, const int* tok_seq, const int* positions,
-                              const int* seq_starts, const int* state_slots, int n, int C, int act, hipStream_t stream) {
+                              const int* seq_starts, const int* state_slots, int n, int C, int act, int portions, hipStream_t stream) {
     LIYAB_REQUIRE(out && in && w && tok_seq && positions && seq_starts && state_slots, "conv_act: null pointer");
     LIYAB_REQUIRE(n >= 0 && n <= 65535 && C > 0 && taps >= 1 && ldo >= C && ldi >= C, "conv_act: bad sizes");
     LIYAB_REQUIRE(taps == 1 || (state != nullptr && n_slots > 0 && state_stride >= static_cast<int64_t>(taps - 1) * C),
                   "conv_act: %d taps need the last %d rows of a request in its slot", taps, taps - 1);
     if (n == 0) return 0;
     const auto aligned = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
-    if (n >= 64 && C % 4 == 0 && ldi % 4 == 0 && ldo % 4 == 0 && state_stride % 4 == 0 && aligned(in) && aligned(out) && aligned(bias) && aligned(state)) {
+    if (portions && n >= 64 && C % 4 == 0 && ldi % 4 == 0 && ldo % 4 == 0 && state_stride % 4 == 0 && aligned(in) && aligned(out) && aligned(bias) && aligned(state)) {
         const dim3 rows((C / 4 + 127) / 128, (n + CONV_TOKENS - 1) / CONV_TOKENS);
         const bool took = out_dtype == kF32
             ? launch_conv_rows<float>(taps, rows, stream, static_cast<float*>(out), ldo, in, ldi, w, bias, state, state_stride, n_slots, tok_seq, positions, seq_starts, state_slots, n, C, act)

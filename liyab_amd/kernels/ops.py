@@ -1541,7 +1541,7 @@ def conv_act(out: torch.Tensor, x: torch.Tensor, weight: torch.Tensor, bias: Opt
         slots, base = state.shape[0], state.data_ptr() + 4 * ring_off
     _step_lists(ctx, n)
     _lib.call("liyab_conv_act", out.data_ptr(), dtype_code(out.dtype), ldo, x.data_ptr(), ldi, weight.data_ptr(), _ptr(bias), taps, base, stride, slots,
-              ctx.tok_seq.data_ptr(), ctx.positions.data_ptr(), ctx.seq_starts.data_ptr(), ctx.state_slots.data_ptr(), n, C, 1 if act else 0,
+              ctx.tok_seq.data_ptr(), ctx.positions.data_ptr(), ctx.seq_starts.data_ptr(), ctx.state_slots.data_ptr(), n, C, 1 if act else 0, 0 if single_token_step(ctx) else 1,
               _stream())
 
 
