@@ -355,18 +355,22 @@ selective_single_kernel(SelectiveArgs a, const T* __restrict__ wt, const float* 
         }
     };
     states(n0);
+    const float z = a.z[t * a.ldz + cc], raw = a.places > 0 ? a.raw[t * a.ldr + cc] : 0.0f;
     // this wave's quarter of the rank; weights [rank, C], a row's channels side by side
     const int kq = (rank + 3) / 4, k1 = min(rank, (wave + 1) * kq);
     float acc = 0.0f;
-    int k = wave * kq;
-    for (; k + 8 <= k1; k += 8) {
-        float w[8];
+    for (int k = wave * kq; k < k1; k += 16) {  // sixteen weights and the row's numbers beside them are asked for together (past the quarter: its last, times zero)
+        float w[16], r[16];
 #pragma unroll
-        for (int j = 0; j < 8; ++j) w[j] = to_float<T>(wt[static_cast<int64_t>(k + j) * a.C + cc]);
+        for (int j = 0; j < 16; ++j) {
+            const int kk = min(k + j, k1 - 1);
+            w[j] = to_float<T>(wt[static_cast<int64_t>(kk) * a.C + cc]);
+            r[j] = row[kk];
+        }
+        settle_loads(w);
 #pragma unroll
-        for (int j = 0; j < 8; ++j) acc = fmaf(row[k + j], w[j], acc);
+        for (int j = 0; j < 16; ++j) acc = fmaf(k + j < k1 ? r[j] : 0.0f, w[j], acc);
     }
-    for (; k < k1; ++k) acc = fmaf(row[k], to_float<T>(wt[static_cast<int64_t>(k) * a.C + cc]), acc);
     part[wave][lane] = acc;
     __syncthreads();
     if (wave == 0) steps[lane] = ss_softplus((part[0][lane] + part[1][lane]) + (part[2][lane] + part[3][lane]) + bias[cc]);
@@ -389,8 +393,8 @@ selective_single_kernel(SelectiveArgs a, const T* __restrict__ wt, const float* 
     __syncthreads();
     if (wave == 0 && c_ok) {
         const float sum = (part[0][lane] + part[1][lane]) + (part[2][lane] + part[3][lane]);
-        static_cast<T*>(a.out)[t * a.C + c] = from_float<T>(fmaf(a.skip[c], x, sum) * ss_silu(a.z[t * a.ldz + c]));
-        if (slot_ok && a.places > 0) base[static_cast<int64_t>(a.N) * a.C + static_cast<int64_t>(pos % a.places) * a.C + c] = a.raw[t * a.ldr + c];
+        static_cast<T*>(a.out)[t * a.C + c] = from_float<T>(fmaf(a.skip[c], x, sum) * ss_silu(z));
+        if (slot_ok && a.places > 0) base[static_cast<int64_t>(a.N) * a.C + static_cast<int64_t>(pos % a.places) * a.C + c] = raw;
     }
 }
 
